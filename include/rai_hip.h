@@ -343,7 +343,8 @@ typedef enum rai_hip_arch {
   RAI_ARCH_PHI2 = 0,  /* rai-models/src/llm/phi2.rs */
   RAI_ARCH_QWEN2 = 1, /* rai-models/src/llm/qwen2.rs */
   RAI_ARCH_GEMMA = 2, /* rai-models/src/llm/gemma.rs */
-  RAI_ARCH_PHI3 = 3   /* rai-models/src/llm/phi3.rs: the Qwen2 block with fused qkv_proj / gate_up_proj, no biases */
+  RAI_ARCH_PHI3 = 3,  /* rai-models/src/llm/phi3.rs: the Qwen2 block with fused qkv_proj / gate_up_proj, no biases */
+  RAI_ARCH_LELITAR = 4 /* latent attention and a mixture of experts in a parallel block (rai_hip_decoder_create_latent) */
 } rai_hip_arch;
 
 /* Union of the serde Config structs phi2.rs:9-24, qwen2.rs:8-24, gemma.rs:12-27. */
@@ -382,6 +383,45 @@ typedef struct rai_hip_decoder rai_hip_decoder;
  * activation arena once; no allocation happens in forward afterwards. */
 int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_decoder **out);
 int rai_hip_decoder_destroy(rai_hip_decoder *dec);
+
+/* A decoder whose layers are described one by one (RAI_ARCH_LELITAR; no counterpart in the reference):
+ *   x <- x + residual_mult * (attention(norm1(x)) + mlp(norm2(x))),
+ * norms in `norm_groups` runs of the width, each divided by its own root mean square; residual stream in f32. */
+typedef enum rai_hip_mlp_kind { RAI_MLP_NONE = 0, RAI_MLP_DENSE = 1, RAI_MLP_MIXTURE = 2 } rai_hip_mlp_kind;
+typedef struct rai_hip_latent_layer {
+  /* Queries through a latent of q_rank values, keys and values from another of kv_rank values, both RMS-normed; no
+   * positional rotation. */
+  int32_t heads;
+  int32_t qk_dim;
+  int32_t v_dim;
+  int32_t q_rank;
+  int32_t kv_rank;
+  int32_t window; /* a token sees the last `window` positions including its own; 0: every earlier one */
+  /* down(act(gate x) * (up x)): one of `intermediate` values, or `experts` of them of which each token takes the `top`
+   * with the largest sigmoid router scores; the score multiplies the expert's input. */
+  int32_t mlp_kind; /* rai_hip_mlp_kind */
+  int32_t mlp_act;  /* RAI_UN_RELU / RAI_UN_SILU / RAI_UN_GELU / RAI_UN_NEW_GELU */
+  int32_t intermediate;
+  int32_t experts;
+  int32_t top;
+  double attn_scale;
+} rai_hip_latent_layer;
+typedef struct rai_hip_latent_config {
+  int32_t dtype; /* RAI_BF16 or RAI_F32 */
+  int32_t vocab_size;
+  int32_t width;
+  int32_t num_layers;
+  int32_t norm_groups;
+  int32_t max_batch;
+  int32_t max_context;
+  double norm_eps;
+  double residual_mult;
+} rai_hip_latent_config;
+/* Parameters are named "embed", "l<i>.norm1", "l<i>.mix.<dq|uq|dkv|uk|uv|g|o>", "l<i>.mix.<dq|dkv>.norm", "l<i>.norm2",
+ * "l<i>.mlp.<gate|up|down>" or "l<i>.mlp.e<k>.<gate|up|down>" and "l<i>.mlp.router", "final.norm", "head".  Sizes may be
+ * any positive numbers (weights are padded internally).  Every rai_hip_decoder_* call works on the result. */
+int rai_hip_decoder_create_latent(int dev, const rai_hip_latent_config *cfg, const rai_hip_latent_layer *layers,
+                                  rai_hip_decoder **out);
 /* Module::update_by_safetensors naming (rai-core/src/nn.rs:183-205, renames
  * phi2.rs:307-313): copy one named parameter from host memory, e.g.
  * "model.layers.3.self_attn.q_proj.weight".  `data` is row-major in the model dtype. */
@@ -425,6 +465,11 @@ int rai_hip_decoder_forward(rai_hip_decoder *dec, const uint32_t *ids_host, int3
 int rai_hip_decoder_forward_hidden(rai_hip_decoder *dec, const uint32_t *ids_host, const void *hidden_in_host,
                                    int32_t batch, int32_t seq, float *hidden_out_host, float *logits_host,
                                    uint32_t *tokens_host);
+/* rai_hip_decoder_forward for callers that need the logits of chosen rows and no token: ids are appended after the cached
+ * context, and logits_host [n_rows, vocab] (f32) receives the logits of rows rows_host[i] = b * seq + s of this call's
+ * tokens (n_rows may be 0).  A prompt may be fed in portions of any size. */
+int rai_hip_decoder_forward_rows(rai_hip_decoder *dec, const uint32_t *ids_host, int32_t batch, int32_t seq,
+                                 const int32_t *rows_host, int32_t n_rows, float *logits_host);
 /* Greedy loop of examples/phi2/src/main.rs:75-95 without repeat penalty: prefill
  * prompt[batch*prompt_len], then n_new single-token steps feeding the device
  * argmax back without host round trips.  tokens_host[batch*n_new]. prefill_ms /

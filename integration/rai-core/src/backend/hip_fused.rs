@@ -99,6 +99,15 @@ impl Decoder {
         Self { h, vocab: cfg.vocab_size as usize }
     }
 
+    /// A latent-attention model (Lelitar), its layers described one by one.
+    pub fn create_latent(dev: c_int, cfg: &RaiHipLatentConfig, layers: &[RaiHipLatentLayer]) -> Self {
+        assert_eq!(layers.len(), cfg.num_layers as usize);
+        let mut h = std::ptr::null_mut();
+        check(unsafe { rai_hip_init(dev) });
+        check(unsafe { rai_hip_decoder_create_latent(dev, cfg, layers.as_ptr(), &mut h) });
+        Self { h, vocab: cfg.vocab_size as usize }
+    }
+
     /// `(name, element count)` of every parameter the driver expects.
     pub fn param_names(&self) -> Vec<(String, i64)> {
         let mut n = 0i32;
@@ -145,6 +154,17 @@ impl Decoder {
             rai_hip_decoder_forward(self.h, ids.as_ptr(), batch as i32, seq as i32, logits.as_mut_ptr(), toks.as_mut_ptr())
         });
         (logits, toks)
+    }
+
+    /// Appends ids `[batch, seq]` after the cached context; logits `[rows.len(), vocab]` of rows `b * seq + s`.
+    pub fn forward_rows(&self, ids: &[u32], batch: usize, seq: usize, rows: &[i32]) -> Vec<f32> {
+        assert_eq!(ids.len(), batch * seq);
+        let mut logits = vec![0f32; rows.len() * self.vocab];
+        check(unsafe {
+            rai_hip_decoder_forward_rows(self.h, ids.as_ptr(), batch as i32, seq as i32, rows.as_ptr(), rows.len() as i32,
+                                         logits.as_mut_ptr())
+        });
+        logits
     }
 
     /// The layer stack with both ends open: `rows` (`[batch * seq, hidden]` in the model dtype's storage form, as raw

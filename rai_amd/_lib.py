@@ -22,7 +22,8 @@ UNARY = {n: i for i, n in enumerate(
 BINARY = {n: i for i, n in enumerate(
     ["add", "sub", "mul", "div", "maximum", "minimum", "eq", "ne", "gt", "ge", "lt", "le"])}
 REDUCE = {"sum": 0, "max": 1, "min": 2}
-ARCH = {"phi2": 0, "qwen2": 1, "gemma": 2, "phi3": 3}
+ARCH = {"phi2": 0, "qwen2": 1, "gemma": 2, "phi3": 3, "lelitar": 4}
+MLP_KIND = {"none": 0, "dense": 1, "moe": 2}
 
 
 class RaiHipError(RuntimeError):
@@ -64,6 +65,16 @@ class DecoderConfig(C.Structure):
         ("rope_theta", C.c_double),
         ("norm_eps", C.c_double),
     ]
+
+
+class LatentLayer(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "qk_dim", "v_dim", "q_rank", "kv_rank", "window", "mlp_kind", "mlp_act",
+                                         "intermediate", "experts", "top")] + [("attn_scale", C.c_double)]
+
+
+class LatentConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("dtype", "vocab_size", "width", "num_layers", "norm_groups", "max_batch",
+                                         "max_context")] + [("norm_eps", C.c_double), ("residual_mult", C.c_double)]
 
 
 _TP = C.POINTER(TensorDesc)
@@ -118,6 +129,7 @@ PROTOTYPES = {
     "rai_hip_rope_tables": [C.c_int, _dbl, _i32, _i32, _TP, _TP],
     "rai_hip_attention": [C.c_int, _TP, _TP, _TP, _dbl, _i32, _i32, _TP],
     "rai_hip_decoder_create": [C.c_int, C.POINTER(DecoderConfig), C.POINTER(_vp)],
+    "rai_hip_decoder_create_latent": [C.c_int, C.POINTER(LatentConfig), C.POINTER(LatentLayer), C.POINTER(_vp)],
     "rai_hip_decoder_destroy": [_vp],
     "rai_hip_decoder_load_param": [_vp, C.c_char_p, _vp, C.c_size_t],
     "rai_hip_decoder_load_safetensors": [_vp, C.POINTER(C.c_char_p), _i32],
@@ -129,6 +141,7 @@ PROTOTYPES = {
     "rai_hip_decoder_forward": [_vp, C.POINTER(C.c_uint32), _i32, _i32, C.POINTER(C.c_float), C.POINTER(C.c_uint32)],
     "rai_hip_decoder_forward_hidden": [_vp, C.POINTER(C.c_uint32), _vp, _i32, _i32, C.POINTER(C.c_float), C.POINTER(C.c_float),
                                        C.POINTER(C.c_uint32)],
+    "rai_hip_decoder_forward_rows": [_vp, C.POINTER(C.c_uint32), _i32, _i32, C.POINTER(_i32), _i32, C.POINTER(C.c_float)],
     "rai_hip_decoder_generate": [_vp, C.POINTER(C.c_uint32), _i32, _i32, _i32, C.POINTER(C.c_uint32),
                                  C.POINTER(C.c_float), C.POINTER(C.c_float)],
     "rai_hip_decoder_generate_sampled": [_vp, C.POINTER(C.c_uint32), _i32, _i32, _i32, C.c_float, _i32, _i64,

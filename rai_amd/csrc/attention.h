@@ -23,6 +23,12 @@ struct AttnArgs {
   // the capacity bound.
   const int *t_dev;
   int t_add;
+  // > 0 (with causal): a sliding window, the query at position p sees keys p - window + 1 .. p only.
+  int window;
+  // Optional output gate (f32_scores form only): feature d of head h of row (b, s) is multiplied by
+  // sigmoid(gate[(b*S + s)*gate_row_stride + h*D + d]).
+  const void *gate;
+  int64_t gate_row_stride;
 };
 
 int launch_attention(hipStream_t st, const AttnArgs &a);

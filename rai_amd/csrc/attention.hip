@@ -27,6 +27,8 @@ template <typename T> __device__ __forceinline__ float round_to(float x) {
 }
 template <> __device__ __forceinline__ float round_to<float>(float x) { return x; }
 
+__device__ __forceinline__ float gate_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
 template <typename T>
 __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
   constexpr int V = AttnVec<T>::V;
@@ -50,6 +52,7 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
   int t_end = a.causal ? (n_keys - a.S + s + 1) : n_keys;
   if (t_end > n_keys) t_end = n_keys;
   if (t_end < 0) t_end = 0;
+  const int t_begin = a.window > 0 && t_end > a.window ? t_end - a.window : 0;   // oldest key of the sliding window
 
   const T *q = (const T *)a.q + b * a.qs[0] + h * a.qs[1] + s * a.qs[2];
   const T *K = (const T *)a.k + b * a.ks[0] + hk * a.ks[1];
@@ -60,7 +63,7 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
   // ---- scores: 16 lanes cooperate on one key row
   {
     const int g = tid >> 4, gl = tid & 15;
-    for (int t = g; t < t_end; t += 16) {
+    for (int t = t_begin + g; t < t_end; t += 16) {
       const T *kr = K + (int64_t)t * a.ks[2];
       float acc = 0.f;
       for (int c = gl; c < ncol; c += 16) {
@@ -76,21 +79,22 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
         float sc;
         if (a.f32_scores) sc = acc * a.scale;
         else sc = round_to<T>(round_to<T>(acc) * round_to<T>(a.scale));
-        scores[t] = sc;
+        scores[t - t_begin] = sc;
       }
     }
   }
   __syncthreads();
 
-  // ---- softmax over scores[0..t_end)
+  // ---- softmax over the scores of keys [t_begin, t_end)
+  const int n_seen = t_end - t_begin;
   float m = -INFINITY;
-  for (int t = tid; t < t_end; t += 256) m = fmaxf(m, scores[t]);
+  for (int t = tid; t < n_seen; t += 256) m = fmaxf(m, scores[t]);
   m = wave_max(m);
   if (lane == 0) sh[wave] = m;
   __syncthreads();
   m = fmaxf(fmaxf(sh[0], sh[1]), fmaxf(sh[2], sh[3]));
   float sum = 0.f;
-  for (int t = tid; t < t_end; t += 256) {
+  for (int t = tid; t < n_seen; t += 256) {
     float e = expf(scores[t] - m);
     if (!a.f32_scores) e = round_to<T>(e);
     scores[t] = e;
@@ -111,10 +115,10 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
 #pragma unroll
     for (int j = 0; j < V; ++j) acc[j] = 0.f;
     if (grp < groups) {
-      for (int t = grp; t < t_end; t += groups) {
+      for (int t = grp; t < n_seen; t += groups) {
         // the reference rounds the normalised probabilities to V's dtype
         const float p = a.f32_scores ? round_to<T>(scores[t] * inv) : round_to<T>(scores[t] / sum);
-        APack<T, V> pk = *reinterpret_cast<const APack<T, V> *>(Vp + (int64_t)t * a.vs[2] + col * V);
+        APack<T, V> pk = *reinterpret_cast<const APack<T, V> *>(Vp + (int64_t)(t_begin + t) * a.vs[2] + col * V);
 #pragma unroll
         for (int j = 0; j < V; ++j) acc[j] = fmaf(p, (float)Scalar<T>::load(&pk.v[j]), acc[j]);
       }
@@ -127,6 +131,8 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
   for (int d = tid; d < D; d += 256) {
     float r = 0.f;
     for (int g = 0; g < groups; ++g) r += red[g * D + d];
+    if (a.gate)
+      r *= gate_sigmoid((float)Scalar<T>::load((const T *)a.gate + ((int64_t)b * a.S + s) * a.gate_row_stride + (int64_t)h * D + d));
     Scalar<T>::store(o + d, (typename Scalar<T>::compute)r);
   }
 }
@@ -842,7 +848,7 @@ template <typename T> static int launch_row(hipStream_t st, const AttnArgs &a) {
   constexpr int V = AttnVec<T>::V;
   RAI_REQUIRE(a.D % V == 0 && a.D / V <= 256, RAI_ERR_BAD_SHAPE, "attention: head_dim %d unsupported", a.D);
   const int ncol = a.D / V, groups = 256 / ncol;
-  const size_t lds = sizeof(float) * ((size_t)a.D + (size_t)groups * a.D + (size_t)a.T);
+  const size_t lds = sizeof(float) * ((size_t)a.D + (size_t)groups * a.D + (size_t)(a.window > 0 && a.window < a.T ? a.window : a.T));
   RAI_REQUIRE(lds <= 150 * 1024, RAI_ERR_UNSUPPORTED, "attention: context %d too long for the row kernel", a.T);
   static size_t attr_bytes = 0;
   if (lds > 64 * 1024 && lds > attr_bytes) {
@@ -918,6 +924,9 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
     int last_q = q0 + NW * 32 < a.S ? q0 + NW * 32 : a.S;
     kv_end = off + last_q < a.T ? off + last_q : a.T;
   }
+  // sliding window: the block's first query sets the oldest key tile any of its queries may see
+  const int first_key = a.window > 0 ? off + q0 - a.window + 1 : 0;
+  const int kv_begin = first_key > 0 ? first_key & ~63 : 0;
   const int wave_last_key = a.causal ? off + q0 + wave * 32 + 31 : a.T - 1;  // newest key any row of this wave may see
   const float scale_r = round_to<bf16_raw>(a.scale);
 
@@ -999,8 +1008,8 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
       store_v(i, x);
     }
   };
-  if (PF && kv_end > 0) load_tile(0);
-  for (int kb = 0; kb < kv_end; kb += 64 * KSP) {
+  if (PF && kv_end > 0) load_tile(kv_begin);
+  for (int kb = kv_begin; kb < kv_end; kb += 64 * KSP) {
     __syncthreads();
     // ---- stage K [64][D] and V^T [D][64], KSP tiles of each
     if (!PF) load_tile(kb);
@@ -1011,6 +1020,7 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
     const int k0 = kb + 64 * kh;       // this wave's tile of the round
     // every key of this tile is masked for this wave, or the tile lies behind the block's keys (barriers stay uniform)
     if (k0 > wave_last_key || k0 >= kv_end) continue;
+    if (a.window > 0 && k0 + 63 <= off + q0 + wave * 32 - a.window) continue;   // older than every query's window
     const uint16_t *const Kt = Ks + kh * KTILE, *const Vw = Vt + kh * VTILE;
 
     // ---- S^T tile: 64 keys x 32 queries
@@ -1029,7 +1039,8 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
     const int q_abs = off + qrow;
     // a tile wholly inside the context and (under a causal mask) wholly at or before this wave's first query
     // needs no masking
-    const bool masked = k0 + 63 >= a.T || (a.causal && k0 + 63 > off + q0 + wave * 32);
+    const bool masked = k0 + 63 >= a.T || (a.causal && k0 + 63 > off + q0 + wave * 32) ||
+                        (a.window > 0 && k0 <= off + q0 + wave * 32 + 31 - a.window);
     if constexpr (F32S) {
 #pragma unroll
       for (int u = 0; u < 2; ++u)
@@ -1053,6 +1064,13 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
       for (int u = 0; u < 2; ++u)
 #pragma unroll
         for (int r = 0; r < 16; ++r) sc[u][r] = u * 32 + 8 * (r >> 2) + (r & 3) > rel ? -INFINITY : sc[u][r];
+      if (a.window > 0) {
+        const int rel_lo = q_abs - a.window - k0 - 4 * half;   // newest key before this lane's window
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) sc[u][r] = u * 32 + 8 * (r >> 2) + (r & 3) <= rel_lo ? -INFINITY : sc[u][r];
+      }
     }
     float mx = -INFINITY;
 #pragma unroll
@@ -1154,12 +1172,21 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
   if (qrow < a.S) {
     const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
     uint16_t *op = (uint16_t *)a.out + ((int64_t)b * a.S + qrow) * a.out_row_stride + (int64_t)h * D;
+    const uint16_t *gp = a.gate ? (const uint16_t *)a.gate + ((int64_t)b * a.S + qrow) * a.gate_row_stride + (int64_t)h * D : nullptr;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         const int d = dt * 32 + 8 * g + 4 * half;
         if (d < D) {
+          if (gp) {
+            const fa_u32x2 gv = *reinterpret_cast<const fa_u32x2 *>(gp + d);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              const uint32_t wd = e < 2 ? gv.x : gv.y;
+              o[dt][4 * g + e] *= gate_sigmoid(__uint_as_float(e & 1 ? wd & 0xffff0000u : wd << 16));
+            }
+          }
           fa_u32x2 w;
           w.x = (uint32_t)f32_to_bf16_bits(o[dt][4 * g] * inv) | ((uint32_t)f32_to_bf16_bits(o[dt][4 * g + 1] * inv) << 16);
           w.y = (uint32_t)f32_to_bf16_bits(o[dt][4 * g + 2] * inv) | ((uint32_t)f32_to_bf16_bits(o[dt][4 * g + 3] * inv) << 16);
@@ -1193,7 +1220,8 @@ template <int D> static int launch_flash(hipStream_t st, const AttnArgs &a) {
 
 static bool flash_eligible(const AttnArgs &a) {
   if (a.dtype != RAI_BF16 || a.S < 16 || a.t_dev) return false;
-  if (a.D != 64 && a.D != 80 && a.D != 128 && a.D != 256) return false;
+  if (a.D != 32 && a.D != 64 && a.D != 80 && a.D != 128 && a.D != 192 && a.D != 256) return false;
+  if (a.gate && ((uintptr_t)a.gate % 8 || a.gate_row_stride % 4)) return false;
   auto al = [](const void *p, const int64_t *s) {
     return (uintptr_t)p % 16 == 0 && s[0] % 8 == 0 && s[1] % 8 == 0 && s[2] % 8 == 0;
   };
@@ -1206,11 +1234,15 @@ int launch_attention(hipStream_t st, const AttnArgs &a) {
               "attention: empty problem");
   RAI_REQUIRE(a.Hq % a.Hkv == 0, RAI_ERR_BAD_SHAPE, "attention: %d query heads not divisible by %d kv heads", a.Hq,
               a.Hkv);
+  RAI_REQUIRE(a.window >= 0 && (!a.window || a.causal) && (!a.gate || a.f32_scores), RAI_ERR_BAD_ARG,
+              "attention: a window needs the causal form, an output gate the f32-score form");
   if (flash_eligible(a)) {
     switch (a.D) {
+      case 32: return launch_flash<32>(st, a);
       case 64: return launch_flash<64>(st, a);
       case 80: return launch_flash<80>(st, a);
       case 128: return launch_flash<128>(st, a);
+      case 192: return launch_flash<192>(st, a);
       default: return launch_flash<256>(st, a);
     }
   }

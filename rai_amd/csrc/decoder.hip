@@ -16,95 +16,8 @@
 // device memory, so consecutive greedy steps need no host round trip.
 #include <algorithm>
 #include <cstdlib>
-#include <map>
-#include <string>
-#include <vector>
 
-#include "attention.h"
-#include "decode_chain.h"
-#include "decode_mega.h"
-#include "gemm.h"
-
-namespace rai {
-
-struct ParamSlot {
-  std::string name;
-  int64_t rows, cols;       // logical [rows, cols] (1-D params: rows = 1)
-  char *dst;                // device address of element [0, 0]
-  int64_t pitch;            // elements between consecutive rows at dst
-  bool loaded;
-  // a parameter whose last rows2 rows go elsewhere (same pitch): Phi-3's gate_up_proj, whose gate rows and
-  // up rows interleave in the packed matrix
-  int64_t rows2;
-  char *dst2;
-};
-
-struct Layer {
-  // Phi-2 (parallel block)
-  char *Wa, *ba, *Wb, *bd, *bf, *ln_w, *ln_b;
-  // Qwen2 / Gemma (sequential block): Wqkv [QD+2KD, H] (+bqkv), Wo [H, QD] (+bo),
-  // Wgu [2I, H] with gate/up rows interleaved, Wdown [H, I], two RMSNorm weights
-  char *Wqkv, *bqkv, *Wo, *bo, *Wgu, *Wdown, *n1_w, *n2_w;
-  // second copies in MFMA-fragment order for the batched-decode streaming kernel (built on first use)
-  char *Wa_f, *Wb_f, *Wqkv_f, *Wo_f, *Wgu_f, *Wdown_f;
-};
-
-}  // namespace rai
-
-using namespace rai;
-
-struct rai_hip_decoder {
-  int dev;
-  rai_hip_decoder_config cfg;
-  size_t es;
-  int H, I, QD, KD, D, Hq, Hkv, V, L, NA, KB;
-  std::vector<ParamSlot> slots;
-  std::map<std::string, int> slot_by_name;
-  std::vector<Layer> layers;
-  char *embed, *lnf_w, *lnf_b, *head_w, *head_b;
-  char *cos_t, *sin_t;  // [max_pos, rot] in the model dtype
-  char *kcache, *vcache;
-  // activations (sized for max_batch * max_context rows)
-  char *x, *x2, *ln, *qkv, *cat, *last, *logits;
-  char *attn, *glu;   // sequential block: attention output [rows, QD], gated MLP activation [rows, I]
-  char *attn_ws;      // partial results of the decode attention's context splits
-  int *attn_counters; // per (batch, head) arrival counters of those splits (zero between launches)
-  float embed_scale;  // Gemma: sqrt(hidden) rounded to the model dtype; 1 otherwise
-  uint32_t *ids, *tokens, *history;
-  char *splitk_ws;        // f32 scratch for prefill GEMMs that split K
-  size_t splitk_ws_bytes;
-  DevState *state;
-  std::vector<void *> allocs;
-  int ctx_len;
-  int64_t max_rows;
-  int history_cap;
-  // persistent per-token kernel (Phi-2, bf16, batch 1): per-layer pointer table, exchange packets
-  MegaLayer *mega_layers;
-  uint64_t *mega_xchg;    // packets exchanged between the blocks of the persistent decode kernel
-  unsigned long long *mega_prof;  // time stamps of the persistent kernel when RAI_HIP_MEGA_PROF is set
-  bool mega_ok;
-  int num_cu;
-  hipGraphExec_t step_graph;   // one captured single-token step (batch step_graph_batch)
-  hipGraphExec_t step_graph_n; // kGraphSteps consecutive single-token steps in one graph (same batch)
-  int step_graph_batch;
-  bool x_holds_next;          // d->x already holds the embedding of d->tokens
-  // token choice of the example loop (repeat penalty, last maximum wins) instead of plain greedy argmax
-  bool sample_on;
-  float sample_penalty;
-  int sample_last_n;
-  uint32_t *token_log;        // [max_batch][token_log_cap]: every token of each sequence so far, prompt first
-  int token_log_cap;
-  float *choice_val;          // [max_batch][kChoiceMaxSplits]: best value of each share of a wide logits row
-  uint32_t *choice_idx;       // and its index
-  unsigned long long *head_best;   // one (value, row) word per block of the head kernel that also chooses the token
-  char *hidden_copy;          // [max_rows, H]: the residual stream after the last layer, kept when a caller asks for it
-  bool want_hidden;           // the running forward copies its final residual stream to hidden_copy
-  char *head_f;               // fragment-order copy of the lm_head matrix
-  bool frag_ready;            // the fragment-order copies match the loaded parameters
-  bool graph_sampled;         // what the cached step graphs were captured with
-  float graph_penalty;
-  int graph_last_n;
-};
+#include "decoder.h"
 
 namespace rai {
 
@@ -476,13 +389,19 @@ __global__ void __launch_bounds__(256) k_to_f32(float *out, const T *in, int64_t
     out[i] = (float)Scalar<T>::load(in + i);
 }
 
+template <typename T>
+__global__ void __launch_bounds__(256) k_pick_rows(T *out, const T *in, const int *rows, int n, int H) {
+  for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < (int64_t)n * H; i += (int64_t)gridDim.x * blockDim.x)
+    out[i] = in[(int64_t)rows[i / H] * H + i % H];
+}
+
 static int grid1d(int64_t n) {
   int64_t b = (n + 255) / 256;
   return (int)(b < kNumCU * 16 ? (b < 1 ? 1 : b) : kNumCU * 16);
 }
 
 // ------------------------------------------------------------------ host-side construction
-static int dalloc(rai_hip_decoder *d, size_t bytes, char **out) {
+int dalloc(rai_hip_decoder *d, size_t bytes, char **out) {
   void *p = nullptr;
   RAI_HIP_TRY(hipSetDevice(d->dev));
   hipError_t e = hipMalloc(&p, bytes ? bytes : 16);
@@ -492,14 +411,14 @@ static int dalloc(rai_hip_decoder *d, size_t bytes, char **out) {
   return RAI_OK;
 }
 
-static void add_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch) {
+void add_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch) {
   d->slot_by_name[name] = (int)d->slots.size();
-  d->slots.push_back(ParamSlot{name, rows, cols, dst, pitch, false, 0, nullptr});
+  d->slots.push_back(ParamSlot{name, rows, cols, dst, pitch, false, 0, nullptr, 0, 0, 0, 0});
 }
 static void add_split_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch,
                            int64_t rows2, char *dst2) {
   d->slot_by_name[name] = (int)d->slots.size();
-  d->slots.push_back(ParamSlot{name, rows, cols, dst, pitch, false, rows2, dst2});
+  d->slots.push_back(ParamSlot{name, rows, cols, dst, pitch, false, rows2, dst2, 0, 0, 0, 0});
 }
 
 // Rotary tables.  Reference chain (phi2.rs:44-64): inv_freq computed with f32
@@ -687,6 +606,10 @@ template <typename T> static void launch_embed(rai_hip_decoder *d, hipStream_t s
   hipLaunchKernelGGL((k_embed<T>), dim3(grid1d(rows * d->H)), dim3(256), 0, st, (T *)d->x, (const T *)d->embed, d->ids,
                      rows, d->H, d->V, index_error_counter(d->dev), d->embed_scale);
 }
+int decoder_embed(rai_hip_decoder *d, hipStream_t st, int64_t rows) {
+  if (d->cfg.dtype == RAI_BF16) launch_embed<bf16_raw>(d, st, rows); else launch_embed<float>(d, st, rows);
+  return launch_check("embed");
+}
 template <typename T> static void launch_rope_append(rai_hip_decoder *d, hipStream_t st, int l, int B, int S) {
   const size_t per_layer = (size_t)d->cfg.max_batch * d->Hkv * d->cfg.max_context * d->D;
   int64_t total = (int64_t)B * S * (d->Hq + 2 * d->Hkv) * d->D;
@@ -726,7 +649,7 @@ static rai_hip_tensor desc1(void *p, int dtype, int64_t n) {
   return t;
 }
 
-static int linear(rai_hip_decoder *d, hipStream_t st, const LinearArgs &a0) {
+int decoder_linear(rai_hip_decoder *d, hipStream_t st, const LinearArgs &a0) {
   LinearArgs a = a0;
   a.dev = d->dev;
   return d->cfg.dtype == RAI_BF16 ? launch_linear_bf16(st, a) : launch_linear_f32(st, a);
@@ -797,7 +720,7 @@ constexpr int64_t kSampleMaxVocab = 15 * 1024 * 32;  // the membership bitmap of
 
 // Chooses the next token of every sequence from d->logits: plain greedy argmax, or the example loop's
 // choice when the decoder is in sampling mode.
-static int launch_token_choice(rai_hip_decoder *d, hipStream_t st, int B, int S, bool advance_step) {
+int launch_token_choice(rai_hip_decoder *d, hipStream_t st, int B, int S, bool advance_step) {
   const int dt = d->cfg.dtype;
   uint32_t *hist = advance_step ? d->history : nullptr;
   const int dstep = advance_step ? 1 : 0;
@@ -850,8 +773,7 @@ static int forward_phi2(rai_hip_decoder *d, int B, int S, bool advance_step, boo
   if (frag) RAI_TRY(ensure_fragments(d, st));
 
   if (!from_tokens) {
-    if (dt == RAI_BF16) launch_embed<bf16_raw>(d, st, M); else launch_embed<float>(d, st, M);
-    RAI_TRY(launch_check("embed"));
+    RAI_TRY(decoder_embed(d, st, M));
   }
 
   char *x = d->x, *xn = d->x2;
@@ -883,7 +805,7 @@ static int forward_phi2(rai_hip_decoder *d, int B, int S, bool advance_step, boo
     a.out2 = d->cat + (size_t)QD * d->es; a.ld2 = d->KB;
     a.M = (int)M; a.N = d->NA; a.K = H; a.n_split = ldq;
     a.act = d->cfg.hidden_act; a.act_from = ldq;
-    RAI_TRY(linear(d, st, a));
+    RAI_TRY(decoder_linear(d, st, a));
 
     const size_t per_layer = (size_t)d->cfg.max_batch * d->Hkv * d->cfg.max_context * d->D;
     if (S == 1) {
@@ -939,7 +861,7 @@ static int forward_phi2(rai_hip_decoder *d, int B, int S, bool advance_step, boo
       ln_ready = linear_fuses_post_norm(b);
       if (!ln_ready) b.post_ln_out = nullptr;
     }
-    RAI_TRY(linear(d, st, b));
+    RAI_TRY(decoder_linear(d, st, b));
     char *tmp = x; x = xn; xn = tmp;
   }
 
@@ -988,7 +910,7 @@ static int forward_phi2(rai_hip_decoder *d, int B, int S, bool advance_step, boo
       return RAI_OK;
     }
   }
-  RAI_TRY(linear(d, st, h));
+  RAI_TRY(decoder_linear(d, st, h));
 
   RAI_TRY(launch_token_choice(d, st, B, S, advance_step));
   d->ctx_len = T_after;
@@ -1026,8 +948,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
   if (frag) RAI_TRY(ensure_fragments(d, st));
 
   if (!from_tokens) {
-    if (dt == RAI_BF16) launch_embed<bf16_raw>(d, st, M); else launch_embed<float>(d, st, M);
-    RAI_TRY(launch_check("embed"));
+    RAI_TRY(decoder_embed(d, st, M));
   }
   auto norm_rows = [&](char *src, char *w, char *dst, int64_t rows, int64_t src_stride) -> int {
     rai_hip_tensor tx = desc2(src, dt, rows, H, src_stride), tw = desc1(w, dt, H), to = desc2(dst, dt, rows, H, H);
@@ -1068,7 +989,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
     a.out1 = d->qkv; a.ld1 = ldq;
     a.M = (int)M; a.N = ldq; a.K = H; a.n_split = ldq;
     a.splitk_ws = d->splitk_ws; a.splitk_ws_bytes = d->splitk_ws_bytes;
-    RAI_TRY(linear(d, st, a));
+    RAI_TRY(decoder_linear(d, st, a));
     }
 
     if (S == 1) {
@@ -1172,7 +1093,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
     o.out1 = x1; o.ld1 = H;
     o.M = (int)M; o.N = H; o.K = QD; o.n_split = H;
     o.splitk_ws = d->splitk_ws; o.splitk_ws_bytes = d->splitk_ws_bytes;
-    RAI_TRY(linear(d, st, o));
+    RAI_TRY(decoder_linear(d, st, o));
 
     LinearArgs g = linear_args_default();
     g.splitk_ws = d->splitk_ws; g.splitk_ws_bytes = d->splitk_ws_bytes;
@@ -1188,7 +1109,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
     g.out1 = d->glu; g.ld1 = I;
     g.M = (int)M; g.N = 2 * I; g.K = H; g.n_split = 2 * I;
     g.act = d->cfg.hidden_act; g.act_from = 0; g.glu = 1;
-    RAI_TRY(linear(d, st, g));
+    RAI_TRY(decoder_linear(d, st, g));
 
     LinearArgs dn = linear_args_default();
     dn.A = d->glu; dn.lda = I;
@@ -1198,7 +1119,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
     dn.out1 = x; dn.ld1 = H;
     dn.M = (int)M; dn.N = H; dn.K = I; dn.n_split = H;
     dn.splitk_ws = d->splitk_ws; dn.splitk_ws_bytes = d->splitk_ws_bytes;
-    RAI_TRY(linear(d, st, dn));
+    RAI_TRY(decoder_linear(d, st, dn));
   }
 
   if (d->want_hidden) RAI_HIP_TRY(hipMemcpyAsync(d->hidden_copy, x, (size_t)M * H * d->es, hipMemcpyDeviceToDevice, st));
@@ -1219,7 +1140,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
   }
   h.out1 = d->logits; h.ld1 = d->V;
   h.M = B; h.N = d->V; h.K = H; h.n_split = d->V;
-  RAI_TRY(linear(d, st, h));
+  RAI_TRY(decoder_linear(d, st, h));
 
   RAI_TRY(launch_token_choice(d, st, B, S, advance_step));
   d->ctx_len = T_after;
@@ -1227,6 +1148,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
 }
 
 static int forward_any(rai_hip_decoder *d, int B, int S, bool advance_step, bool from_tokens = false) {
+  if (d->latent) return forward_latent(d, B, S, advance_step, from_tokens);
   return d->cfg.arch == RAI_ARCH_PHI2 ? forward_phi2(d, B, S, advance_step, from_tokens)
                                        : forward_seq(d, B, S, advance_step, from_tokens);
 }
@@ -1315,12 +1237,76 @@ static int check_call(rai_hip_decoder *d, int B, int S) {
   return RAI_OK;
 }
 
+void decoder_init_fields(rai_hip_decoder *d, int dev, const rai_hip_decoder_config &cfg0) {
+  d->dev = dev;
+  d->cfg = cfg0;
+  const rai_hip_decoder_config *cfg = &d->cfg;
+  d->es = dtype_size(cfg->dtype);
+  d->H = cfg->hidden_size; d->I = cfg->intermediate_size; d->D = cfg->head_dim;
+  d->Hq = cfg->num_attention_heads; d->Hkv = cfg->num_key_value_heads;
+  d->QD = d->Hq * d->D; d->KD = d->Hkv * d->D; d->V = cfg->vocab_size; d->L = cfg->num_hidden_layers;
+  d->NA = d->QD + 2 * d->KD + d->I;
+  d->KB = d->QD + d->I;
+  d->ctx_len = 0;
+  d->step_graph = nullptr;
+  d->step_graph_n = nullptr;
+  d->step_graph_batch = 0;
+  d->x_holds_next = false;
+  d->sample_on = false; d->sample_penalty = 0.f; d->sample_last_n = 0;
+  d->token_log = nullptr; d->token_log_cap = 0;
+  d->graph_sampled = false; d->graph_penalty = 0.f; d->graph_last_n = 0;
+  d->head_f = nullptr; d->frag_ready = false;
+  d->hidden_copy = nullptr; d->want_hidden = false;
+  d->choice_val = nullptr; d->choice_idx = nullptr; d->head_best = nullptr;
+  d->mega_layers = nullptr;
+  d->mega_ok = false;
+  d->mega_prof = nullptr;
+  d->mega_xchg = nullptr;
+  d->latent = nullptr;
+  d->max_rows = (int64_t)cfg->max_batch * cfg->max_context;
+  d->history_cap = cfg->max_context;
+  hipDeviceProp_t prop;
+  d->num_cu = hipGetDeviceProperties(&prop, dev) == hipSuccess ? prop.multiProcessorCount : kNumCU;
+}
+
+// Buffers every family has: ids, tokens and their history, the logits, the device state and the scratch of the token
+// choice and of the K-split products.
+int decoder_alloc_common(rai_hip_decoder *d) {
+  const auto *cfg = &d->cfg;
+  char *tmp = nullptr;
+  RAI_TRY(dalloc(d, d->max_rows * sizeof(uint32_t), &tmp));
+  d->ids = (uint32_t *)tmp;
+  RAI_TRY(dalloc(d, (size_t)cfg->max_batch * sizeof(uint32_t), &tmp));
+  d->tokens = (uint32_t *)tmp;
+  RAI_TRY(dalloc(d, (size_t)d->history_cap * cfg->max_batch * sizeof(uint32_t), &tmp));
+  d->history = (uint32_t *)tmp;
+  d->token_log_cap = cfg->max_context + 1;
+  RAI_TRY(dalloc(d, (size_t)d->token_log_cap * cfg->max_batch * sizeof(uint32_t), &tmp));
+  d->token_log = (uint32_t *)tmp;
+  RAI_TRY(dalloc(d, sizeof(DevState), &tmp));
+  d->state = (DevState *)tmp;
+  d->splitk_ws_bytes = (size_t)12 * d->max_rows * d->H * sizeof(float);
+  if (d->splitk_ws_bytes > ((size_t)256 << 20)) d->splitk_ws_bytes = (size_t)256 << 20;
+  // the stream-K form of the tile kernel (prefill products of 136 tiles and more) parks partial tiles here
+  if (cfg->dtype == RAI_BF16 && d->max_rows >= 256 && d->splitk_ws_bytes < ((size_t)192 << 20))
+    d->splitk_ws_bytes = (size_t)192 << 20;
+  RAI_TRY(dalloc(d, d->splitk_ws_bytes, &d->splitk_ws));
+  RAI_TRY(dalloc(d, (size_t)cfg->max_batch * kChoiceMaxSplits * sizeof(float), &tmp));
+  d->choice_val = (float *)tmp;
+  RAI_TRY(dalloc(d, (size_t)cfg->max_batch * kChoiceMaxSplits * sizeof(uint32_t), &tmp));
+  d->choice_idx = (uint32_t *)tmp;
+  RAI_TRY(dalloc(d, (size_t)cfg->max_batch * d->V * d->es, &d->logits));
+  RAI_HIP_TRY(hipMemset(d->state, 0, sizeof(DevState)));
+  return RAI_OK;
+}
+
 }  // namespace rai
 
 extern "C" {
 
 int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_decoder **out) {
   RAI_REQUIRE(cfg && out, RAI_ERR_BAD_ARG, "decoder_create: null argument");
+  RAI_REQUIRE(cfg->arch != RAI_ARCH_LELITAR, RAI_ERR_UNSUPPORTED, "decoder_create: this architecture is built by decoder_create_latent");
   RAI_REQUIRE(cfg->arch == RAI_ARCH_PHI2 || cfg->arch == RAI_ARCH_QWEN2 || cfg->arch == RAI_ARCH_GEMMA ||
                   cfg->arch == RAI_ARCH_PHI3,
               RAI_ERR_UNSUPPORTED, "decoder_create: architecture %d not available", cfg->arch);
@@ -1339,25 +1325,7 @@ int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_d
               "decoder_create: qk_layernorm (rai-models/src/llm/phi2.rs:207-216) is not implemented by the decoder drivers");
   if (!ctx(dev)) return RAI_ERR_HIP;
   rai_hip_decoder *d = new rai_hip_decoder();
-  d->dev = dev;
-  d->cfg = *cfg;
-  d->es = dtype_size(cfg->dtype);
-  d->H = cfg->hidden_size; d->I = cfg->intermediate_size; d->D = cfg->head_dim;
-  d->Hq = cfg->num_attention_heads; d->Hkv = cfg->num_key_value_heads;
-  d->QD = d->Hq * d->D; d->KD = d->Hkv * d->D; d->V = cfg->vocab_size; d->L = cfg->num_hidden_layers;
-  d->NA = d->QD + 2 * d->KD + d->I;
-  d->KB = d->QD + d->I;
-  d->ctx_len = 0;
-  d->step_graph = nullptr;
-  d->step_graph_n = nullptr;
-  d->step_graph_batch = 0;
-  d->x_holds_next = false;
-  d->sample_on = false; d->sample_penalty = 0.f; d->sample_last_n = 0;
-  d->token_log = nullptr; d->token_log_cap = 0;
-  d->graph_sampled = false; d->graph_penalty = 0.f; d->graph_last_n = 0;
-  d->head_f = nullptr; d->frag_ready = false;
-  d->hidden_copy = nullptr; d->want_hidden = false;
-  d->choice_val = nullptr; d->choice_idx = nullptr; d->head_best = nullptr;
+  decoder_init_fields(d, dev, *cfg);
   const int vec = (int)(16 / d->es);
   int st = RAI_OK;
   auto bail = [&](int code) {
@@ -1370,57 +1338,26 @@ int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_d
   if (cfg->arch == RAI_ARCH_GEMMA) d->embed_scale = round_dt((float)sqrt((double)d->H), cfg->dtype);
   if ((st = (cfg->arch == RAI_ARCH_PHI2 ? create_phi2(d) : create_seq(d))) != RAI_OK) return bail(st);
   const size_t es = d->es;
-  d->max_rows = (int64_t)cfg->max_batch * cfg->max_context;
   const size_t kv = (size_t)d->L * cfg->max_batch * d->Hkv * cfg->max_context * d->D * es;
   const size_t rope = (size_t)cfg->max_position_embeddings * cfg->rotary_dim * es;
-  d->history_cap = cfg->max_context;
   char *tmp = nullptr;
+  if ((st = decoder_alloc_common(d))) return bail(st);
   if ((st = dalloc(d, kv, &d->kcache)) || (st = dalloc(d, kv, &d->vcache)) || (st = dalloc(d, rope, &d->cos_t)) ||
       (st = dalloc(d, rope, &d->sin_t)) || (st = dalloc(d, d->max_rows * d->H * es, &d->x)) ||
       (st = dalloc(d, d->max_rows * d->H * es, &d->x2)) || (st = dalloc(d, d->max_rows * d->H * es, &d->ln)) ||
       (st = dalloc(d, d->max_rows * (d->QD + 2 * d->KD) * es, &d->qkv)) ||
       (st = dalloc(d, cfg->arch == RAI_ARCH_PHI2 ? d->max_rows * d->KB * es : 16, &d->cat)) ||
       (st = dalloc(d, cfg->arch == RAI_ARCH_PHI2 ? 16 : d->max_rows * d->QD * es, &d->attn)) ||
-      (st = dalloc(d, cfg->arch == RAI_ARCH_PHI2 ? 16 : d->max_rows * d->I * es, &d->glu)) || (st = dalloc(d, (size_t)cfg->max_batch * d->H * es, &d->last)) ||
-      (st = dalloc(d, (size_t)cfg->max_batch * d->V * es, &d->logits)))
+      (st = dalloc(d, cfg->arch == RAI_ARCH_PHI2 ? 16 : d->max_rows * d->I * es, &d->glu)) || (st = dalloc(d, (size_t)cfg->max_batch * d->H * es, &d->last)))
     return bail(st);
-  if ((st = dalloc(d, d->max_rows * sizeof(uint32_t), &tmp))) return bail(st);
-  d->ids = (uint32_t *)tmp;
-  if ((st = dalloc(d, (size_t)cfg->max_batch * sizeof(uint32_t), &tmp))) return bail(st);
-  d->tokens = (uint32_t *)tmp;
-  if ((st = dalloc(d, (size_t)d->history_cap * cfg->max_batch * sizeof(uint32_t), &tmp))) return bail(st);
-  d->history = (uint32_t *)tmp;
-  d->token_log_cap = cfg->max_context + 1;
-  if ((st = dalloc(d, (size_t)d->token_log_cap * cfg->max_batch * sizeof(uint32_t), &tmp))) return bail(st);
-  d->token_log = (uint32_t *)tmp;
-  if ((st = dalloc(d, sizeof(DevState), &tmp))) return bail(st);
-  d->state = (DevState *)tmp;
-  d->splitk_ws_bytes = (size_t)12 * d->max_rows * d->H * sizeof(float);
-  if (d->splitk_ws_bytes > ((size_t)256 << 20)) d->splitk_ws_bytes = (size_t)256 << 20;
-  // the stream-K form of the tile kernel (prefill products of 136 tiles and more) parks partial tiles here
-  if (cfg->dtype == RAI_BF16 && d->max_rows >= 256 && d->splitk_ws_bytes < ((size_t)192 << 20))
-    d->splitk_ws_bytes = (size_t)192 << 20;
-  if ((st = dalloc(d, d->splitk_ws_bytes, &d->splitk_ws))) return bail(st);
   if ((st = dalloc(d, attention_decode_ws_bytes(cfg->max_batch, d->Hq, d->D), &d->attn_ws))) return bail(st);
   if ((st = dalloc(d, attention_decode_counter_bytes(cfg->max_batch, d->Hq), &tmp))) return bail(st);
   d->attn_counters = (int *)tmp;
-  if ((st = dalloc(d, (size_t)cfg->max_batch * kChoiceMaxSplits * sizeof(float), &tmp))) return bail(st);
-  d->choice_val = (float *)tmp;
-  if ((st = dalloc(d, (size_t)cfg->max_batch * kChoiceMaxSplits * sizeof(uint32_t), &tmp))) return bail(st);
-  d->choice_idx = (uint32_t *)tmp;
   if ((st = dalloc(d, 256 * sizeof(unsigned long long), &tmp))) return bail(st);
   d->head_best = (unsigned long long *)tmp;
   if (hipMemset(d->attn_counters, 0, attention_decode_counter_bytes(cfg->max_batch, d->Hq)) != hipSuccess)
     return bail(fail(RAI_ERR_HIP, "decoder_create: memset failed"));
 
-  d->mega_layers = nullptr;
-  d->mega_ok = false;
-  d->mega_prof = nullptr;
-  {
-    hipDeviceProp_t prop;
-    d->num_cu = hipGetDeviceProperties(&prop, dev) == hipSuccess ? prop.multiProcessorCount : kNumCU;
-  }
-  d->mega_xchg = nullptr;
   if (cfg->arch == RAI_ARCH_PHI2 && cfg->dtype == RAI_BF16 && getenv("RAI_HIP_NO_MEGA") == nullptr) {
     {  // zeroed: tag 0 is never a valid exchange tag
       // x and q|k|v: two values to a packet; activations: 16 packets for each of up to 256 producers;
@@ -1448,8 +1385,7 @@ int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_d
     MegaArgs m = mega_args(d);
     d->mega_ok = mega_eligible(m, d->D, d->num_cu, nullptr);
   }
-  if (hipMemset(d->state, 0, sizeof(DevState)) != hipSuccess || hipMemset(d->kcache, 0, kv) != hipSuccess ||
-      hipMemset(d->vcache, 0, kv) != hipSuccess)
+  if (hipMemset(d->kcache, 0, kv) != hipSuccess || hipMemset(d->vcache, 0, kv) != hipSuccess)
     return bail(fail(RAI_ERR_HIP, "decoder_create: memset failed"));
   if ((st = build_rope_tables(d)) != RAI_OK) return bail(st);
   *out = d;
@@ -1463,6 +1399,7 @@ int rai_hip_decoder_destroy(rai_hip_decoder *d) {
   if (d->step_graph) (void)hipGraphExecDestroy(d->step_graph);
   if (d->step_graph_n) (void)hipGraphExecDestroy(d->step_graph_n);
   for (void *p : d->allocs) (void)hipFree(p);
+  delete d->latent;
   delete d;
   return RAI_OK;
 }
@@ -1499,12 +1436,24 @@ int rai_hip_decoder_load_param(rai_hip_decoder *d, const char *name, const void 
   RAI_HIP_TRY(hipSetDevice(d->dev));
   RAI_HIP_TRY(hipStreamSynchronize(stream_of(d->dev)));
   const size_t row_bytes = (size_t)s.cols * d->es, rows1 = (size_t)(s.rows - s.rows2);
+  if (s.row_group || s.col_group) {   // padded heads: one copy per (row group, column group)
+    const int64_t rg = s.row_group ? s.row_group : s.rows, cg = s.col_group ? s.col_group : s.cols;
+    for (int64_t r = 0; r < s.rows; r += rg)
+      for (int64_t c = 0; c < s.cols; c += cg)
+        RAI_HIP_TRY(hipMemcpy2D(s.dst + (size_t)((r / rg) * s.row_stride + (c / cg) * s.col_stride) * d->es, (size_t)s.pitch * d->es,
+                                (const char *)host_data + ((size_t)r * s.cols + c) * d->es, row_bytes, (size_t)cg * d->es,
+                                (size_t)rg, hipMemcpyHostToDevice));
+    s.loaded = true;
+    if (d->latent) d->latent->derived_ready = false;
+    return RAI_OK;
+  }
   RAI_HIP_TRY(hipMemcpy2D(s.dst, (size_t)s.pitch * d->es, host_data, row_bytes, row_bytes, rows1, hipMemcpyHostToDevice));
   if (s.rows2 > 0)
     RAI_HIP_TRY(hipMemcpy2D(s.dst2, (size_t)s.pitch * d->es, (const char *)host_data + rows1 * row_bytes, row_bytes, row_bytes,
                             (size_t)s.rows2, hipMemcpyHostToDevice));
   s.loaded = true;
   d->frag_ready = false;   // the fragment-order copies are rebuilt on the next batched decode step
+  if (d->latent) d->latent->derived_ready = false;
   return RAI_OK;
 }
 
@@ -1547,7 +1496,7 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
   RAI_TRY(check_call(d, batch, seq));
   hipStream_t st = stream_of(d->dev);
   const size_t rows_bytes = (size_t)batch * seq * d->H * d->es;
-  if (hidden_out_host && !d->hidden_copy) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
+  if (hidden_out_host && !d->hidden_copy && !d->latent) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
   if (ids_host) {
     RAI_HIP_TRY(hipMemcpyAsync(d->ids, ids_host, (size_t)batch * seq * sizeof(uint32_t), hipMemcpyHostToDevice, st));
   } else {
@@ -1559,7 +1508,8 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
   d->want_hidden = false;
   d->x_holds_next = false;
   RAI_TRY(rc);
-  if (hidden_out_host) RAI_TRY(widen_to_host(d, st, d->hidden_copy, (int64_t)batch * seq * d->H, hidden_out_host));
+  if (hidden_out_host && d->latent) RAI_TRY(latent_hidden_to_host(d, (int64_t)batch * seq, hidden_out_host));
+  else if (hidden_out_host) RAI_TRY(widen_to_host(d, st, d->hidden_copy, (int64_t)batch * seq * d->H, hidden_out_host));
   if (logits_host) RAI_TRY(widen_to_host(d, st, d->logits, (int64_t)batch * d->V, logits_host));
   if (tokens_host) RAI_TRY(rai_hip_d2h(d->dev, tokens_host, d->tokens, (size_t)batch * sizeof(uint32_t)));
   if (hidden_out_host || logits_host || tokens_host) {
@@ -1568,6 +1518,75 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
     RAI_TRY(rai_hip_index_errors(d->dev, &bad));
     RAI_REQUIRE(bad == 0, RAI_ERR_INDEX, "decoder: %llu token ids outside the vocabulary", (unsigned long long)bad);
   }
+  return RAI_OK;
+}
+
+// Logits of n rows of the residual stream that the last forward left in hidden_copy (rows: device indices).
+static int head_rows(rai_hip_decoder *d, hipStream_t st, const int *rows_dev, int n, char *gathered, char *logits) {
+  if (d->latent) return latent_head_rows(d, st, rows_dev, n, logits);
+  const int dt = d->cfg.dtype, H = d->H;
+  if (dt == RAI_BF16)
+    hipLaunchKernelGGL((k_pick_rows<bf16_raw>), dim3(grid1d((int64_t)n * H)), dim3(256), 0, st, (bf16_raw *)gathered,
+                       (const bf16_raw *)d->hidden_copy, rows_dev, n, H);
+  else
+    hipLaunchKernelGGL((k_pick_rows<float>), dim3(grid1d((int64_t)n * H)), dim3(256), 0, st, (float *)gathered,
+                       (const float *)d->hidden_copy, rows_dev, n, H);
+  RAI_TRY(launch_check("pick_rows"));
+  rai_hip_tensor tx = desc2(gathered, dt, n, H, H), tw = desc1(d->lnf_w, dt, H), to = desc2(gathered + (size_t)n * H * d->es, dt, n, H, H);
+  if (d->cfg.arch == RAI_ARCH_PHI2) {
+    rai_hip_tensor tb = desc1(d->lnf_b, dt, H);
+    RAI_TRY(rai_hip_layer_norm(d->dev, &tx, &tw, &tb, d->cfg.norm_eps, &to));
+  } else {
+    RAI_TRY(rai_hip_rms_norm(d->dev, &tx, &tw, d->cfg.norm_eps, d->cfg.arch == RAI_ARCH_GEMMA, &to));
+  }
+  LinearArgs h = linear_args_default();
+  h.A = to.data; h.lda = H;
+  h.W = d->head_w; h.ldw = H; h.bias = d->head_b;
+  h.out1 = logits; h.ld1 = d->V;
+  h.M = n; h.N = d->V; h.K = H; h.n_split = d->V;
+  h.splitk_ws = d->splitk_ws; h.splitk_ws_bytes = d->splitk_ws_bytes;
+  return decoder_linear(d, st, h);
+}
+
+int rai_hip_decoder_forward_rows(rai_hip_decoder *d, const uint32_t *ids_host, int32_t batch, int32_t seq,
+                                 const int32_t *rows_host, int32_t n_rows, float *logits_host) {
+  RAI_REQUIRE(ids_host && n_rows >= 0 && (n_rows == 0 || (rows_host && logits_host)), RAI_ERR_BAD_ARG, "forward_rows: null argument");
+  RAI_TRY(check_call(d, batch, seq));
+  RAI_REQUIRE(n_rows <= batch * seq, RAI_ERR_BAD_ARG, "forward_rows: %d rows of %d tokens", n_rows, batch * seq);
+  for (int i = 0; i < n_rows; ++i)
+    RAI_REQUIRE(rows_host[i] >= 0 && rows_host[i] < batch * seq, RAI_ERR_BAD_ARG, "forward_rows: row %d outside this call's %d tokens",
+                rows_host[i], batch * seq);
+  hipStream_t st = stream_of(d->dev);
+  if (!d->hidden_copy && !d->latent && n_rows) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
+  RAI_HIP_TRY(hipMemcpyAsync(d->ids, ids_host, (size_t)batch * seq * sizeof(uint32_t), hipMemcpyHostToDevice, st));
+  d->want_hidden = n_rows > 0;
+  const int rc = forward_any(d, batch, seq, false);
+  d->want_hidden = false;
+  d->x_holds_next = false;
+  RAI_TRY(rc);
+  // in shares of the head product's rows, so that the logits of a long prompt need no large buffer
+  const int share = n_rows < 256 ? n_rows : 256;
+  if (n_rows) {
+    void *rows_dev = nullptr, *gathered = nullptr, *logits = nullptr;
+    int st_rc = rai_hip_alloc(d->dev, (size_t)n_rows * sizeof(int), &rows_dev);
+    if (st_rc == RAI_OK) st_rc = rai_hip_alloc(d->dev, (size_t)2 * share * d->H * d->es, &gathered);
+    if (st_rc == RAI_OK) st_rc = rai_hip_alloc(d->dev, (size_t)share * d->V * d->es, &logits);
+    if (st_rc == RAI_OK) st_rc = rai_hip_h2d(d->dev, rows_dev, rows_host, (size_t)n_rows * sizeof(int));
+    for (int i = 0; st_rc == RAI_OK && i < n_rows; i += share) {
+      const int n = n_rows - i < share ? n_rows - i : share;
+      st_rc = head_rows(d, st, (const int *)rows_dev + i, n, (char *)gathered, (char *)logits);
+      if (st_rc == RAI_OK) st_rc = widen_to_host(d, st, (const char *)logits, (int64_t)n * d->V, logits_host + (int64_t)i * d->V);
+    }
+    for (void *p : {rows_dev, gathered, logits})
+      if (p) (void)rai_hip_release(p);
+    RAI_TRY(st_rc);
+  } else {
+    RAI_TRY(rai_hip_sync(d->dev));
+  }
+  RAI_TRY(check_fault(d));
+  uint64_t bad = 0;
+  RAI_TRY(rai_hip_index_errors(d->dev, &bad));
+  RAI_REQUIRE(bad == 0, RAI_ERR_INDEX, "decoder: %llu token ids outside the vocabulary", (unsigned long long)bad);
   return RAI_OK;
 }
 

@@ -28,6 +28,11 @@ struct LinearArgs {
   int n_split;   // first column written to out2
   int act;       // rai_hip_unary_op activation or -1
   int act_from;  // activation applies to columns >= act_from
+  // != 0: residual (when given) and out1 are f32 whatever the operands' dtype, and out = residual + out_scale *
+  // act(acc + bias): a residual stream kept in f32 under bf16 products, or plain f32 results (router logits) without a
+  // residual.  One output, no gated pairs.
+  int f32_out;
+  float out_scale;
   // Gated MLP (rai-models/src/llm/qwen2.rs:100-104: act(gate(x)) * up(x)): W rows are
   // interleaved gate_0, up_0, gate_1, up_1, ...; N counts the interleaved rows and
   // N/2 columns are written to out1.  No residual, no output split.

@@ -10,6 +10,7 @@
 #include <cstdlib>
 
 #include "gemm.h"
+#include "latent.h"
 
 namespace rai {
 
@@ -167,7 +168,7 @@ __global__ void __launch_bounds__(NWV * 64) k_linear_bf16_skinny(LinearArgs a, i
       }
     }
     k0 += 64 * 8 * U;
-    const bool row_done = k0 >= K;
+    const bool row_done = k0 - lane * 8 >= K;   // the same for every lane, also where K ends inside the last 512
     const int n_cur = n_base;
     if (row_done) {
       n_base += R;
@@ -222,6 +223,10 @@ __global__ void __launch_bounds__(NWV * 64) k_linear_bf16_skinny(LinearArgs a, i
             if (m >= a.M) break;
             float v = acc[r][m] + bv;
             if (do_act) v = act_eval(a.act, v);
+            if (a.f32_out) {
+              ((float *)a.out1)[(int64_t)m * a.ld1 + n] = fmaf(a.out_scale, v, res ? ((const float *)a.residual)[(int64_t)m * a.ldr + n] : 0.f);
+              continue;
+            }
             if (res) v += bf16_bits_to_f32(res[(int64_t)m * a.ldr + n]);
             dst[(int64_t)m * ld + col] = f32_to_bf16_bits(v);
           }
@@ -364,6 +369,10 @@ __device__ __forceinline__ void gemv_reg_rows(const LinearArgs &a, int n_begin, 
         if (n >= n_end) break;
         float v = acc[r] + (bias ? bf16_bits_to_f32(bias[n]) : 0.f) + (bias2 ? bf16_bits_to_f32(bias2[n]) : 0.f);
         if (a.act >= 0 && n >= a.act_from) v = act_eval(a.act, v);
+        if (a.f32_out) {
+          ((float *)a.out1)[n] = fmaf(a.out_scale, v, res ? ((const float *)a.residual)[n] : 0.f);
+          continue;
+        }
         if (res) v += bf16_bits_to_f32(res[n]);
         if (n < a.n_split) ((uint16_t *)a.out1)[n] = f32_to_bf16_bits(v);
         else ((uint16_t *)a.out2)[n - a.n_split] = f32_to_bf16_bits(v);
@@ -396,7 +405,7 @@ __global__ void __launch_bounds__(256) k_gemv_bf16_reg_group(GemvGroupArgs g, in
   for (int i = 1; i < kGemvGroupMax; ++i)
     if (s == i) { a.W = g.W[i]; a.ldw = g.ldw[i]; a.bias = g.bias[i]; a.out1 = g.out[i]; a.N = g.N[i]; a.act = g.act[i]; base = g.wave_base[i]; }
   a.bias2 = nullptr; a.residual = nullptr; a.ldr = 0; a.ld1 = a.N; a.out2 = nullptr; a.ld2 = 0;
-  a.M = 1; a.K = g.K; a.n_split = a.N; a.act_from = 0; a.glu = 0;
+  a.M = 1; a.K = g.K; a.n_split = a.N; a.act_from = 0; a.glu = 0; a.f32_out = 0; a.out_scale = 1.f;
   a.ln_w = g.ln_w; a.ln_b = g.ln_b; a.ln_eps = g.ln_eps; a.ln_kind = g.ln_kind;
   a.A2 = nullptr; a.W2 = nullptr; a.ldw2 = 0; a.K2 = 0;
   gemv_reg_rows<KC, R>(a, (gw - base) * rows_per_wave, rows_per_wave);
@@ -404,13 +413,11 @@ __global__ void __launch_bounds__(256) k_gemv_bf16_reg_group(GemvGroupArgs g, in
 
 // ============================================================ f32 NT tile kernel
 // 64x64 tile, BK=16, 256 threads each computing a 4x4 micro-tile with FMA.
-__global__ void __launch_bounds__(256) k_linear_f32(LinearArgs a) {
+__device__ __forceinline__ void linear_f32_tile(const LinearArgs &a, int tile_m, int tile_n) {
   constexpr int BM = 64, BN = 64, BK = 16;
   __shared__ float As[BK][BM + 4];
   __shared__ float Bs[BK][BN + 4];
   const int tid = threadIdx.x;
-  const int tiles_m = (a.M + BM - 1) / BM;
-  const int tile_n = blockIdx.x / tiles_m, tile_m = blockIdx.x % tiles_m;
   const int m0 = tile_m * BM, n0 = tile_n * BN;
   const float *A = (const float *)a.A;
   const float *W = (const float *)a.W;
@@ -477,11 +484,28 @@ __global__ void __launch_bounds__(256) k_linear_f32(LinearArgs a) {
       if (n >= a.N) continue;
       float v = acc[i][j] + (bias ? bias[n] : 0.f) + (bias2 ? bias2[n] : 0.f);
       if (a.act >= 0 && n >= a.act_from) v = act_eval(a.act, v);
+      if (a.f32_out) v *= a.out_scale;
       if (res) v += res[(int64_t)m * a.ldr + n];
       if (n < a.n_split) ((float *)a.out1)[(int64_t)m * a.ld1 + n] = v;
       else ((float *)a.out2)[(int64_t)m * a.ld2 + (n - a.n_split)] = v;
     }
   }
+}
+
+__global__ void __launch_bounds__(256) k_linear_f32(LinearArgs a) {
+  const int tiles_m = (a.M + 63) / 64;
+  linear_f32_tile(a, blockIdx.x % tiles_m, blockIdx.x / tiles_m);
+}
+
+// The same tile over the rows of one expert (see MoePlan): blockIdx.x = column tile, blockIdx.y = row tile.
+__global__ void __launch_bounds__(256) k_linear_f32_grouped(LinearArgs a, int64_t w_stride, const int4 *tiles, const int *n_tiles) {
+  if ((int)blockIdx.y >= *n_tiles) return;
+  const int4 t = tiles[blockIdx.y];
+  a.A = (const float *)a.A + (int64_t)t.y * a.lda;
+  a.W = (const float *)a.W + (int64_t)t.x * w_stride;
+  a.out1 = (float *)a.out1 + (int64_t)t.y * a.ld1;
+  a.M = t.z;
+  linear_f32_tile(a, 0, blockIdx.x);
 }
 
 // ============================================================ generic strided batched matmul
@@ -638,6 +662,7 @@ int launch_linear_bf16_skinny(hipStream_t st, const LinearArgs &a) {
                 RAI_ERR_UNSUPPORTED, "linear: second product not served (one row, no norm, no gate)");
   if (a.glu) RAI_REQUIRE(a.N % 2 == 0 && !a.residual && a.n_split == a.N && a.act >= 0, RAI_ERR_BAD_ARG,
                          "linear: bad gated-MLP arguments");
+  RAI_REQUIRE(!a.f32_out || (a.n_split == a.N && !a.glu), RAI_ERR_BAD_ARG, "linear: an f32 output is a single, ungated one");
   if (a.M == 1 && a.K <= 4096 && a.N >= 1024 && !dual) {
     // activation vector in registers (at most 8 chunks of 16 bytes per lane)
     if (a.K <= 2048) return launch_gemv_reg<4, 4>(st, a, 8);
@@ -782,6 +807,11 @@ int launch_linear_f32(hipStream_t st, const LinearArgs &a) {
   const int tiles = ((a.M + 63) / 64) * ((a.N + 63) / 64);
   hipLaunchKernelGGL(k_linear_f32, dim3(tiles), dim3(256), 0, st, a);
   return launch_check("linear_f32");
+}
+
+int launch_linear_f32_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan) {
+  hipLaunchKernelGGL(k_linear_f32_grouped, dim3((a.N + 63) / 64, plan.cap_tiles), dim3(256), 0, st, a, w_stride, plan.tiles, plan.n_tiles);
+  return launch_check("linear_f32_grouped");
 }
 
 // Lends the device's scratch block to a tile GEMM that may split K.

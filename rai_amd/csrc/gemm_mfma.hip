@@ -18,6 +18,7 @@
 #include <type_traits>
 
 #include "gemm.h"
+#include "latent.h"
 
 namespace rai {
 
@@ -207,6 +208,29 @@ __device__ __forceinline__ void gemm_tile_epilogue(const LinearArgs &a, f32x16 (
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] += bv[e];
       if (a.act >= 0) act8(a.act, v, n, a.act_from);
+      if (a.f32_out) {
+        float *dst = (float *)a.out1 + (int64_t)m * a.ld1 + n;
+        const float *rsrc = res ? (const float *)a.residual + (int64_t)m * a.ldr + n : nullptr;
+        if (whole && a.ld1 % 4 == 0 && (!res || a.ldr % 4 == 0) && (((uintptr_t)a.out1 | (uintptr_t)a.residual) & 15) == 0) {
+          f32x4 r0 = {0.f, 0.f, 0.f, 0.f}, r1 = r0;
+          if (rsrc) {
+            r0 = *reinterpret_cast<const f32x4 *>(rsrc);
+            r1 = *reinterpret_cast<const f32x4 *>(rsrc + 4);
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            r0[e] = fmaf(a.out_scale, v[e], r0[e]);
+            r1[e] = fmaf(a.out_scale, v[4 + e], r1[e]);
+          }
+          *reinterpret_cast<f32x4 *>(dst) = r0;
+          *reinterpret_cast<f32x4 *>(dst + 4) = r1;
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            if (e < lim) dst[e] = fmaf(a.out_scale, v[e], rsrc ? rsrc[e] : 0.f);
+        }
+        continue;
+      }
       if (res) {
         if (vec_out) {
           float rv[8];
@@ -675,6 +699,30 @@ __global__ void __launch_bounds__(64 * WGM * WGN) k_gemm_bf16_mfma_dma(LinearArg
   gemm_tile_epilogue<BM, BN, dma_lds_bytes<BM, BN, NS, WGN, WGM>(), WGN, WGM>(a, acc, lds, m0, n0, wave, lane, split, partial);
 }
 
+// The same tile over the rows of one expert (see MoePlan): a block finds its expert and rows in the device-side table,
+// whose length only the device knows; the grid covers the largest it can be and the blocks behind the end leave.
+template <int BM, int BN, int WGN>
+__global__ void __launch_bounds__(128 * WGN) k_gemm_bf16_mfma_grouped(LinearArgs a, int64_t w_stride, const int4 *table, const int *n_tiles) {
+  extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tiles_m = *n_tiles, tiles_n = (a.N + BN - 1) / BN;
+  const int total = tiles_m * tiles_n;
+  if ((int)blockIdx.x >= (total + kXcds - 1) / kXcds * kXcds) return;
+  const int tile = xcd_remap(blockIdx.x, total);
+  if (tile >= total) return;
+  // an XCD's run walks all column tiles of one row tile group: the experts' weights are read once, their rows from L2
+  int tile_m, tile_n;
+  tile_coords(tile, tiles_m, tiles_n, &tile_m, &tile_n);
+  const int4 t = table[tile_m];
+  a.A = (const uint16_t *)a.A + (int64_t)t.y * a.lda;
+  a.W = (const uint16_t *)a.W + (int64_t)t.x * w_stride;
+  a.out1 = (uint16_t *)a.out1 + (int64_t)t.y * a.ld1;
+  a.M = t.z;
+  f32x16 acc[BM / 64][BN / (32 * WGN)];
+  dma_tile_mainloop_k64<BM, BN, WGN>(a, lds, 0, tile_n * BN, 0, a.K / 64, wave, lane, acc);
+  gemm_tile_epilogue<BM, BN, dma_lds_bytes<BM, BN, 2, WGN>(), WGN>(a, acc, lds, 0, tile_n * BN, wave, lane, 0, nullptr);
+}
+
 // ---- stream-K form of the eight-wave 256x256 tile kernel ---------------------------------------------------------
 // One block per CU.  When the tile count is not a multiple of the CU count, the last partial round would leave CUs
 // idle for a whole tile time (140 tiles on 256 CUs: 45 % of the machine).  Here the K tiles of those `sk_tiles` tiles
@@ -849,6 +897,10 @@ __global__ void __launch_bounds__(256) k_splitk_epilogue(LinearArgs a, int split
     for (int s = 0; s < splits; ++s) x += partial[(int64_t)s * total + e];
     x += (bias ? bf16_bits_to_f32(bias[n]) : 0.f) + (bias2 ? bf16_bits_to_f32(bias2[n]) : 0.f);
     if (a.act >= 0 && n >= a.act_from) x = act_eval(a.act, x);
+    if (a.f32_out) {
+      ((float *)a.out1)[(int64_t)m * a.ld1 + n] = fmaf(a.out_scale, x, res ? ((const float *)a.residual)[(int64_t)m * a.ldr + n] : 0.f);
+      continue;
+    }
     if (res) x += bf16_bits_to_f32(res[(int64_t)m * a.ldr + n]);
     if (n < a.n_split) ((uint16_t *)a.out1)[(int64_t)m * a.ld1 + n] = f32_to_bf16_bits(x);
     else ((uint16_t *)a.out2)[(int64_t)m * a.ld2 + (n - a.n_split)] = f32_to_bf16_bits(x);
@@ -997,7 +1049,7 @@ __global__ void __launch_bounds__(256) k_splitk_epilogue_ln(LinearArgs a, int sp
 // Whether the pass over the partial sums can also normalise the rows: one ungated output, whole 16-byte packs.
 static bool post_norm_fits(const LinearArgs &a) {
   auto al16 = [](const void *p) { return ((uintptr_t)p & 15) == 0; };
-  return a.post_ln_out && !a.glu && a.n_split >= a.N && a.N % 8 == 0 && a.N <= 4096 && a.ld1 % 8 == 0 && al16(a.out1) &&
+  return a.post_ln_out && !a.glu && !a.f32_out && a.n_split >= a.N && a.N % 8 == 0 && a.N <= 4096 && a.ld1 % 8 == 0 && al16(a.out1) &&
          al16(a.post_ln_out) && (!a.bias || al16(a.bias)) && (!a.bias2 || al16(a.bias2)) &&
          (!a.residual || (a.ldr % 8 == 0 && al16(a.residual))) && (!a.post_ln_w || al16(a.post_ln_w)) &&
          (!a.post_ln_b || al16(a.post_ln_b)) && a.splitk_ws && ((uintptr_t)a.splitk_ws & 15) == 0;
@@ -1308,6 +1360,10 @@ __global__ void __launch_bounds__(256) k_linear_bf16_mfma_skinny(LinearArgs a, i
       const int nn = n + e;
       float x = v[e] + (bias ? bf16_bits_to_f32(bias[nn]) : 0.f) + (bias2 ? bf16_bits_to_f32(bias2[nn]) : 0.f);
       if (a.act >= 0 && nn >= a.act_from) x = act_eval(a.act, x);
+      if (a.f32_out) {
+        ((float *)a.out1)[(int64_t)m * a.ld1 + nn] = fmaf(a.out_scale, x, res ? ((const float *)a.residual)[(int64_t)m * a.ldr + nn] : 0.f);
+        continue;
+      }
       if (res) x += bf16_bits_to_f32(res[(int64_t)m * a.ldr + nn]);
       if (nn < a.n_split) ((uint16_t *)a.out1)[(int64_t)m * a.ld1 + nn] = f32_to_bf16_bits(x);
       else ((uint16_t *)a.out2)[(int64_t)m * a.ld2 + (nn - a.n_split)] = f32_to_bf16_bits(x);
@@ -1535,6 +1591,19 @@ __global__ void __launch_bounds__(512) k_linear_bf16_mfma_stream(LinearArgs a, i
       else { dst[0] = o[0]; dst[1] = o[1]; }
       return;
     }
+    if (a.f32_out) {
+      float *dst = (float *)a.out1 + (int64_t)m * a.ld1 + n;
+      const float *rsrc = res ? (const float *)a.residual + (int64_t)m * a.ldr + n : nullptr;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (e < lim) {
+          float y = x[e] + ((bias ? bf16_bits_to_f32(bias[n + e]) : 0.f) + (bias2 ? bf16_bits_to_f32(bias2[n + e]) : 0.f));
+          if (a.act >= 0 && n + e >= a.act_from) y = act_eval(a.act, y);
+          dst[e] = fmaf(a.out_scale, y, rsrc ? rsrc[e] : 0.f);
+        }
+      }
+      return;
+    }
     uint16_t o[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -1752,6 +1821,23 @@ static int tile_splits(const LinearArgs &a) {
   return splits;
 }
 
+int launch_linear_bf16_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan) {
+  RAI_REQUIRE(a.K % 64 == 0 && a.lda % 8 == 0 && a.ldw % 8 == 0 && w_stride % 8 == 0 && a.n_split == a.N && !a.residual && !a.f32_out &&
+                  (!a.glu || a.N % 8 == 0),
+              RAI_ERR_BAD_ARG, "linear grouped: %d x %d not served", a.N, a.K);
+  constexpr int BM = 128, BN = 128;
+  constexpr size_t lds = dma_lds_bytes<BM, BN, 2, 2>();
+  static bool attr_set = false;
+  if (lds > 64 * 1024 && !attr_set) {
+    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_gemm_bf16_mfma_grouped<BM, BN, 2>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    attr_set = true;
+  }
+  const int total = plan.cap_tiles * ((a.N + BN - 1) / BN);
+  hipLaunchKernelGGL((k_gemm_bf16_mfma_grouped<BM, BN, 2>), dim3((total + kXcds - 1) / kXcds * kXcds), dim3(256), lds, st, a, w_stride,
+                     plan.tiles, plan.n_tiles);
+  return launch_check("gemm_bf16_mfma_grouped");
+}
+
 bool linear_fuses_post_norm(const LinearArgs &a) {
   // the tile kernels serve more than 64 rows; their split-K pass is the one that can normalise
   // (RAI_HIP_NO_POST_NORM: run the norm as its own launch, for comparison)
@@ -1774,6 +1860,7 @@ int launch_linear_bf16_mfma(hipStream_t st, const LinearArgs &a) {
               "linear: fused norm needs M <= 8, or an RMS norm with M <= 64 and K within one block's span");
   if (a.glu) RAI_REQUIRE(a.N % 8 == 0 && !a.residual && a.n_split == a.N && a.act >= 0, RAI_ERR_BAD_ARG,
                          "linear mfma: bad gated-MLP arguments");
+  RAI_REQUIRE(!a.f32_out || (a.n_split == a.N && !a.glu), RAI_ERR_BAD_ARG, "linear mfma: an f32 output is a single, ungated one");
   RAI_REQUIRE(a.K % 32 == 0, RAI_ERR_UNSUPPORTED, "linear mfma: K=%d must be a multiple of 32", a.K);
   RAI_REQUIRE(a.lda % 8 == 0 && a.ldw % 8 == 0 && (uintptr_t)a.A % 16 == 0 && (uintptr_t)a.W % 16 == 0,
               RAI_ERR_BAD_STRIDE, "linear mfma: operands must be 16-byte aligned with row strides multiple of 8");

@@ -7,6 +7,7 @@
 // rai-nn/src/rms_norm.rs:18-22, rai-models/src/llm/gemma.rs:42-54,
 // rotary: rai-models/src/llm/phi2.rs:44-78, qwen2.rs:33-72.
 #include "common.h"
+#include "latent.h"
 
 namespace rai {
 
@@ -223,6 +224,122 @@ k_rope_tables(TT *cos_t, TT *sin_t, int64_t max_pos, int rot, double theta, int 
     Scalar<TT>::store(cos_t + e, (typename Scalar<TT>::compute)cosf(ang));
     Scalar<TT>::store(sin_t + e, (typename Scalar<TT>::compute)sinf(ang));
   }
+}
+
+// ---------------------------------------------------------------- grouped RMS norm of an f32 residual stream
+// One block per output row (see StreamNormArgs).  A thread owns packs of V elements, tid, tid + 256, ...; the first
+// ITEMS of them stay in registers between the two passes, any others are formed again (ITEMS == 0: all of them).  The
+// sum of squares of a pack goes to LDS and one wave sums each group's packs in a fixed order, so the statistics do not
+// depend on how a group's packs fall on the waves.
+template <typename T, int V, int ITEMS>
+__global__ void __launch_bounds__(256) k_stream_norm(StreamNormArgs a) {
+  extern __shared__ float sn_lds[];   // [packs] sums of squares | [groups] scales
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int packs = a.width / V, gpacks = packs / a.groups;
+  float *scale = sn_lds + packs;
+  const int64_t r = blockIdx.x;
+  const int64_t row = a.row_map ? a.row_map[r] : a.first + r * a.step;
+  const T *add = (const T *)a.add;
+  const int *add_rows = add ? a.add_rows + row * a.top : nullptr;
+  auto form = [&](int p, float (&v)[V]) {
+    if (a.src_f32) {
+      const NPack<float, V> s = *reinterpret_cast<const NPack<float, V> *>((const float *)a.src + row * a.src_ld + p * V);
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = s.v[e];
+    } else {
+      const NPack<T, V> s = *reinterpret_cast<const NPack<T, V> *>((const T *)a.src + row * a.src_ld + p * V);
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = (float)Scalar<T>::load(&s.v[e]);
+    }
+    if (add) {
+      float sum[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) sum[e] = 0.f;
+      for (int j = 0; j < a.top; ++j) {
+        const NPack<T, V> s = *reinterpret_cast<const NPack<T, V> *>(add + (int64_t)add_rows[j] * a.add_ld + p * V);
+#pragma unroll
+        for (int e = 0; e < V; ++e) sum[e] += (float)Scalar<T>::load(&s.v[e]);
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = fmaf(a.add_scale, sum[e], v[e]);
+    }
+  };
+  float keep[ITEMS > 0 ? ITEMS : 1][V];
+  auto square = [&](int p, const float (&v)[V]) {
+    float q = 0.f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) q = fmaf(v[e], v[e], q);
+    sn_lds[p] = q;
+  };
+#pragma unroll
+  for (int i = 0; i < ITEMS; ++i)
+    if (tid + i * 256 < packs) {
+      form(tid + i * 256, keep[i]);
+      square(tid + i * 256, keep[i]);
+    }
+  for (int p = tid + ITEMS * 256; p < packs; p += 256) {
+    float v[V];
+    form(p, v);
+    square(p, v);
+  }
+  __syncthreads();
+  for (int g = wave; g < a.groups; g += 4) {
+    float q = 0.f;
+    for (int p = lane; p < gpacks; p += 64) q += sn_lds[g * gpacks + p];
+    q = wave_sum(q);
+    if (lane == 0) scale[g] = 1.0f / sqrtf(q / (float)(gpacks * V) + a.eps);
+  }
+  __syncthreads();
+  auto finish = [&](int p, const float (&v)[V]) {
+    const float sc = scale[p / gpacks];
+    if (a.x) {
+      NPack<float, V> o;
+#pragma unroll
+      for (int e = 0; e < V; ++e) o.v[e] = v[e];
+      *reinterpret_cast<NPack<float, V> *>(a.x + row * a.x_ld + p * V) = o;
+    }
+    auto put = [&](const void *w, void *h) {
+      const NPack<T, V> wp = *reinterpret_cast<const NPack<T, V> *>((const T *)w + p * V);
+      NPack<T, V> o;
+#pragma unroll
+      for (int e = 0; e < V; ++e) Scalar<T>::store(&o.v[e], v[e] * sc * (float)Scalar<T>::load(&wp.v[e]));
+      *reinterpret_cast<NPack<T, V> *>((T *)h + r * a.h_ld + p * V) = o;
+    };
+    if (a.h1) put(a.w1, a.h1);
+    if (a.h2) put(a.w2, a.h2);
+  };
+#pragma unroll
+  for (int i = 0; i < ITEMS; ++i)
+    if (tid + i * 256 < packs) finish(tid + i * 256, keep[i]);
+  for (int p = tid + ITEMS * 256; p < packs; p += 256) {
+    float v[V];
+    form(p, v);
+    finish(p, v);
+  }
+  for (int c = a.width + tid; c < a.h_ld; c += 256) {
+    if (a.h1) Scalar<T>::store((T *)a.h1 + r * a.h_ld + c, 0.f);
+    if (a.h2) Scalar<T>::store((T *)a.h2 + r * a.h_ld + c, 0.f);
+  }
+}
+
+template <typename T> static int launch_stream_norm_t(hipStream_t st, const StreamNormArgs &a) {
+  auto al = [](const void *p, int64_t ld, size_t es) { return !p || ((uintptr_t)p % 16 == 0 && ld * es % 16 == 0); };
+  const bool vec = (a.width / a.groups) % 8 == 0 && al(a.src, a.src_ld, a.src_f32 ? 4 : sizeof(T)) && al(a.x, a.x_ld, 4) &&
+                   al(a.add, a.add_ld, sizeof(T)) && al(a.w1, 8, 2) && al(a.w2, 8, 2) && al(a.h1, a.h_ld, sizeof(T)) && al(a.h2, a.h_ld, sizeof(T));
+  const int packs = vec ? a.width / 8 : a.width;
+  const size_t lds = (size_t)(packs + a.groups) * sizeof(float);
+  RAI_REQUIRE(lds <= 64 * 1024, RAI_ERR_UNSUPPORTED, "stream norm: width %d not served", a.width);
+  const dim3 grid((unsigned)a.rows), block(256);
+  if (!vec) hipLaunchKernelGGL((k_stream_norm<T, 1, 0>), grid, block, lds, st, a);
+  else if (packs <= 256) hipLaunchKernelGGL((k_stream_norm<T, 8, 1>), grid, block, lds, st, a);
+  else hipLaunchKernelGGL((k_stream_norm<T, 8, 2>), grid, block, lds, st, a);
+  return launch_check("stream_norm");
+}
+
+int launch_stream_norm(hipStream_t st, int dtype, const StreamNormArgs &a) {
+  RAI_REQUIRE(a.rows > 0 && a.width > 0 && a.groups > 0 && a.width % a.groups == 0 && a.h_ld >= a.width, RAI_ERR_BAD_SHAPE,
+              "stream norm: width %d in %d groups", a.width, a.groups);
+  return dtype == RAI_BF16 ? launch_stream_norm_t<bf16_raw>(st, a) : launch_stream_norm_t<float>(st, a);
 }
 
 static int norm_impl(int dev, const rai_hip_tensor *x, const rai_hip_tensor *w, const rai_hip_tensor *b, double eps,

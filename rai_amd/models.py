@@ -11,7 +11,7 @@ import ctypes as C
 import numpy as np
 
 from . import _lib
-from ._lib import ARCH, DTYPE_BY_NAME, UNARY, DecoderConfig, call
+from ._lib import ARCH, DTYPE_BY_NAME, MLP_KIND, UNARY, DecoderConfig, LatentConfig, LatentLayer, call
 
 _ACT = {"gelu_new": "new_gelu", "new_gelu": "new_gelu", "gelu": "gelu", "silu": "silu", "relu": "relu"}
 
@@ -47,6 +47,31 @@ class Decoder:
         self._h = C.c_void_p()
         call("rai_hip_init", dev)
         call("rai_hip_decoder_create", dev, C.byref(cfg), C.byref(self._h))
+
+    @classmethod
+    def latent(cls, dtype, *, vocab_size, width, layers, norm_eps, norm_groups=1, residual_mult=1.0, max_batch=1,
+               max_context=2048, dev=0):
+        """A decoder of latent-attention layers described one by one (rai_hip_decoder_create_latent): every entry of
+        `layers` is a dict with the fields of _lib.LatentLayer; mlp_kind and mlp_act by name."""
+        c = LatentConfig(dtype=DTYPE_BY_NAME[dtype], vocab_size=vocab_size, width=width, num_layers=len(layers),
+                         norm_groups=norm_groups, max_batch=max_batch, max_context=max_context, norm_eps=norm_eps,
+                         residual_mult=residual_mult)
+        arr = (LatentLayer * len(layers))()
+        for i, spec in enumerate(layers):
+            spec = dict(spec)
+            spec["mlp_kind"] = MLP_KIND[spec.get("mlp_kind", "none")]
+            spec["mlp_act"] = UNARY[_ACT[spec.get("mlp_act", "silu")]]
+            for k, v in spec.items():
+                setattr(arr[i], k, v)
+        self = cls.__new__(cls)
+        self._h = C.c_void_p()
+        # the fields the other methods read
+        self.cfg = DecoderConfig(arch=ARCH["lelitar"], dtype=c.dtype, vocab_size=vocab_size, hidden_size=width,
+                                 num_hidden_layers=len(layers), max_batch=max_batch, max_context=max_context)
+        self.dtype, self.dev = dtype, dev
+        call("rai_hip_init", dev)
+        call("rai_hip_decoder_create_latent", dev, C.byref(c), arr, C.byref(self._h))
+        return self
 
     def close(self):
         if self._h:
@@ -112,6 +137,16 @@ class Decoder:
              logits.ctypes.data_as(C.POINTER(C.c_float)) if want_logits else None,
              toks.ctypes.data_as(C.POINTER(C.c_uint32)))
         return hidden, logits, toks
+
+    def forward_rows(self, ids, rows=()):
+        """Appends ids [B, S] after the cached context; logits [len(rows), vocab] f32 of the given rows (b * S + s)."""
+        ids = np.ascontiguousarray(ids, dtype=np.uint32)
+        b, s = ids.shape
+        rows = np.ascontiguousarray(rows, dtype=np.int32)
+        logits = np.empty((rows.size, self.cfg.vocab_size), np.float32)
+        call("rai_hip_decoder_forward_rows", self._h, ids.ctypes.data_as(C.POINTER(C.c_uint32)), b, s,
+             rows.ctypes.data_as(C.POINTER(C.c_int32)), rows.size, logits.ctypes.data_as(C.POINTER(C.c_float)))
+        return logits
 
     def generate(self, prompt, n_new):
         """Greedy decode: returns (tokens [B, n_new], prefill_ms, decode_ms)."""

@@ -45,10 +45,12 @@ def test_ctypes_structs_match_header_layout():
     from rai_amd import _lib
     assert ctypes.sizeof(_lib.TensorDesc) == 8 + 4 + 4 + 8 * 8 + 8 * 8 + 8
     text = (ROOT / "include" / "rai_hip.h").read_text()
-    body = text[text.index("typedef struct rai_hip_decoder_config {"):text.index("} rai_hip_decoder_config;")]
-    body = re.sub(r"/\*.*?\*/", "", body, flags=re.S)
-    fields = re.findall(r"(?:int32_t|double)\s+(\w+)\s*;", body)
-    assert fields == [f[0] for f in _lib.DecoderConfig._fields_]
+    for struct, mirror in (("decoder_config", _lib.DecoderConfig), ("latent_layer", _lib.LatentLayer),
+                           ("latent_config", _lib.LatentConfig)):
+        body = text[text.index(f"typedef struct rai_hip_{struct} {{"):text.index(f"}} rai_hip_{struct};")]
+        body = re.sub(r"/\*.*?\*/", "", body, flags=re.S)
+        fields = re.findall(r"(int32_t|double)\s+(\w+)\s*;", body)
+        assert fields == [("double" if t is ctypes.c_double else "int32_t", n) for n, t in mirror._fields_]
     enum = text[text.index("typedef enum rai_hip_unary_op {"):text.index("} rai_hip_unary_op;")]
     for name, val in re.findall(r"RAI_UN_(\w+)\s*=\s*(\d+)", enum):
         assert _lib.UNARY[name.lower()] == int(val)

@@ -407,6 +407,16 @@ def test_fused_linear_bias_act_residual(R, dt, m):
     assert_close(down(R.linear(up(x, dt), up(w, dt))), onn.linear(x, w, None, dt), dt, "linear plain")
 
 
+@pytest.mark.parametrize("m", [1, 2, 3, 4, 5, 8])
+@pytest.mark.parametrize("k,n", [(2304, 2560), (2304, 512), (4160, 3000), (8968, 640), (1544, 5200)])
+def test_linear_few_rows_k_ends_inside_a_step(R, m, k, n):
+    """Up to 8 rows, K more than one step of the weight-streaming kernel and not a multiple of 512: the last step covers
+    only some of a wave's lanes."""
+    g = rng(126)
+    x, w, b = rand(g, (m, k), "bf16"), rand(g, (n, k), "bf16", 0.03), rand(g, (n,), "bf16")
+    assert_close(down(R.linear(up(x, "bf16"), up(w, "bf16"), up(b, "bf16"))), onn.linear(x, w, b, "bf16"), "bf16", f"linear {m}x{k}x{n}")
+
+
 @pytest.mark.parametrize("kernel", ["stream", "skinny", "tile"])
 @pytest.mark.parametrize("m", [9, 16, 31, 64])
 @pytest.mark.parametrize("k,n", [(4096, 200), (1056, 2048), (16384, 64), (96, 50), (2048, 16384)])
