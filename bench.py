@@ -223,6 +223,83 @@ def run_gemma_decode(args):
     dec.close()
 
 
+# Layers like those of real models, Lelitar beside the framework's closest family (Qwen2: gated MLP, RMS norms, one
+# head layout) at equal width, heads and MLP.  (width, heads, q_rank, kv_rank, window, ff, experts, expert ff, top, layers)
+LELITAR_SIZES = {
+    "1024": dict(width=1024, heads=8, q_rank=384, kv_rank=256, window=512, ff=4096, experts=32, eff=512, top=4, layers=8),
+    "2048": dict(width=2048, heads=16, q_rank=768, kv_rank=512, window=1024, ff=8192, experts=64, eff=1024, top=6, layers=4),
+    "4096": dict(width=4096, heads=32, q_rank=1536, kv_rank=512, window=2048, ff=14336, experts=16, eff=3584, top=2, layers=4),
+}
+LELITAR_VOCAB = 32768
+
+
+def lelitar_case(size, kind, max_batch, max_context):
+    """A decoder of one size: kind 'dense', 'moe' or 'qwen2', with its multiply-adds and weight bytes per token."""
+    from rai_amd.models import Decoder
+    z, hd = LELITAR_SIZES[size], 128
+    w, qd, n = z["width"], z["heads"] * 128, z["layers"]
+    if kind == "qwen2":
+        dec = Decoder("qwen2", "bf16", vocab_size=LELITAR_VOCAB, hidden_size=w, intermediate_size=z["ff"], num_hidden_layers=n,
+                      num_attention_heads=z["heads"], head_dim=hd, max_position_embeddings=max_context, hidden_act="silu",
+                      norm_eps=1e-6, max_batch=max_batch, max_context=max_context)
+        lin = 4 * w * qd + 3 * w * z["ff"]
+        return dec, dict(lin=lin, weights=lin, keys=lambda t: t, key_flops=4 * qd, key_bytes=4 * qd, layers=n)
+    layer = dict(heads=z["heads"], qk_dim=hd, v_dim=hd, q_rank=z["q_rank"], kv_rank=z["kv_rank"], window=z["window"], attn_scale=hd ** -0.5)
+    attn = w * (z["q_rank"] + z["kv_rank"] + qd) + z["q_rank"] * qd + 2 * z["kv_rank"] * qd + qd * w
+    if kind == "dense":
+        layer.update(mlp_kind="dense", mlp_act="relu", intermediate=z["ff"])
+        mlp = lambda rows: 3 * w * z["ff"]
+        lin = attn + 3 * w * z["ff"]
+    else:
+        layer.update(mlp_kind="moe", mlp_act="silu", intermediate=z["eff"], experts=z["experts"], top=z["top"])
+        # experts a step of `rows` tokens is expected to touch, at uniform routing
+        mlp = lambda rows: 3 * w * z["eff"] * z["experts"] * (1 - (1 - z["top"] / z["experts"]) ** rows) + w * z["experts"]
+        lin = attn + 3 * w * z["eff"] * z["top"] + w * z["experts"]
+    dec = Decoder.latent("bf16", vocab_size=LELITAR_VOCAB, width=w, layers=[layer] * n, norm_eps=1e-6, norm_groups=4,
+                         residual_mult=0.5, max_batch=max_batch, max_context=max_context)
+    return dec, dict(lin=lin, weights=lambda rows: attn + mlp(rows), keys=lambda t: min(t, z["window"]), key_flops=4 * qd,
+                     key_bytes=2 * z["kv_rank"], layers=n)
+
+
+def run_lelitar(args):
+    """Prefill and decode of the Lelitar design beside the closest family of equal size; one line per case."""
+    from rai_amd import synthetic
+    B, CTX, NEWT = 32, 1024, 33
+    sizes = args.lelitar_sizes.split(",") if args.lelitar_sizes else list(LELITAR_SIZES)
+    table = {}
+    for size in sizes:
+        for kind in ("qwen2", "dense", "moe"):
+            if args.lelitar_kinds and kind not in args.lelitar_kinds.split(","):
+                continue
+            dec, c = lelitar_case(size, kind, B, CTX + NEWT)
+            synthetic.load_tiled_params(dec)
+            w = LELITAR_SIZES[size]["width"]
+            head = LELITAR_VOCAB * w
+            row = {}
+            for batch in (1, B):
+                ids = synthetic.prompt(LELITAR_VOCAB, batch, CTX)
+                pre, dcd = [], []
+                for it in range(args.warmup + args.steps):
+                    _, p, d = dec.generate(ids, NEWT)
+                    if it >= args.warmup:
+                        pre.append(p)
+                        dcd.append(d / (NEWT - 1))
+                p, d = float(np.mean(pre)) / 1e3, float(np.mean(dcd)) / 1e3
+                seen = sum(c["keys"](t) for t in range(1, CTX + 1)) / CTX
+                flops = 2.0 * batch * CTX * c["layers"] * c["lin"] + batch * CTX * c["layers"] * seen * c["key_flops"] + 2.0 * batch * head
+                wb = c["weights"](batch) if callable(c["weights"]) else c["weights"]
+                byts = 2.0 * (c["layers"] * wb + head) + c["layers"] * batch * c["keys"](CTX + NEWT / 2) * c["key_bytes"]
+                row[f"prefill_b{batch}"] = dict(tokens_per_s=round(batch * CTX / p), ms=round(p * 1e3, 3), tflops=round(flops / p / 1e12, 1))
+                row[f"decode_b{batch}"] = dict(tokens_per_s=round(batch / d, 1), us=round(d * 1e6, 1), gb_per_s=round(byts / d / 1e9))
+            table[f"{size} {kind}"] = row
+            print(json.dumps({"case": f"{size} {kind}", **row}), file=sys.stderr, flush=True)
+            dec.close()
+    first = next(iter(table.values()))
+    _line("Lelitar layers beside Qwen2 layers of equal size, prefill tok/s of the first case", first[f"prefill_b{B}"]["tokens_per_s"], "tokens/s",
+          args.steps, args.warmup, first[f"prefill_b{B}"]["ms"],
+          f"latent-attention decoders of {sizes} wide layers, bf16, prompts of {CTX}, batch 1 and {B}, random weights", {"cases": table})
+
+
 def run_ops(args):
     """Primitive sweep, bf16 and f32.  Every op is launched through the C ABI into an output allocated beforehand,
     with the tensor descriptors built once, so the timed loop holds launches only: `loop_us` is the hipEvent time of
@@ -504,8 +581,10 @@ def main():
                     help="tokens decoded through the lazy-graph path for the graph_decode_* fields (0: skip)")
     ap.add_argument("--cold", action="store_true",
                     help="gemm-tiles: rotate over weight copies so every launch reads its weight from HBM, as in a model")
-    ap.add_argument("--workload", default="phi2-decode", choices=["phi2-decode", "qwen2-prefill", "gemma-decode", "ops", "gemm-tiles", "peaks"],
+    ap.add_argument("--workload", default="phi2-decode", choices=["phi2-decode", "qwen2-prefill", "gemma-decode", "lelitar", "ops", "gemm-tiles", "peaks"],
                     help="phi2-decode is the headline line; the others are the remaining configurations of the path")
+    ap.add_argument("--lelitar-sizes", default="", help="lelitar: comma-separated widths (default: all)")
+    ap.add_argument("--lelitar-kinds", default="", help="lelitar: comma-separated subset of qwen2,dense,moe (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build measures one GPU; --gpus must be 1 (multi-GPU sharding is a design note only)")
@@ -513,6 +592,8 @@ def main():
         return run_qwen2_prefill(args)
     if args.workload == "gemma-decode":
         return run_gemma_decode(args)
+    if args.workload == "lelitar":
+        return run_lelitar(args)
     if args.workload == "ops":
         return run_ops(args)
     if args.workload == "gemm-tiles":

@@ -54,6 +54,8 @@ struct LatentLayer {
   char *Wb;                    // [Hp, QD + Fp]: o | down as one contraction (Fp = 0 without a dense MLP)
   char *Wr;                    // mixture: router [experts, Hp]
   char *We_gu, *We_dn;         // [experts][2 EFp, Hp] interleaved, [experts][Hp, EFp]
+  // Wd, Wuq, Wgu and Wb in MFMA-fragment order for 9 .. 64 rows (built on first use)
+  char *Wd_f, *Wuq_f, *Wgu_f, *Wb_f;
   char *cache;                 // [max_batch][max_context][Rp] normalised latents
 };
 
@@ -141,6 +143,8 @@ void add_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t
 int decoder_embed(rai_hip_decoder *d, hipStream_t st, int64_t rows);
 int decoder_linear(rai_hip_decoder *d, hipStream_t st, const LinearArgs &a);
 int launch_token_choice(rai_hip_decoder *d, hipStream_t st, int B, int S, bool advance_step);
+bool wants_fragments(const rai_hip_decoder *d, int64_t M);
+int decoder_fragments(rai_hip_decoder *d, hipStream_t st, char *W, int64_t ldw, int N, int K, char **dst);
 void decoder_init_fields(rai_hip_decoder *d, int dev, const rai_hip_decoder_config &cfg);
 int decoder_alloc_common(rai_hip_decoder *d);
 

@@ -688,17 +688,18 @@ static MegaArgs mega_args(rai_hip_decoder *d) {
 // kernel reads 1 KB per load instruction from a copy of the matrix in MFMA-fragment order.  The copies are made on
 // the first such step after the parameters changed (never under stream capture: generate runs its first
 // single-token step eagerly) and double the weight memory of the decoder.
-static bool wants_fragments(const rai_hip_decoder *d, int64_t M) {
+bool wants_fragments(const rai_hip_decoder *d, int64_t M) {
   static const bool off = getenv("RAI_HIP_NO_FRAG") != nullptr;
   return !off && d->cfg.dtype == RAI_BF16 && M > 8 && M <= 64;
 }
+int decoder_fragments(rai_hip_decoder *d, hipStream_t st, char *W, int64_t ldw, int N, int K, char **dst) {
+  if (!W || K % 32) { *dst = nullptr; return RAI_OK; }
+  if (!*dst) RAI_TRY(dalloc(d, linear_fragment_elems(N, K) * d->es, dst));
+  return launch_linear_fragment_layout(st, W, ldw, N, K, *dst);
+}
 static int ensure_fragments(rai_hip_decoder *d, hipStream_t st) {
   if (d->frag_ready) return RAI_OK;
-  auto one = [&](char *W, int64_t ldw, int N, int K, char **dst) -> int {
-    if (!W || K % 32) { *dst = nullptr; return RAI_OK; }
-    if (!*dst) RAI_TRY(dalloc(d, linear_fragment_elems(N, K) * d->es, dst));
-    return launch_linear_fragment_layout(st, W, ldw, N, K, *dst);
-  };
+  auto one = [&](char *W, int64_t ldw, int N, int K, char **dst) { return decoder_fragments(d, st, W, ldw, N, K, dst); };
   const int NQ = d->QD + 2 * d->KD;
   for (Layer &ly : d->layers) {
     if (d->cfg.arch == RAI_ARCH_PHI2) {

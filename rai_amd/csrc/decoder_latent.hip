@@ -187,6 +187,21 @@ static int ensure_derived(rai_hip_decoder *d, hipStream_t st) {
   return RAI_OK;
 }
 
+static int ensure_latent_fragments(rai_hip_decoder *d, hipStream_t st) {
+  LatentModel &lm = *d->latent;
+  if (d->frag_ready) return RAI_OK;
+  for (LatentLayer &y : lm.layers) {
+    const int KB = y.QD + y.Fp;
+    RAI_TRY(decoder_fragments(d, st, y.Wd, lm.Hp, y.ldn, lm.Hp, &y.Wd_f));
+    RAI_TRY(decoder_fragments(d, st, y.Wuq, y.Qp, y.QD, y.Qp, &y.Wuq_f));
+    RAI_TRY(decoder_fragments(d, st, y.Wgu, lm.Hp, 2 * y.Fp, lm.Hp, &y.Wgu_f));
+    RAI_TRY(decoder_fragments(d, st, y.Wb, KB, lm.Hp, KB, &y.Wb_f));
+  }
+  RAI_TRY(decoder_fragments(d, st, d->head_w, lm.Hp, d->V, lm.Hp, &d->head_f));
+  d->frag_ready = true;
+  return RAI_OK;
+}
+
 static LinearArgs latent_linear_args(rai_hip_decoder *d, const void *A, int64_t lda, int64_t M, const char *W, int N, int K) {
   LinearArgs a = linear_args_default();
   a.A = A; a.lda = lda;
@@ -197,10 +212,11 @@ static LinearArgs latent_linear_args(rai_hip_decoder *d, const void *A, int64_t 
 }
 
 // out = mult * A W^T + out, out the f32 stream
-static int residual_linear(rai_hip_decoder *d, hipStream_t st, const void *A, int64_t lda, int64_t M, const char *W, int K) {
+static int residual_linear(rai_hip_decoder *d, hipStream_t st, const void *A, int64_t lda, int64_t M, const char *W, int K, const char *Wfrag) {
   LatentModel &lm = *d->latent;
   LinearArgs a = latent_linear_args(d, A, lda, M, W, lm.Hp, K);
   a.ldw = lda;   // the activation buffer and the packed matrix have the same columns
+  a.Wfrag = Wfrag;
   a.out1 = lm.xs; a.ld1 = lm.Hp;
   a.residual = lm.xs; a.ldr = lm.Hp;
   a.f32_out = 1; a.out_scale = (float)lm.c.residual_mult;
@@ -263,7 +279,7 @@ static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int
   RAI_TRY(decoder_linear(d, st, r));
   RAI_TRY(launch_moe_route(st, lm.rlogits, M, y.c.experts, top, lm.rchoice, lm.rweight));
   const int64_t slots = M * top;
-  const int bm = dt == RAI_BF16 ? kGroupedRowsBf16 : kGroupedRowsF32;
+  const int bm = linear_grouped_rows(dt, slots, y.c.experts);
   MoePlan plan = lm.plan;
   plan.cap_tiles = moe_max_tiles(slots, y.c.experts, bm);
   RAI_TRY(launch_moe_plan(st, lm.rchoice, slots, y.c.experts, bm, plan, lm.rpos));
@@ -275,8 +291,8 @@ static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int
   o.out1 = lm.eout; o.ld1 = Hp;
   const int64_t gs = (int64_t)2 * y.EFp * Hp, os = (int64_t)Hp * y.EFp;
   if (dt == RAI_BF16) {
-    RAI_TRY(launch_linear_bf16_grouped(st, g, gs, plan));
-    return launch_linear_bf16_grouped(st, o, os, plan);
+    RAI_TRY(launch_linear_bf16_grouped(st, g, gs, plan, bm));
+    return launch_linear_bf16_grouped(st, o, os, plan, bm);
   }
   RAI_TRY(launch_linear_f32_grouped(st, g, gs, plan));
   return launch_linear_f32_grouped(st, o, os, plan);
@@ -378,6 +394,8 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
     return RAI_OK;
   }
 
+  const bool frag = wants_fragments(d, M);
+  if (frag || wants_fragments(d, B)) RAI_TRY(ensure_latent_fragments(d, st));
   const LatentLayer *pending = nullptr;   // the mixture whose outputs are not yet part of the stream
   for (int l = 0; l < d->L; ++l) {
     const LatentLayer &y = lm.layers[l];
@@ -394,6 +412,7 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
 
     LinearArgs a = latent_linear_args(d, lm.h1, Hp, M, y.Wd, y.ldn, Hp);
     a.out1 = lm.dn; a.ld1 = y.ldn;
+    a.Wfrag = frag ? y.Wd_f : nullptr;
     RAI_TRY(decoder_linear(d, st, a));
     const bool absorb = S < kAbsorbRows;
     LatentNormArgs ln;
@@ -408,16 +427,18 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
     RAI_TRY(launch_latent_norm(st, dt, ln));
     LinearArgs q = latent_linear_args(d, lm.cq, y.Qp, M, y.Wuq, y.QD, y.Qp);
     q.out1 = lm.q; q.ld1 = y.QD;
+    q.Wfrag = frag ? y.Wuq_f : nullptr;
     RAI_TRY(decoder_linear(d, st, q));
     RAI_TRY(absorb ? absorbed_attention(d, st, y, B, S) : expanded_attention(d, st, y, B, S));
 
     if (y.c.mlp_kind == RAI_MLP_DENSE) {
       LinearArgs g = latent_linear_args(d, lm.h2, Hp, M, y.Wgu, 2 * y.Fp, Hp);
       g.out1 = lm.cat + (size_t)y.QD * d->es; g.ld1 = y.QD + y.Fp;
+      g.Wfrag = frag ? y.Wgu_f : nullptr;
       g.act = y.c.mlp_act; g.act_from = 0; g.glu = 1;
       RAI_TRY(decoder_linear(d, st, g));
     }
-    RAI_TRY(residual_linear(d, st, lm.cat, y.QD + y.Fp, M, y.Wb, y.QD + y.Fp));
+    RAI_TRY(residual_linear(d, st, lm.cat, y.QD + y.Fp, M, y.Wb, y.QD + y.Fp, frag ? y.Wb_f : nullptr));
     if (y.c.mlp_kind == RAI_MLP_MIXTURE) {
       RAI_TRY(mixture(d, st, y, M));
       pending = &y;
@@ -438,6 +459,7 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
   RAI_TRY(launch_stream_norm(st, dt, n));
   LinearArgs h = latent_linear_args(d, d->last, Hp, B, d->head_w, d->V, Hp);
   h.out1 = d->logits; h.ld1 = d->V;
+  h.Wfrag = wants_fragments(d, B) ? d->head_f : nullptr;
   RAI_TRY(decoder_linear(d, st, h));
   RAI_TRY(launch_token_choice(d, st, B, S, advance_step));
   d->ctx_len += S;

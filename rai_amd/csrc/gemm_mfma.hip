@@ -1821,21 +1821,29 @@ static int tile_splits(const LinearArgs &a) {
   return splits;
 }
 
-int launch_linear_bf16_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan) {
-  RAI_REQUIRE(a.K % 64 == 0 && a.lda % 8 == 0 && a.ldw % 8 == 0 && w_stride % 8 == 0 && a.n_split == a.N && !a.residual && !a.f32_out &&
-                  (!a.glu || a.N % 8 == 0),
-              RAI_ERR_BAD_ARG, "linear grouped: %d x %d not served", a.N, a.K);
-  constexpr int BM = 128, BN = 128;
-  constexpr size_t lds = dma_lds_bytes<BM, BN, 2, 2>();
+template <int BM, int BN, int WGN>
+static int launch_grouped_cfg(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan) {
+  constexpr size_t lds = dma_lds_bytes<BM, BN, 2, WGN>();
   static bool attr_set = false;
   if (lds > 64 * 1024 && !attr_set) {
-    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_gemm_bf16_mfma_grouped<BM, BN, 2>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_gemm_bf16_mfma_grouped<BM, BN, WGN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     attr_set = true;
   }
   const int total = plan.cap_tiles * ((a.N + BN - 1) / BN);
-  hipLaunchKernelGGL((k_gemm_bf16_mfma_grouped<BM, BN, 2>), dim3((total + kXcds - 1) / kXcds * kXcds), dim3(256), lds, st, a, w_stride,
+  hipLaunchKernelGGL((k_gemm_bf16_mfma_grouped<BM, BN, WGN>), dim3((total + kXcds - 1) / kXcds * kXcds), dim3(128 * WGN), lds, st, a, w_stride,
                      plan.tiles, plan.n_tiles);
   return launch_check("gemm_bf16_mfma_grouped");
+}
+// The eight-wave 256 x 256 tile once the experts have a few such tiles each, so that partly filled ones weigh little.
+int linear_grouped_rows(int dtype, int64_t slots, int experts) {
+  if (dtype != RAI_BF16) return kGroupedRowsF32;
+  return slots >= (int64_t)experts * 4 * 256 ? 256 : kGroupedRowsBf16;
+}
+int launch_linear_bf16_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan, int bm) {
+  RAI_REQUIRE(a.K % 64 == 0 && a.lda % 8 == 0 && a.ldw % 8 == 0 && w_stride % 8 == 0 && a.n_split == a.N && !a.residual && !a.f32_out &&
+                  (!a.glu || a.N % 8 == 0),
+              RAI_ERR_BAD_ARG, "linear grouped: %d x %d not served", a.N, a.K);
+  return bm == 256 ? launch_grouped_cfg<256, 256, 4>(st, a, w_stride, plan) : launch_grouped_cfg<128, 128, 2>(st, a, w_stride, plan);
 }
 
 bool linear_fuses_post_norm(const LinearArgs &a) {

@@ -141,8 +141,9 @@ int launch_moe_plan(hipStream_t st, const int *choice, int64_t slots, int expert
 int launch_moe_gather(hipStream_t st, int dtype, const void *h, int64_t ld, int cols, const MoePlan &plan, const float *weight, int top,
                       int64_t slots, void *out);
 // One Linear per expert over its rows of the sorted order: W of expert e is w_stride elements behind that of e - 1.
-constexpr int kGroupedRowsBf16 = 128, kGroupedRowsF32 = 64;   // row tile (`bm` of the plan) of the two forms
-int launch_linear_bf16_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan);
+constexpr int kGroupedRowsBf16 = 128, kGroupedRowsF32 = 64;   // smallest row tile (`bm` of the plan) of the two forms
+int linear_grouped_rows(int dtype, int64_t slots, int experts);   // the row tile to plan for
+int launch_linear_bf16_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan, int bm);
 int launch_linear_f32_grouped(hipStream_t st, const LinearArgs &a, int64_t w_stride, const MoePlan &plan);
 
 }  // namespace rai

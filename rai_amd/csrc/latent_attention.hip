@@ -13,6 +13,24 @@ namespace rai {
 
 template <typename T> struct alignas(16) LPack { T v[16 / sizeof(T)]; };
 
+// acc + the dot product of two packs; bf16 pairs through v_dot2_f32_bf16 (exact products, f32 sums)
+__device__ __forceinline__ float pack_dot(const LPack<float> &a, const LPack<float> &b, float acc) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) acc = fmaf(a.v[e], b.v[e], acc);
+  return acc;
+}
+__device__ __forceinline__ float pack_dot(const LPack<bf16_raw> &a, const LPack<bf16_raw> &b, float acc) {
+  typedef __attribute__((ext_vector_type(2))) __bf16 pair;
+#pragma unroll
+  for (int e = 0; e < 8; e += 2) {
+    pair p, q;
+    __builtin_memcpy(&p, &a.v[e], 4);
+    __builtin_memcpy(&q, &b.v[e], 4);
+    acc = __builtin_amdgcn_fdot2_f32_bf16(p, q, acc, false);
+  }
+  return acc;
+}
+
 // ---------------------------------------------------------------- norms of the two latents, cache append
 // One wave per (row, latent): kind 0 = query latent, 1 = cached latent.
 template <typename T>
@@ -81,23 +99,37 @@ __global__ void __launch_bounds__(256) k_latent_absorb(const T *q, const T *WukT
 #pragma unroll
   for (int i = 0; i < NP; ++i) wr[i] = *reinterpret_cast<const LPack<T> *>(w + i * 4 * V);
   const int m0 = blockIdx.z * rows_per_block, m1 = m0 + rows_per_block < rows ? m0 + rows_per_block : rows;
-  for (int m = m0; m < m1; ++m) {
-    const T *qr = q + ((int64_t)m * heads + h) * Dp + part * V;
-    float acc = 0.f;
-    auto piece = [&](const LPack<T> &wv, int i) {
-      const LPack<T> qv = *reinterpret_cast<const LPack<T> *>(qr + i * 4 * V);
-#pragma unroll
-      for (int e = 0; e < V; ++e) acc = fmaf((float)Scalar<T>::load(&wv.v[e]), (float)Scalar<T>::load(&qv.v[e]), acc);
-    };
-    if constexpr (NP > 0) {
-#pragma unroll
-      for (int i = 0; i < NP; ++i) piece(wr[i], i);
-    } else {
-      for (int i = 0; i < np; ++i) piece(*reinterpret_cast<const LPack<T> *>(w + i * 4 * V), i);
-    }
+  auto finish = [&](int m, float acc) {
     acc += __shfl_xor(acc, 1, 64);
     acc += __shfl_xor(acc, 2, 64);
-    if (part == 0) Scalar<T>::store(qa + ((int64_t)m * heads + h) * Rp + r, acc);
+    if (part == 0 && m < m1) Scalar<T>::store(qa + ((int64_t)m * heads + h) * Rp + r, acc);
+  };
+  if constexpr (NP > 0) {
+    constexpr int G = NP <= 4 ? 4 : 2;   // rows whose queries are in flight together
+    for (int m = m0; m < m1; m += G) {
+      LPack<T> qv[G][NP];
+#pragma unroll
+      for (int g = 0; g < G; ++g) {
+        const T *qr = q + ((int64_t)(m + g < m1 ? m + g : m1 - 1) * heads + h) * Dp + part * V;
+#pragma unroll
+        for (int i = 0; i < NP; ++i) qv[g][i] = *reinterpret_cast<const LPack<T> *>(qr + i * 4 * V);
+      }
+#pragma unroll
+      for (int g = 0; g < G; ++g) {
+        float acc = 0.f;
+#pragma unroll
+        for (int i = 0; i < NP; ++i) acc = pack_dot(wr[i], qv[g][i], acc);
+        finish(m + g, acc);
+      }
+    }
+  } else {
+    for (int m = m0; m < m1; ++m) {
+      const T *qr = q + ((int64_t)m * heads + h) * Dp + part * V;
+      float acc = 0.f;
+      for (int i = 0; i < np; ++i)
+        acc = pack_dot(*reinterpret_cast<const LPack<T> *>(w + i * 4 * V), *reinterpret_cast<const LPack<T> *>(qr + i * 4 * V), acc);
+      finish(m, acc);
+    }
   }
 }
 
@@ -119,6 +151,10 @@ int launch_latent_transpose_uk(hipStream_t st, int dtype, const void *Wuk, void 
 }
 
 // ---------------------------------------------------------------- absorbed attention
+// The context is split for about this many blocks: two per CU of the MFMA form (a block serves up to 16 heads), four of
+// the other.
+constexpr int kLatentBlocks = 4 * kNumCU, kLatentMfmaBlocks = 2 * kNumCU;
+
 // Keys of query row m: the last min(pos + 1, window) positions up to its own, shared out evenly over the splits.
 struct LatentSpan { int lo, hi; };
 __device__ __forceinline__ LatentSpan latent_span(const LatentAttnArgs &a, int m, int split) {
@@ -242,17 +278,18 @@ __global__ void __launch_bounds__(256) k_latent_attn_mfma(LatentAttnArgs a) {
 
   for (int k0 = sp.lo; k0 < sp.hi; k0 += kLatKeys) {
     if (k0 != sp.lo) __syncthreads();   // the tile before has been read
-    for (int c = tid; c < kLatKeys * cpr; c += 256 * 4) {
-      la_u32x4 v[4];
+    constexpr int U = 8;   // a thread's pieces of the tile in flight
+    for (int c = tid; c < kLatKeys * cpr; c += 256 * U) {
+      la_u32x4 v[U];
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
+      for (int u = 0; u < U; ++u) {
         const int cc = c + u * 256;
         const int row = cc / cpr;
         const int key = k0 + row < sp.hi ? k0 + row : sp.hi - 1;   // rows past the span repeat its last key, masked below
         if (cc < kLatKeys * cpr) v[u] = *reinterpret_cast<const la_u32x4 *>(cache + (int64_t)key * Rp + (cc - row * cpr) * 8);
       }
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
+      for (int u = 0; u < U; ++u) {
         const int cc = c + u * 256;
         const int row = cc / cpr;
         if (cc < kLatKeys * cpr) *reinterpret_cast<la_u32x4 *>(cs + row * pitch + (cc - row * cpr) * 8) = v[u];
@@ -323,50 +360,111 @@ __global__ void __launch_bounds__(256) k_latent_attn_mfma(LatentAttnArgs a) {
   }
 }
 
-// Merges the splits of one (row, head) and takes the latent through kOutFeatures rows of uv and the output gate.
-constexpr int kOutFeatures = 16;
-template <typename T>
-__global__ void __launch_bounds__(256) k_latent_out(LatentAttnArgs a) {
+// Merges the splits of one (row, head) and takes the latent through `features` rows of uv and the output gate.  With few
+// rows a head's features are shared out over several blocks, each of which merges for itself (what is merged is small and
+// in the L2); with many, one block serves the whole head.  A wave's first weight rows are requested before anything else.
+// R weight rows of C 16-byte chunks per lane are requested at a time.
+template <typename T, int R, int C>
+__global__ void __launch_bounds__(256) k_latent_out(LatentAttnArgs a, int features) {
   constexpr int V = 16 / sizeof(T);
   extern __shared__ __attribute__((aligned(16))) float lo_lds[];   // latents[Rp] | weight[splits]
-  const int h = blockIdx.x, d0 = blockIdx.y * kOutFeatures, m = blockIdx.z;
+  const int h = blockIdx.x, d0 = blockIdx.y * features, m = blockIdx.z;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  float *o = lo_lds, *wt = o + a.Rp;
+  T *o = reinterpret_cast<T *>(lo_lds);
+  float *wt = lo_lds + a.Rp;
   const float *ws = latent_ws(a, m, h, 0);
   const int64_t step = a.Rp + 2;
-  float mx = -INFINITY;
-  for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ws[s * step]);
-  float l = 0.f;
-  for (int s = 0; s < a.splits; ++s) l += ws[s * step + 1] * expf(ws[s * step] - mx);
-  const float inv = 1.0f / l;
-  for (int s = tid; s < a.splits; s += 256) wt[s] = ws[s * step + 1] > 0.f ? expf(ws[s * step] - mx) * inv : 0.f;
-  __syncthreads();
-  for (int r = tid; r < a.Rp; r += 256) {
-    float acc = 0.f;
-    for (int s = 0; s < a.splits; ++s)
-      if (wt[s] > 0.f) acc = fmaf(wt[s], ws[s * step + 2 + r], acc);   // a split without keys has written no latents
-    o[r] = acc;
+  const T *W = (const T *)a.Wuv + ((int64_t)h * a.Dp + d0 + wave * R) * a.Rp + lane * V;   // rows d0 + wave * R + 16 i + r
+  LPack<T> w[R][C], next[R][C];
+  const bool whole = a.Rp <= C * 64 * V;   // one request holds whole rows: the next rows fly while these are multiplied
+  auto request = [&](LPack<T> (&w)[R][C], const T *p, int c0) {
+#pragma unroll
+    for (int r = 0; r < R; ++r)
+#pragma unroll
+      for (int c = 0; c < C; ++c)
+        if ((c0 + c) * 64 * V + lane * V < a.Rp) w[r][c] = *reinterpret_cast<const LPack<T> *>(p + (int64_t)r * a.Rp + (c0 + c) * 64 * V);
+  };
+  request(w, W, 0);
+  // the splits' weights: one split per lane, every wave for itself
+  {
+    constexpr int SL = kLatentBlocks / 64;   // most splits of a lane
+    float ms[SL], ls[SL], mx = -INFINITY, l = 0.f;
+#pragma unroll
+    for (int i = 0; i < SL; ++i) {
+      const int s = lane + i * 64;
+      ms[i] = s < a.splits ? ws[s * step] : -INFINITY;
+      ls[i] = s < a.splits ? ws[s * step + 1] : 0.f;
+      mx = fmaxf(mx, ms[i]);
+    }
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < SL; ++i) {
+      ms[i] = ls[i] > 0.f ? expf(ms[i] - mx) : 0.f;
+      l = fmaf(ls[i], ms[i], l);
+    }
+    const float inv = 1.0f / wave_sum(l);
+    if (wave == 0) {
+#pragma unroll
+      for (int i = 0; i < SL; ++i)
+        if (lane + i * 64 < a.splits) wt[lane + i * 64] = ms[i] * inv;
+    }
   }
   __syncthreads();
-  for (int d = d0 + wave; d < d0 + kOutFeatures; d += 4) {
-    const T *w = (const T *)a.Wuv + ((int64_t)h * a.Dp + d) * a.Rp;
-    float acc = 0.f;
-    for (int r = lane * V; r < a.Rp; r += 64 * V) {
-      const LPack<T> wv = *reinterpret_cast<const LPack<T> *>(w + r);
+  typedef __attribute__((ext_vector_type(2))) float f32x2;
+  for (int r = 2 * tid; r < a.Rp; r += 512) {
+    f32x2 acc = {0.f, 0.f};
+    for (int s0 = 0; s0 < a.splits; s0 += 16) {   // sixteen splits in flight
+      f32x2 x[16];
 #pragma unroll
-      for (int e = 0; e < V; ++e) acc = fmaf(o[r + e], (float)Scalar<T>::load(&wv.v[e]), acc);
+      for (int i = 0; i < 16; ++i) x[i] = *reinterpret_cast<const f32x2 *>(ws + (s0 + i < a.splits ? s0 + i : a.splits - 1) * step + 2 + r);
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const float f = s0 + i < a.splits ? wt[s0 + i] : 0.f;
+        if (f > 0.f) { acc.x = fmaf(f, x[i].x, acc.x); acc.y = fmaf(f, x[i].y, acc.y); }   // a split without keys has written no latents
+      }
     }
-    acc = wave_sum(acc);
-    if (lane == 0) {
-      const float g = (float)Scalar<T>::load((const T *)a.gate + (int64_t)m * a.ldg + h * a.Dp + d);
-      Scalar<T>::store((T *)a.out + (int64_t)m * a.ldo + h * a.Dp + d, acc / (1.0f + expf(-g)));
+    // the merged latent meets uv as the value it stands for would meet the cache: in T
+    Scalar<T>::store(o + r, acc.x);
+    Scalar<T>::store(o + r + 1, acc.y);
+  }
+  __syncthreads();
+  for (int d = d0 + wave * R; d < d0 + features; d += 4 * R, W += (int64_t)4 * R * a.Rp) {
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = 0.f;
+    const bool more = whole && d + 4 * R < d0 + features;
+    if (more) request(next, W + (int64_t)4 * R * a.Rp, 0);
+    for (int c0 = 0; c0 * 64 * V < a.Rp; c0 += C) {
+      if (!whole && (c0 || d != d0 + wave * R)) request(w, W, c0);
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        const int k = (c0 + c) * 64 * V + lane * V;
+        if (k < a.Rp) {
+          const LPack<T> ov = *reinterpret_cast<const LPack<T> *>(o + k);
+#pragma unroll
+          for (int r = 0; r < R; ++r) acc[r] = pack_dot(w[r][c], ov, acc[r]);
+        }
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = wave_sum(acc[r]);
+    if (lane < R) {
+      float v = acc[0];
+#pragma unroll
+      for (int r = 1; r < R; ++r) v = lane == r ? acc[r] : v;
+      const int f = h * a.Dp + d + lane;
+      const float g = (float)Scalar<T>::load((const T *)a.gate + (int64_t)m * a.ldg + f);
+      Scalar<T>::store((T *)a.out + (int64_t)m * a.ldo + f, v / (1.0f + expf(-g)));
+    }
+    if (more) {
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+#pragma unroll
+        for (int c = 0; c < C; ++c) w[r][c] = next[r][c];
     }
   }
 }
 
-// The context is split for about this many blocks: two per CU of the MFMA form (a block serves up to 16 heads), four of
-// the other.
-constexpr int kLatentBlocks = 4 * kNumCU, kLatentMfmaBlocks = 2 * kNumCU;
 size_t latent_attn_ws_floats(int rows, int heads, int Rp) {
   return ((size_t)rows * heads + kLatentBlocks + 16 * kLatentMfmaBlocks) * (Rp + 2);
 }
@@ -419,7 +517,14 @@ template <typename T> static int launch_latent_attention_t(hipStream_t st, Laten
     hipLaunchKernelGGL(k_latent_attn<T>, dim3(a.splits, a.heads, rows), dim3(256), lds, st, a);
     RAI_TRY(launch_check("latent_attn"));
   }
-  hipLaunchKernelGGL(k_latent_out<T>, dim3(a.heads, a.Dp / kOutFeatures, rows), dim3(256), (size_t)(a.Rp + a.splits) * sizeof(float), st, a);
+  const bool narrow = a.Rp <= 64 * (int)(16 / sizeof(T));   // one chunk per lane holds a weight row
+  const bool many = rows * a.heads >= kNumCU;
+  const int features = many ? a.Dp : 16;
+#define RAI_LATENT_OUT(R, C) \
+  hipLaunchKernelGGL((k_latent_out<T, R, C>), dim3(a.heads, a.Dp / features, rows), dim3(256), (size_t)(a.Rp + a.splits) * sizeof(float), st, a, features)
+  if (many) { if (narrow) RAI_LATENT_OUT(8, 1); else RAI_LATENT_OUT(8, 2); }
+  else { if (narrow) RAI_LATENT_OUT(4, 1); else RAI_LATENT_OUT(4, 2); }
+#undef RAI_LATENT_OUT
   return launch_check("latent_out");
 }
 

@@ -249,18 +249,21 @@ struct DownChunk {
   int meta;   // LDS offset | columns << 20
 };
 
-template <int Q>   // chunks a wave has in flight
-__global__ void __launch_bounds__(256) k_latent_down(LatentDownArgs a) {
+// A block of eight waves shares one copy of the activations; a wave owns one output row and has Q chunks in flight, each
+// replaced by the chunk Q places on as soon as it has been multiplied.
+constexpr int kDownWaves = 8, kDownThreads = kDownWaves * 64;
+template <int Q>
+__global__ void __launch_bounds__(kDownThreads) k_latent_down(LatentDownArgs a) {
   extern __shared__ __attribute__((aligned(16))) char dn_lds[];
   const int tid = threadIdx.x, lane = tid & 63;
   const int c0 = (a.K0 + 511) / 512, c1 = (a.K1 + 511) / 512, chunks = c0 + a.top * c1;
   const int Kt = a.K0 + a.top * a.K1;
   DownChunk *table = reinterpret_cast<DownChunk *>(dn_lds);
   uint16_t *xs = reinterpret_cast<uint16_t *>(table + chunks);
-  const int n = blockIdx.x * 4 + (tid >> 6);
+  const int n = blockIdx.x * kDownWaves + (tid >> 6);
   float res = 0.f;
   if (n < a.H) res = a.res_f32 ? ((const float *)a.res)[n] : bf16_bits_to_f32(((const uint16_t *)a.res)[n]);
-  for (int c = tid; c < chunks; c += 256) {
+  for (int c = tid; c < chunks; c += kDownThreads) {
     DownChunk d;
     if (c < c0) {
       d.w = (const uint16_t *)a.W0 + c * 512;
@@ -276,39 +279,38 @@ __global__ void __launch_bounds__(256) k_latent_down(LatentDownArgs a) {
   }
   __syncthreads();
   ld_u32x4 w[Q];
-  auto request = [&](int first) {
-#pragma unroll
-    for (int u = 0; u < Q; ++u) {
-      const int c = first + u;
-      w[u] = ld_u32x4{0u, 0u, 0u, 0u};
-      if (c < chunks) {
-        const DownChunk d = table[c];
-        if (lane * 8 < (d.meta >> 20) && n < a.N) w[u] = __builtin_nontemporal_load(reinterpret_cast<const ld_u32x4 *>(d.w + (int64_t)n * d.ld + lane * 8));
-      }
+  auto request = [&](ld_u32x4 &dst, int c) {
+    if (c < chunks) {
+      const DownChunk d = table[c];
+      if (lane * 8 < (d.meta >> 20) && n < a.N) dst = __builtin_nontemporal_load(reinterpret_cast<const ld_u32x4 *>(d.w + (int64_t)n * d.ld + lane * 8));
     }
   };
   // the activations come from the L2 and are asked for first; they reach LDS while the weights are on their way
-  constexpr int XP = 6;
+  constexpr int XP = 3;
   ld_u32x4 xp[XP];
   auto x_at = [&](int k) { return *reinterpret_cast<const ld_u32x4 *>(k < a.K0 ? (const uint16_t *)a.x0 + k : (const uint16_t *)a.x1 + (k - a.K0)); };
 #pragma unroll
   for (int i = 0; i < XP; ++i)
-    if ((tid + i * 256) * 8 < Kt) xp[i] = x_at((tid + i * 256) * 8);
-  request(0);
+    if ((tid + i * kDownThreads) * 8 < Kt) xp[i] = x_at((tid + i * kDownThreads) * 8);
+#pragma unroll
+  for (int u = 0; u < Q; ++u) {
+    w[u] = ld_u32x4{0u, 0u, 0u, 0u};
+    request(w[u], u);
+  }
 #pragma unroll
   for (int i = 0; i < XP; ++i)
-    if ((tid + i * 256) * 8 < Kt) *reinterpret_cast<ld_u32x4 *>(xs + (tid + i * 256) * 8) = xp[i];
-  for (int k = (tid + XP * 256) * 8; k < Kt; k += 256 * 8) *reinterpret_cast<ld_u32x4 *>(xs + k) = x_at(k);
+    if ((tid + i * kDownThreads) * 8 < Kt) *reinterpret_cast<ld_u32x4 *>(xs + (tid + i * kDownThreads) * 8) = xp[i];
+  for (int k = (tid + XP * kDownThreads) * 8; k < Kt; k += kDownThreads * 8) *reinterpret_cast<ld_u32x4 *>(xs + k) = x_at(k);
   __syncthreads();
   float acc = 0.f;
   for (int first = 0; first < chunks; first += Q) {
-    if (first) request(first);
 #pragma unroll
     for (int u = 0; u < Q; ++u) {
       const int c = first + u;
       if (c < chunks) {
         const int meta = table[c].meta;
         if (lane * 8 < (meta >> 20)) acc = ld_dot8(w[u], *reinterpret_cast<const ld_u32x4 *>(xs + (meta & 0xfffff) + lane * 8), acc);
+        request(w[u], c + Q);
       }
     }
   }
@@ -363,7 +365,7 @@ template <int Q> static int launch_latent_down_q(hipStream_t st, const LatentDow
     RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_latent_down<Q>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024));
     attr_set = true;
   }
-  hipLaunchKernelGGL(k_latent_down<Q>, dim3((a.N + 3) / 4), dim3(256), lds, st, a);
+  hipLaunchKernelGGL(k_latent_down<Q>, dim3((a.N + kDownWaves - 1) / kDownWaves), dim3(kDownThreads), lds, st, a);
   return launch_check("latent_down");
 }
 int launch_latent_down(hipStream_t st, const LatentDownArgs &a) {
@@ -372,8 +374,8 @@ int launch_latent_down(hipStream_t st, const LatentDownArgs &a) {
   RAI_REQUIRE(lds <= 150 * 1024 && a.K0 % 8 == 0 && a.K1 % 8 == 0, RAI_ERR_UNSUPPORTED, "latent down: %d + %d x %d columns", a.K0, a.top, a.K1);
   if (chunks <= 8) return launch_latent_down_q<8>(st, a, lds);
   if (chunks <= 16) return launch_latent_down_q<16>(st, a, lds);
-  if (chunks <= 24) return launch_latent_down_q<24>(st, a, lds);
-  return launch_latent_down_q<32>(st, a, lds);
+  if (chunks > 16 && chunks <= 24) return launch_latent_down_q<24>(st, a, lds);
+  return launch_latent_down_q<16>(st, a, lds);
 }
 
 }  // namespace rai

@@ -68,6 +68,25 @@ def load_random_params(decoder, seed=0, std=0.02, workers=8):
                 pending.append(ex.submit(make, nxt))
 
 
+def is_norm_weight(name):
+    return name.endswith("norm.weight") or name.rsplit(".", 1)[-1] in ("norm", "norm1", "norm2")
+
+
+def load_tiled_params(decoder, seed=0, std=0.02, block=1 << 24):
+    """load_random_params for large models of which only the timing matters: every matrix is cut from one block of
+    N(0, std) values, each from another place of it, so that generating gigabytes does not take the host minutes."""
+    rng = np.random.Generator(np.random.PCG64(seed))
+    values = to_storage(rng.standard_normal(block, dtype=np.float32) * np.float32(std), decoder.dtype)
+    for name, numel in decoder.param_names().items():
+        if is_norm_weight(name):
+            a = to_storage(np.ones(numel, np.float32), decoder.dtype)
+        elif name.endswith(".bias"):
+            a = to_storage(np.zeros(numel, np.float32), decoder.dtype)
+        else:
+            a = np.resize(np.roll(values, -(zlib.crc32(name.encode()) % block)), numel)
+        decoder.load_param(name, a)
+
+
 def prompt(vocab_size, batch, length, seed=1):
     rng = np.random.Generator(np.random.PCG64(seed))
     return rng.integers(0, vocab_size, (batch, length)).astype(np.uint32)
