@@ -120,7 +120,7 @@ static int create_latent(rai_hip_decoder *d, const rai_hip_latent_config &cfg, c
   // activations, sized for the widest layer
   int Qp = 0, Rp = 0, QD = 0, ldn = 0, KB = 0, EFp = 0, experts = 0;
   size_t ws = 0;
-  int64_t top = 0, tiles = 0;
+  int64_t top = 0, tiles = 0, counts = 0;
   const int64_t rows = d->max_rows;
   const int64_t absorb_rows = std::min<int64_t>(rows, (int64_t)cfg.max_batch * (kAbsorbRows - 1));
   size_t qa = 0;
@@ -134,6 +134,7 @@ static int create_latent(rai_hip_decoder *d, const rai_hip_latent_config &cfg, c
       experts = std::max(experts, y.c.experts);
       top = std::max<int64_t>(top, y.c.top);
       tiles = std::max<int64_t>(tiles, moe_max_tiles(rows * y.c.top, y.c.experts, bm));
+      counts = std::max(counts, moe_plan_counts(rows * y.c.top, y.c.experts));
     }
   }
   char *tmp = nullptr;
@@ -167,6 +168,8 @@ static int create_latent(rai_hip_decoder *d, const rai_hip_latent_config &cfg, c
     lm.rpos = (int *)tmp;
     RAI_TRY(zalloc(d, slots * sizeof(int), &tmp));
     lm.plan.slot_of = (int *)tmp;
+    RAI_TRY(zalloc(d, counts * sizeof(int), &tmp));
+    lm.plan.counts = (int *)tmp;
     RAI_TRY(zalloc(d, tiles * sizeof(int4), &tmp));
     lm.plan.tiles = (int4 *)tmp;
     RAI_TRY(zalloc(d, sizeof(int), &tmp));
@@ -269,8 +272,9 @@ static int absorbed_attention(rai_hip_decoder *d, hipStream_t st, const LatentLa
   return launch_latent_attention(st, d->cfg.dtype, t);
 }
 
-// Leaves the experts' outputs in lm.eout, row lm.rpos[token * top + j].
-static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int64_t M) {
+// Adds the mixture to the stream when *pending comes back null; otherwise leaves the experts' outputs in lm.eout, row
+// lm.rpos[token * top + j], for the next stream norm to add.
+static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int64_t M, const LatentLayer **pending) {
   LatentModel &lm = *d->latent;
   const int dt = d->cfg.dtype, Hp = lm.Hp, top = y.c.top;
   LinearArgs r = latent_linear_args(d, lm.h2, Hp, M, y.Wr, y.c.experts, Hp);
@@ -279,6 +283,23 @@ static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int
   RAI_TRY(decoder_linear(d, st, r));
   RAI_TRY(launch_moe_route(st, lm.rlogits, M, y.c.experts, top, lm.rchoice, lm.rweight));
   const int64_t slots = M * top;
+  const int64_t gs = (int64_t)2 * y.EFp * Hp, os = (int64_t)Hp * y.EFp;
+  if (dt == RAI_BF16 && moe_slots_serves(slots, Hp, top, y.EFp)) {
+    MoeSlotsArgs m;
+    memset(&m, 0, sizeof(m));
+    m.h = lm.h2; m.ld = Hp; m.slots = (int)slots; m.top = top; m.choice = lm.rchoice; m.weight = lm.rweight;
+    m.We_gu = y.We_gu; m.Hp = Hp; m.EFp = y.EFp; m.act = y.c.mlp_act; m.gu_stride = gs; m.eact = lm.eact;
+    RAI_TRY(launch_moe_slots(st, m));
+    LatentDownArgs dn;
+    memset(&dn, 0, sizeof(dn));
+    dn.x1 = lm.eact; dn.W1 = y.We_dn; dn.K1 = y.EFp; dn.top = top; dn.stride1 = os; dn.choice = lm.rchoice;
+    dn.res = lm.xs; dn.res_f32 = 1; dn.H = d->H; dn.N = Hp; dn.rows = (int)M;
+    dn.mult = (float)lm.c.residual_mult;
+    dn.out = lm.xs;
+    *pending = nullptr;
+    return launch_latent_down(st, dn);
+  }
+  *pending = &y;
   const int bm = linear_grouped_rows(dt, slots, y.c.experts);
   MoePlan plan = lm.plan;
   plan.cap_tiles = moe_max_tiles(slots, y.c.experts, bm);
@@ -289,7 +310,6 @@ static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int
   g.act = y.c.mlp_act; g.act_from = 0; g.glu = 1;
   LinearArgs o = latent_linear_args(d, lm.eact, y.EFp, slots, y.We_dn, Hp, y.EFp);
   o.out1 = lm.eout; o.ld1 = Hp;
-  const int64_t gs = (int64_t)2 * y.EFp * Hp, os = (int64_t)Hp * y.EFp;
   if (dt == RAI_BF16) {
     RAI_TRY(launch_linear_bf16_grouped(st, g, gs, plan, bm));
     return launch_linear_bf16_grouped(st, o, os, plan, bm);
@@ -321,13 +341,14 @@ static void add_pending(rai_hip_decoder *d, const LatentLayer *y, StreamNormArgs
 // One bf16 row: six launches a layer, nothing materialised between a norm and the product it feeds.
 static bool single_row_ok(const rai_hip_decoder *d) {
   const LatentModel &lm = *d->latent;
-  int rank = 0;
+  int rank = 0, experts = 0;
   int64_t cols = 0;
   for (const LatentLayer &y : lm.layers) {
     rank = std::max(rank, std::max(y.Qp, y.Rp));
+    if (y.c.mlp_kind == RAI_MLP_MIXTURE) experts = std::max(experts, y.c.experts);
     cols = std::max<int64_t>(cols, y.QD + y.Fp + (int64_t)y.c.top * y.EFp);
   }
-  return d->cfg.dtype == RAI_BF16 && latent_single_row_serves(d->H, lm.c.norm_groups, rank, cols);
+  return d->cfg.dtype == RAI_BF16 && latent_single_row_serves(d->H, lm.c.norm_groups, rank, experts, cols);
 }
 
 static int single_row_layers(rai_hip_decoder *d, hipStream_t st) {
@@ -365,7 +386,7 @@ static int single_row_layers(rai_hip_decoder *d, hipStream_t st) {
     memset(&dn, 0, sizeof(dn));
     dn.x0 = lm.cat; dn.W0 = y.Wb; dn.K0 = y.QD + y.Fp;
     if (moe) { dn.x1 = lm.eact; dn.W1 = y.We_dn; dn.K1 = y.EFp; dn.top = y.c.top; dn.stride1 = (int64_t)lm.Hp * y.EFp; dn.choice = lm.rchoice; }
-    dn.res = src; dn.res_f32 = l > 0; dn.H = d->H; dn.N = lm.Hp;
+    dn.res = src; dn.res_f32 = l > 0; dn.H = d->H; dn.N = lm.Hp; dn.rows = 1;
     dn.mult = (float)lm.c.residual_mult;
     dn.out = lm.xs;
     RAI_TRY(launch_latent_down(st, dn));
@@ -440,8 +461,7 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
     }
     RAI_TRY(residual_linear(d, st, lm.cat, y.QD + y.Fp, M, y.Wb, y.QD + y.Fp, frag ? y.Wb_f : nullptr));
     if (y.c.mlp_kind == RAI_MLP_MIXTURE) {
-      RAI_TRY(mixture(d, st, y, M));
-      pending = &y;
+      RAI_TRY(mixture(d, st, y, M, &pending));
     }
   }
 

@@ -109,6 +109,22 @@ struct LatentMidArgs {
   int waves_q, waves_e, rows_per_wave;   // filled in by the launcher
 };
 int launch_latent_mid(hipStream_t st, LatentMidArgs a);
+// Few rows of a mixture: gated rows of every slot's expert on weight[slot] * h[slot / top] -> eact [slots, EFp]
+struct MoeSlotsArgs {
+  const void *h;                // [tokens] rows, ld apart
+  int64_t ld;
+  int slots, top;
+  const int *choice;
+  const float *weight;
+  const void *We_gu;
+  int Hp, EFp, act;
+  int64_t gu_stride;
+  void *eact;
+  int waves_e, rows_per_wave;   // filled in by the launcher
+};
+bool moe_slots_serves(int64_t slots, int Hp, int top, int EFp);
+int launch_moe_slots(hipStream_t st, MoeSlotsArgs a);
+// For each of `rows` rows (x0, x1, choice, res and out dense, row by row):
 // out[n] = res[n] + mult * (W0[n] . x0 + sum_j W1[choice[j]][n] . x1[j]); rows of W0 (W1) are K0 (K1) long
 struct LatentDownArgs {
   const void *x0, *W0;
@@ -118,12 +134,12 @@ struct LatentDownArgs {
   int64_t stride1;
   const int *choice;
   const void *res;
-  int res_f32, H, N;
+  int res_f32, H, N, rows;
   float mult;
   float *out;
 };
 int launch_latent_down(hipStream_t st, const LatentDownArgs &a);
-bool latent_single_row_serves(int width, int groups, int max_rank, int64_t down_columns);
+bool latent_single_row_serves(int width, int groups, int max_rank, int max_experts, int64_t down_columns);
 
 // ---- mixture of experts
 // Device-side plan of one mixture: the (token, choice) slots sorted by expert, cut into row tiles of `bm`.
@@ -131,9 +147,13 @@ struct MoePlan {
   int4 *tiles;     // {expert, first sorted row, rows, 0}
   int *n_tiles;    // device count
   int *slot_of;    // sorted row -> slot
+  int *counts;     // scratch, moe_plan_counts()
   int cap_tiles;
 };
 int moe_max_tiles(int64_t slots, int experts, int bm);
+constexpr int64_t kPlanFewSlots = 8192;   // up to here the plan is one launch
+constexpr int kPlanExperts = 2048;
+int64_t moe_plan_counts(int64_t slots, int experts);   // ints
 // choice[t * top + j], weight[t * top + j]: the `top` largest sigmoid scores of the token's logits, in decreasing order.
 int launch_moe_route(hipStream_t st, const float *logits, int64_t tokens, int experts, int top, int *choice, float *weight);
 int launch_moe_plan(hipStream_t st, const int *choice, int64_t slots, int experts, int bm, const MoePlan &plan, int *row_of_slot);

@@ -10,6 +10,7 @@
 #include <cstdlib>
 
 #include "latent.h"
+#include "moe.h"
 
 namespace rai {
 
@@ -144,28 +145,57 @@ __global__ void __launch_bounds__(256) k_latent_in(LatentInArgs a) {
   });
 }
 
-// The j-th best of the wave's logits and its score, by the rule of k_moe_route.
-__device__ __forceinline__ int nth_expert(const float *z, int experts, int j, int lane, float *score) {
-  uint32_t taken = 0;
-  float bv = 0.f;
-  int bi = 0;
-  for (int t = 0; t <= j; ++t) {
-    bv = -INFINITY;
-    bi = 0x7fffffff;
-    for (int i = 0; lane + i * 64 < experts; ++i) {
-      const float v = z[lane + i * 64];
-      if (!((taken >> i) & 1u) && (v > bv || bi == 0x7fffffff)) { bv = v; bi = lane + i * 64; }
-    }
+// The expert of rank j among the logits, and its score (the choice of k_moe_route_ranked).
+template <int N> __device__ __forceinline__ int nth_of(const float *z, int experts, int j, int lane, float *score) {
+  float v[N];
+  int rank[N], e = 0;
+  float zj = 0.f;
+  rank_experts<N>(z, experts, lane, v, rank);
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64);
-      const int oi = __shfl_xor(bi, o, 64);
-      if (oi != 0x7fffffff && (bi == 0x7fffffff || ov > bv || (ov == bv && oi < bi))) { bv = ov; bi = oi; }
+  for (int i = 0; i < N; ++i) {
+    const unsigned long long hit = __ballot(rank[i] == j);
+    if (hit) {   // exactly one lane of one i
+      const int l = __ffsll(hit) - 1;
+      e = 64 * i + l;
+      zj = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v[i]), l));
     }
-    if ((bi & 63) == lane) taken |= 1u << (bi >> 6);
   }
-  *score = 1.0f / (1.0f + expf(-bv));
-  return __builtin_amdgcn_readfirstlane(bi);
+  *score = router_score(zj);
+  return __builtin_amdgcn_readfirstlane(e);
+}
+__device__ __forceinline__ int nth_expert(const float *z, int experts, int j, int lane, float *score) {
+  if (experts <= 64) return nth_of<1>(z, experts, j, lane, score);
+  if (experts <= 128) return nth_of<2>(z, experts, j, lane, score);
+  return nth_of<4>(z, experts, j, lane, score);
+}
+
+// Gated rows [n0, n1) of one expert on score * h, to out[n / 2].
+template <int KC>
+__device__ __forceinline__ void expert_rows(const uint16_t *h, const uint16_t *W, int K, int n0, int n1, float score, int act, uint16_t *out, int lane) {
+  ld_u32x4 xv[KC];
+#pragma unroll
+  for (int u = 0; u < KC; ++u)
+    xv[u] = lane * 8 + u * 512 < K ? *reinterpret_cast<const ld_u32x4 *>(h + lane * 8 + u * 512) : ld_u32x4{0u, 0u, 0u, 0u};
+  RowSet<KC, 2> rs;
+  rs.load(W, K, n0, n1 - 1, K, lane);
+#pragma unroll
+  for (int u = 0; u < KC; ++u)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) xv[u][i] = pack_bf16x2(score * lo_f32(xv[u][i]), score * hi_f32(xv[u][i]));
+  stream_rows<KC>(rs, xv, W, K, n0, n1, K, lane, [&](int n, float v0, float v1) { out[n >> 1] = f32_to_bf16_bits(gated(act, v0, v1)); });
+}
+
+// Few rows: every (token, choice) slot is a product of its own, the expert's weights shared through the caches where two
+// tokens chose it.
+template <int KC>
+__global__ void __launch_bounds__(256) k_moe_slots(MoeSlotsArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int gw = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
+  const int slot = gw / a.waves_e, n0 = (gw - slot * a.waves_e) * a.rows_per_wave, N = 2 * a.EFp;
+  if (slot >= a.slots) return;
+  const int n1 = n0 + a.rows_per_wave < N ? n0 + a.rows_per_wave : N;
+  expert_rows<KC>((const uint16_t *)a.h + (int64_t)(slot / a.top) * a.ld, (const uint16_t *)a.We_gu + (int64_t)a.choice[slot] * a.gu_stride, a.Hp, n0, n1,
+                  a.weight[slot], a.act, (uint16_t *)a.eact + (int64_t)slot * a.EFp, lane);
 }
 
 template <int KC>
@@ -224,21 +254,11 @@ __global__ void __launch_bounds__(256) k_latent_mid(LatentMidArgs a) {
   gw -= a.waves_q;
   const int slot = gw / a.waves_e, n0 = (gw - slot * a.waves_e) * a.rows_per_wave, N = 2 * a.EFp;
   const int n1 = n0 + a.rows_per_wave < N ? n0 + a.rows_per_wave : N;
-#pragma unroll
-  for (int u = 0; u < KC; ++u)
-    xv[u] = lane * 8 + u * 512 < a.Hp ? *reinterpret_cast<const ld_u32x4 *>((const uint16_t *)a.h2 + lane * 8 + u * 512) : ld_u32x4{0u, 0u, 0u, 0u};
   float score;
   const int e = nth_expert(a.rlogits, a.experts, slot, lane, &score);
   if (n0 == 0 && lane == 0) a.choice[slot] = e;
-  const uint16_t *W = (const uint16_t *)a.We_gu + (int64_t)e * a.gu_stride;
-  RowSet<KC, 2> rs;
-  rs.load(W, a.Hp, n0, n1 - 1, a.Hp, lane);
-#pragma unroll
-  for (int u = 0; u < KC; ++u)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) xv[u][i] = pack_bf16x2(score * lo_f32(xv[u][i]), score * hi_f32(xv[u][i]));
-  uint16_t *out = (uint16_t *)a.eact + (int64_t)slot * a.EFp;
-  stream_rows<KC>(rs, xv, W, a.Hp, n0, n1, a.Hp, lane, [&](int n, float v0, float v1) { out[n >> 1] = f32_to_bf16_bits(gated(a.act, v0, v1)); });
+  expert_rows<KC>((const uint16_t *)a.h2, (const uint16_t *)a.We_gu + (int64_t)e * a.gu_stride, a.Hp, n0, n1, score, a.act,
+                  (uint16_t *)a.eact + (int64_t)slot * a.EFp, lane);
 }
 
 // Chunks of up to 512 columns of the concatenated contraction: where the weights of row 0 are, the row stride, where the
@@ -256,6 +276,14 @@ template <int Q>
 __global__ void __launch_bounds__(kDownThreads) k_latent_down(LatentDownArgs a) {
   extern __shared__ __attribute__((aligned(16))) char dn_lds[];
   const int tid = threadIdx.x, lane = tid & 63;
+  {   // this block's row
+    const int64_t m = blockIdx.y;
+    a.x0 = (const uint16_t *)a.x0 + m * a.K0;
+    a.x1 = (const uint16_t *)a.x1 + m * a.top * a.K1;
+    if (a.top) a.choice += m * a.top;
+    a.res = a.res_f32 ? (const void *)((const float *)a.res + m * a.N) : (const void *)((const uint16_t *)a.res + m * a.H);
+    a.out += m * a.N;
+  }
   const int c0 = (a.K0 + 511) / 512, c1 = (a.K1 + 511) / 512, chunks = c0 + a.top * c1;
   const int Kt = a.K0 + a.top * a.K1;
   DownChunk *table = reinterpret_cast<DownChunk *>(dn_lds);
@@ -319,10 +347,10 @@ __global__ void __launch_bounds__(kDownThreads) k_latent_down(LatentDownArgs a) 
 }
 
 // ---------------------------------------------------------------- launchers
-bool latent_single_row_serves(int width, int groups, int max_rank, int64_t down_columns) {
+bool latent_single_row_serves(int width, int groups, int max_rank, int max_experts, int64_t down_columns) {
   const char *off = getenv("RAI_HIP_NO_LATENT_FUSED");   // read per call: the tests compare both forms in one process
   if (off && *off && *off != '0') return false;
-  return width % 8 == 0 && width <= 4096 && groups <= 16 && (width / groups) % 8 == 0 && max_rank <= 4096 && down_columns * 2 + 16 * 1024 <= 150 * 1024;
+  return width % 8 == 0 && width <= 4096 && groups <= 16 && (width / groups) % 8 == 0 && max_rank <= 4096 && max_experts <= kRankedExperts && down_columns * 2 + 16 * 1024 <= 150 * 1024;
 }
 
 int launch_latent_in(hipStream_t st, LatentInArgs a) {
@@ -359,13 +387,31 @@ int launch_latent_mid(hipStream_t st, LatentMidArgs a) {
   return launch_check("latent_mid");
 }
 
+bool moe_slots_serves(int64_t slots, int Hp, int top, int EFp) {
+  const char *off = getenv("RAI_HIP_NO_LATENT_FUSED");   // read per call: the tests compare both forms in one process
+  if (off && *off && *off != '0') return false;
+  return slots <= 64 && Hp <= 4096 && (int64_t)top * EFp * 2 + 16 * 1024 <= 150 * 1024;
+}
+int launch_moe_slots(hipStream_t st, MoeSlotsArgs a) {
+  int rpw = (a.slots * 2 * a.EFp + kNumCU * 16 - 1) / (kNumCU * 16);
+  a.rows_per_wave = rpw < 2 ? 2 : (rpw + 1) / 2 * 2;
+  a.waves_e = (2 * a.EFp + a.rows_per_wave - 1) / a.rows_per_wave;
+  const dim3 grid((a.slots * a.waves_e + 3) / 4), block(256);
+  if (a.Hp <= 512) hipLaunchKernelGGL(k_moe_slots<1>, grid, block, 0, st, a);
+  else if (a.Hp <= 1024) hipLaunchKernelGGL(k_moe_slots<2>, grid, block, 0, st, a);
+  else if (a.Hp <= 2048) hipLaunchKernelGGL(k_moe_slots<4>, grid, block, 0, st, a);
+  else if (a.Hp <= 2560) hipLaunchKernelGGL(k_moe_slots<5>, grid, block, 0, st, a);
+  else hipLaunchKernelGGL(k_moe_slots<8>, grid, block, 0, st, a);
+  return launch_check("moe_slots");
+}
+
 template <int Q> static int launch_latent_down_q(hipStream_t st, const LatentDownArgs &a, size_t lds) {
   static bool attr_set = false;
   if (!attr_set) {
     RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_latent_down<Q>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024));
     attr_set = true;
   }
-  hipLaunchKernelGGL(k_latent_down<Q>, dim3((a.N + kDownWaves - 1) / kDownWaves), dim3(kDownThreads), lds, st, a);
+  hipLaunchKernelGGL(k_latent_down<Q>, dim3((a.N + kDownWaves - 1) / kDownWaves, a.rows), dim3(kDownThreads), lds, st, a);
   return launch_check("latent_down");
 }
 int launch_latent_down(hipStream_t st, const LatentDownArgs &a) {

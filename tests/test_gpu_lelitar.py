@@ -80,6 +80,8 @@ SIZES = {
                                  lm.layer(heads=2, dim=3, vdim=9, q_rank=13, kv_rank=5, window=2, mlp="moe", ff=3, experts=5, top=5, scale=0.5)],
                                 vocab=77, width=33, groups=11),
     "window 1": lm.config([lm.layer(window=1), lm.layer(window=1, mlp="moe")]),
+    "130 experts": lm.config([lm.layer(mlp="moe", experts=130, top=3, ff=16), lm.layer(mlp="moe", experts=65, top=2, ff=24)]),
+    "300 experts": lm.config([lm.layer(mlp="moe", experts=300, top=5, ff=16)]),
     "every expert": lm.config([lm.layer(mlp="moe", experts=4, top=4)]),
     "wide": lm.config([lm.layer(heads=20, dim=128, vdim=128, q_rank=768, kv_rank=512, window=100, ff=1024, scale=0.088)], width=2304, groups=9),
 }
@@ -186,7 +188,7 @@ def test_far_key_without_a_window(hip, dt, far):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("batch,n", [(1, 1), (1, 6), (1, 200), (9, 40), (3, 130)])
+@pytest.mark.parametrize("batch,n", [(1, 1), (1, 6), (1, 200), (9, 40), (3, 130), (4, 1100)])
 def test_uneven_experts(hip, dt, batch, n):
     """A router that sends nearly every token to the same two of many experts: full and partial row tiles, experts
     without rows, more rows than one tile."""
@@ -197,10 +199,28 @@ def test_uneven_experts(hip, dt, batch, n):
     p["l0.mlp.router"][31, 0] = 3.0
     p["l0.mlp.router"][5, 0] = 2.0
     p = {k: rnd(v, dt) for k, v in p.items()}
-    dec, ids = lm.build(cfg, p, dt, max_batch=batch), tokens(cfg, (batch, n), 14)
+    dec, ids = lm.build(cfg, p, dt, max_batch=batch, max_context=max(64, n)), tokens(cfg, (batch, n), 14)
     got = lm.run_portions(dec, ids, [n])
     for b in range(batch):
         assert_close(got[b], lelitar.Model(cfg, p).logits(ids[b]), dt, f"row {b}")
+    dec.close()
+
+
+@pytest.mark.parametrize("switch", ["RAI_HIP_NO_LATENT_FUSED", "RAI_HIP_NO_LATENT_MFMA"])
+def test_the_plain_forms_of_the_bf16_kernels(hip, monkeypatch, switch):
+    """The launches without folded-in norms and routing, and the absorbed attention without MFMA, against the
+    restatement and against the forms that normally run."""
+    cfg = lm.mixed_config()
+    p = lm.random_params(cfg, "bf16", 23)
+    dec, ids = lm.build(cfg, p, "bf16", max_batch=3), tokens(cfg, (3, 40), 24)
+    want = np.stack([lelitar.Model(cfg, p).logits(r) for r in ids])
+    usual = [lm.run_portions(dec, ids, [30, 1]), lm.run_portions(dec, ids[:1], [33, 1])]
+    monkeypatch.setenv(switch, "1")
+    plain = [lm.run_portions(dec, ids, [30, 1]), lm.run_portions(dec, ids[:1], [33, 1])]
+    for a, b in zip(usual, plain):
+        assert_close(a, want[:len(a)], "bf16", "usual forms")
+        assert_close(b, want[:len(b)], "bf16", f"{switch}=1")
+        assert_close(b, a, "bf16", "one against the other")
     dec.close()
 
 
