@@ -54,8 +54,8 @@ struct LatentLayer {
   char *Wb;                    // [Hp, QD + Fp]: o | down as one contraction (Fp = 0 without a dense MLP)
   char *Wr;                    // mixture: router [experts, Hp]
   char *We_gu, *We_dn;         // [experts][2 EFp, Hp] interleaved, [experts][Hp, EFp]
-  // Wd, Wuq, Wgu and Wb in MFMA-fragment order for 9 .. 64 rows (built on first use)
-  char *Wd_f, *Wuq_f, *Wgu_f, *Wb_f;
+  // Wd, Wuq, Wgu, Wb and Wr in MFMA-fragment order for 9 .. 64 rows (built on first use)
+  char *Wd_f, *Wuq_f, *Wgu_f, *Wb_f, *Wr_f;
   char *cache;                 // [max_batch][max_context][Rp] normalised latents
 };
 

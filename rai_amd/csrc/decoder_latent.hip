@@ -199,6 +199,7 @@ static int ensure_latent_fragments(rai_hip_decoder *d, hipStream_t st) {
     RAI_TRY(decoder_fragments(d, st, y.Wuq, y.Qp, y.QD, y.Qp, &y.Wuq_f));
     RAI_TRY(decoder_fragments(d, st, y.Wgu, lm.Hp, 2 * y.Fp, lm.Hp, &y.Wgu_f));
     RAI_TRY(decoder_fragments(d, st, y.Wb, KB, lm.Hp, KB, &y.Wb_f));
+    RAI_TRY(decoder_fragments(d, st, y.Wr, lm.Hp, y.c.experts, lm.Hp, &y.Wr_f));
   }
   RAI_TRY(decoder_fragments(d, st, d->head_w, lm.Hp, d->V, lm.Hp, &d->head_f));
   d->frag_ready = true;
@@ -280,11 +281,12 @@ static int mixture(rai_hip_decoder *d, hipStream_t st, const LatentLayer &y, int
   LinearArgs r = latent_linear_args(d, lm.h2, Hp, M, y.Wr, y.c.experts, Hp);
   r.out1 = lm.rlogits; r.ld1 = y.c.experts;
   r.f32_out = 1; r.out_scale = 1.f;
+  r.Wfrag = wants_fragments(d, M) ? y.Wr_f : nullptr;
   RAI_TRY(decoder_linear(d, st, r));
   RAI_TRY(launch_moe_route(st, lm.rlogits, M, y.c.experts, top, lm.rchoice, lm.rweight));
   const int64_t slots = M * top;
   const int64_t gs = (int64_t)2 * y.EFp * Hp, os = (int64_t)Hp * y.EFp;
-  if (dt == RAI_BF16 && moe_slots_serves(slots, Hp, top, y.EFp)) {
+  if (dt == RAI_BF16 && moe_slots_serves(slots, y.c.experts, Hp, top, y.EFp)) {
     MoeSlotsArgs m;
     memset(&m, 0, sizeof(m));
     m.h = lm.h2; m.ld = Hp; m.slots = (int)slots; m.top = top; m.choice = lm.rchoice; m.weight = lm.rweight;

@@ -1458,7 +1458,8 @@ __device__ __forceinline__ f32x4 load_f32x4_device(const float *p) {
                __uint_as_float((uint32_t)(hi >> 32))};
 }
 
-template <int MT, int KS, int G, bool FRAG>
+// F32O: the f32 output of LinearArgs::f32_out (fragment-order weights only; a branch in the bf16 form costs it 1 %)
+template <int MT, int KS, int G, bool FRAG, bool F32O>
 __global__ void __launch_bounds__(512) k_linear_bf16_mfma_stream(LinearArgs a, int tiles, float *partial, int *tickets) {
   __shared__ int s_ticket;
   constexpr int NW = 8;
@@ -1591,7 +1592,7 @@ __global__ void __launch_bounds__(512) k_linear_bf16_mfma_stream(LinearArgs a, i
       else { dst[0] = o[0]; dst[1] = o[1]; }
       return;
     }
-    if (a.f32_out) {
+    if constexpr (F32O) {
       float *dst = (float *)a.out1 + (int64_t)m * a.ld1 + n;
       const float *rsrc = res ? (const float *)a.residual + (int64_t)m * a.ldr + n : nullptr;
 #pragma unroll
@@ -1725,9 +1726,10 @@ __global__ void __launch_bounds__(512) k_linear_bf16_mfma_stream(LinearArgs a, i
   }
 }
 
-template <int MT, int KS, int G, bool FRAG = false>
+template <int MT, int KS, int G, bool FRAG = false, bool F32O = false>
 static int launch_mfma_stream_cfg(hipStream_t st, const LinearArgs &a, int splits) {
   if constexpr (!FRAG) {
+    if (a.f32_out) return launch_mfma_stream_cfg<MT, KS, G, true, true>(st, a, splits);
     if (a.Wfrag) return launch_mfma_stream_cfg<MT, KS, G, true>(st, a, splits);
   }
   const int tiles = (a.N + 15) / 16;
@@ -1738,7 +1740,7 @@ static int launch_mfma_stream_cfg(hipStream_t st, const LinearArgs &a, int split
   const size_t lds = (size_t)8 * MT * 16 * (4 * G + 1) * sizeof(f32x4);
   static bool attr_set = false;
   if (lds > 64 * 1024 && !attr_set) {
-    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_linear_bf16_mfma_stream<MT, KS, G, FRAG>,
+    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_linear_bf16_mfma_stream<MT, KS, G, FRAG, F32O>,
                                     hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     attr_set = true;
   }
@@ -1751,7 +1753,7 @@ static int launch_mfma_stream_cfg(hipStream_t st, const LinearArgs &a, int split
     int dev = -1;
     if (linear_device(a, &dev) == RAI_OK) tickets = splitk_tickets_of(dev);
   }
-  hipLaunchKernelGGL((k_linear_bf16_mfma_stream<MT, KS, G, FRAG>), dim3(blocks_x, splits), dim3(512), lds, st, a, tiles,
+  hipLaunchKernelGGL((k_linear_bf16_mfma_stream<MT, KS, G, FRAG, F32O>), dim3(blocks_x, splits), dim3(512), lds, st, a, tiles,
                      partial, tickets);
   RAI_TRY(launch_check("linear_bf16_mfma_stream"));
   if (splits > 1 && !tickets) {
@@ -1874,7 +1876,7 @@ int launch_linear_bf16_mfma(hipStream_t st, const LinearArgs &a) {
               RAI_ERR_BAD_STRIDE, "linear mfma: operands must be 16-byte aligned with row strides multiple of 8");
   const bool no_skinny = getenv("RAI_HIP_NO_MFMA_SKINNY") != nullptr;
   const bool no_stream = getenv("RAI_HIP_NO_MFMA_STREAM") != nullptr;
-  if (a.M <= 64 && !no_skinny && !no_stream) {
+  if (a.M <= 64 && !no_skinny && !no_stream && (!a.f32_out || a.Wfrag)) {
     int splits = 1;
     if (a.M <= 16 && mfma_stream_fits<1, 8>(a, &splits)) return launch_mfma_stream<1, 8>(st, a, splits);
     if (a.M > 16 && a.M <= 32 && mfma_stream_fits<2, 8>(a, &splits)) return launch_mfma_stream<2, 8>(st, a, splits);

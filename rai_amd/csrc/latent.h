@@ -122,7 +122,7 @@ struct MoeSlotsArgs {
   void *eact;
   int waves_e, rows_per_wave;   // filled in by the launcher
 };
-bool moe_slots_serves(int64_t slots, int Hp, int top, int EFp);
+bool moe_slots_serves(int64_t slots, int experts, int Hp, int top, int EFp);
 int launch_moe_slots(hipStream_t st, MoeSlotsArgs a);
 // For each of `rows` rows (x0, x1, choice, res and out dense, row by row):
 // out[n] = res[n] + mult * (W0[n] . x0 + sum_j W1[choice[j]][n] . x1[j]); rows of W0 (W1) are K0 (K1) long

@@ -387,10 +387,11 @@ int launch_latent_mid(hipStream_t st, LatentMidArgs a) {
   return launch_check("latent_mid");
 }
 
-bool moe_slots_serves(int64_t slots, int Hp, int top, int EFp) {
+bool moe_slots_serves(int64_t slots, int experts, int Hp, int top, int EFp) {
   const char *off = getenv("RAI_HIP_NO_LATENT_FUSED");   // read per call: the tests compare both forms in one process
   if (off && *off && *off != '0') return false;
-  return slots <= 64 && Hp <= 4096 && (int64_t)top * EFp * 2 + 16 * 1024 <= 150 * 1024;
+  // more slots than experts: several tokens share an expert, whose weights the grouped tiles read once
+  return slots <= 64 && slots <= experts && Hp <= 4096 && (int64_t)top * EFp * 2 + 16 * 1024 <= 150 * 1024;
 }
 int launch_moe_slots(hipStream_t st, MoeSlotsArgs a) {
   int rpw = (a.slots * 2 * a.EFp + kNumCU * 16 - 1) / (kNumCU * 16);
