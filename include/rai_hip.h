@@ -419,7 +419,8 @@ typedef struct rai_hip_latent_config {
 } rai_hip_latent_config;
 /* Parameters are named "embed", "l<i>.norm1", "l<i>.mix.<dq|uq|dkv|uk|uv|g|o>", "l<i>.mix.<dq|dkv>.norm", "l<i>.norm2",
  * "l<i>.mlp.<gate|up|down>" or "l<i>.mlp.e<k>.<gate|up|down>" and "l<i>.mlp.router", "final.norm", "head".  Sizes may be
- * any positive numbers (weights are padded internally).  Every rai_hip_decoder_* call works on the result. */
+ * any positive numbers (weights are padded internally).  Every rai_hip_decoder_* call works on the result,
+ * except the two rai_hip_decoder_time_* measurements. */
 int rai_hip_decoder_create_latent(int dev, const rai_hip_latent_config *cfg, const rai_hip_latent_layer *layers,
                                   rai_hip_decoder **out);
 /* Module::update_by_safetensors naming (rai-core/src/nn.rs:183-205, renames

@@ -73,7 +73,6 @@ struct LatentModel {
   MoePlan plan;
   float *ws;                   // partial results of the absorbed attention's context splits
   bool derived_ready;          // WukT matches the loaded parameters
-  int max_top;
 };
 
 }  // namespace rai

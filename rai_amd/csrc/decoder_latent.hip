@@ -176,7 +176,6 @@ static int create_latent(rai_hip_decoder *d, const rai_hip_latent_config &cfg, c
     lm.plan.n_tiles = (int *)tmp;
     lm.plan.cap_tiles = (int)tiles;
   }
-  lm.max_top = (int)top;
   return RAI_OK;
 }
 
