@@ -344,7 +344,8 @@ typedef enum rai_hip_arch {
   RAI_ARCH_QWEN2 = 1, /* rai-models/src/llm/qwen2.rs */
   RAI_ARCH_GEMMA = 2, /* rai-models/src/llm/gemma.rs */
   RAI_ARCH_PHI3 = 3,  /* rai-models/src/llm/phi3.rs: the Qwen2 block with fused qkv_proj / gate_up_proj, no biases */
-  RAI_ARCH_LELITAR = 4 /* latent attention and a mixture of experts in a parallel block (rai_hip_decoder_create_latent) */
+  RAI_ARCH_LELITAR = 4, /* latent attention and a mixture of experts in a parallel block (rai_hip_decoder_create_latent) */
+  RAI_ARCH_BEZADRA = 5 /* attention and gated delta rule layers in a parallel block, some of them looped (rai_hip_decoder_create_hybrid) */
 } rai_hip_arch;
 
 /* Union of the serde Config structs phi2.rs:9-24, qwen2.rs:8-24, gemma.rs:12-27. */
@@ -422,6 +423,61 @@ typedef struct rai_hip_latent_config {
  * any positive numbers (weights are padded internally).  Every rai_hip_decoder_* call works on the result,
  * except the two rai_hip_decoder_time_* measurements. */
 int rai_hip_decoder_create_latent(int dev, const rai_hip_latent_config *cfg, const rai_hip_latent_layer *layers,
+                                  rai_hip_decoder **out);
+
+/* A decoder whose layers are attention or a recurrence, described one by one (RAI_ARCH_BEZADRA; no counterpart in the
+ * reference):
+ *   x <- x + (mixer(norm(x)) + mlp(norm(x))),   one layer norm for both; residual stream in f32.
+ * Layers loop_start .. loop_stop - 1 run loop_times times with the same weights, each pass with a cache or state of its
+ * own; ahead of pass t, x <- W_in [x; embedding output] + step[t]. */
+typedef enum rai_hip_mixer_kind { RAI_MIXER_ATTENTION = 0, RAI_MIXER_CHANNEL_DELTA = 1 } rai_hip_mixer_kind;
+typedef struct rai_hip_hybrid_layer {
+  int32_t mixer; /* rai_hip_mixer_kind */
+  int32_t heads;
+  int32_t kv_heads; /* attention: key/value heads; delta rule: query/key heads */
+  int32_t qk_dim;
+  int32_t v_dim;
+  /* attention: rotary positions on the first rot_dims features of q and k (rot_factor > 0: waves longer than
+   * rot_original / rot_low positions stretched by it, those shorter than rot_original / rot_high kept, blended between),
+   * scores cap * tanh(scale q.k / cap) (softcap 0: not capped), a learned sink per head in the softmax, an output gate */
+  int32_t rot_dims;
+  /* delta rule: taps of the convolutions on q, k and v, ranks of the decay's and the output gate's factors */
+  int32_t conv_taps;
+  int32_t decay_rank;
+  int32_t gate_rank;
+  /* down(a sigmoid(mlp_alpha a) (b + 1)), a = gate h cut off above mlp_limit, b = up h cut off at +-mlp_limit */
+  int32_t mlp_kind; /* RAI_MLP_NONE or RAI_MLP_DENSE */
+  int32_t intermediate;
+  double attn_scale;
+  double softcap;
+  double rot_base;
+  double rot_factor;
+  double rot_low;
+  double rot_high;
+  double rot_original;
+  double mlp_limit;
+  double mlp_alpha;
+} rai_hip_hybrid_layer;
+typedef struct rai_hip_hybrid_config {
+  int32_t dtype; /* RAI_BF16 or RAI_F32 */
+  int32_t vocab_size;
+  int32_t width;
+  int32_t num_layers;
+  int32_t loop_start; /* loop_times == 0: no loop */
+  int32_t loop_stop;
+  int32_t loop_times;
+  int32_t max_batch;
+  int32_t max_context;
+  double norm_eps;
+  double embed_scale; /* the embedding output is embed[token] * embed_scale */
+  double logit_scale; /* logits = embed . norm(x) * logit_scale */
+} rai_hip_hybrid_config;
+/* Parameters are named "embed", "loop.in", "loop.step", "l<i>.norm1", "l<i>.mix.<q|k|v|sink|g|o>" (attention) or
+ * "l<i>.mix.<q|k|v|b|A_log|norm|a1|a2|dt_bias|g1|g2|o>" and "l<i>.mix.<q|k|v>.conv" (delta rule),
+ * "l<i>.mlp.<gate|up|down>", "final.norm".  Sizes may be any positive numbers (weights are padded internally), the delta
+ * rule's head sizes up to 512.  Every rai_hip_decoder_* call works on the result, except the two rai_hip_decoder_time_*
+ * measurements; rows given to rai_hip_decoder_forward_hidden stand for embedding rows, ahead of embed_scale. */
+int rai_hip_decoder_create_hybrid(int dev, const rai_hip_hybrid_config *cfg, const rai_hip_hybrid_layer *layers,
                                   rai_hip_decoder **out);
 /* Module::update_by_safetensors naming (rai-core/src/nn.rs:183-205, renames
  * phi2.rs:307-313): copy one named parameter from host memory, e.g.

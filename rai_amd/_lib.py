@@ -22,8 +22,9 @@ UNARY = {n: i for i, n in enumerate(
 BINARY = {n: i for i, n in enumerate(
     ["add", "sub", "mul", "div", "maximum", "minimum", "eq", "ne", "gt", "ge", "lt", "le"])}
 REDUCE = {"sum": 0, "max": 1, "min": 2}
-ARCH = {"phi2": 0, "qwen2": 1, "gemma": 2, "phi3": 3, "lelitar": 4}
+ARCH = {"phi2": 0, "qwen2": 1, "gemma": 2, "phi3": 3, "lelitar": 4, "bezadra": 5}
 MLP_KIND = {"none": 0, "dense": 1, "moe": 2}
+MIXER = {"attention": 0, "channel_delta": 1}
 
 
 class RaiHipError(RuntimeError):
@@ -75,6 +76,19 @@ class LatentLayer(C.Structure):
 class LatentConfig(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("dtype", "vocab_size", "width", "num_layers", "norm_groups", "max_batch",
                                          "max_context")] + [("norm_eps", C.c_double), ("residual_mult", C.c_double)]
+
+
+class HybridLayer(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "qk_dim", "v_dim", "rot_dims", "conv_taps", "decay_rank",
+                                         "gate_rank", "mlp_kind", "intermediate")] + \
+               [(n, C.c_double) for n in ("attn_scale", "softcap", "rot_base", "rot_factor", "rot_low", "rot_high", "rot_original",
+                                          "mlp_limit", "mlp_alpha")]
+
+
+class HybridConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("dtype", "vocab_size", "width", "num_layers", "loop_start", "loop_stop", "loop_times",
+                                         "max_batch", "max_context")] + \
+               [(n, C.c_double) for n in ("norm_eps", "embed_scale", "logit_scale")]
 
 
 _TP = C.POINTER(TensorDesc)
@@ -130,6 +144,7 @@ PROTOTYPES = {
     "rai_hip_attention": [C.c_int, _TP, _TP, _TP, _dbl, _i32, _i32, _TP],
     "rai_hip_decoder_create": [C.c_int, C.POINTER(DecoderConfig), C.POINTER(_vp)],
     "rai_hip_decoder_create_latent": [C.c_int, C.POINTER(LatentConfig), C.POINTER(LatentLayer), C.POINTER(_vp)],
+    "rai_hip_decoder_create_hybrid": [C.c_int, C.POINTER(HybridConfig), C.POINTER(HybridLayer), C.POINTER(_vp)],
     "rai_hip_decoder_destroy": [_vp],
     "rai_hip_decoder_load_param": [_vp, C.c_char_p, _vp, C.c_size_t],
     "rai_hip_decoder_load_safetensors": [_vp, C.POINTER(C.c_char_p), _i32],

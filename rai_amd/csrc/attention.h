@@ -29,6 +29,10 @@ struct AttnArgs {
   // sigmoid(gate[(b*S + s)*gate_row_stride + h*D + d]).
   const void *gate;
   int64_t gate_row_stride;
+  // f32_scores form only.  softcap > 0: a score s becomes softcap * tanh(s / softcap).  sink: one value per query head
+  // (model dtype) whose exponential joins the softmax's denominator, without a key or a value.
+  float softcap;
+  const void *sink;
 };
 
 int launch_attention(hipStream_t st, const AttnArgs &a);
@@ -41,7 +45,12 @@ struct AttnDecodeArgs {
   void *kcache, *vcache;  // this layer's [B][Hkv][Tmax][D]
   void *out;
   int64_t out_row_stride;
-  const void *cos_t, *sin_t;  // [max_pos, rot] in the model dtype
+  const void *cos_t, *sin_t;  // [max_pos, rot] in the model dtype, or f32 (tab_f32: rotated in f32, rounded once)
+  int tab_f32;
+  float softcap;              // as in AttnArgs, f32_scores form only
+  const void *sink;
+  const void *gate;           // output gate of sequence b: gate + b * gate_row_stride, features as in AttnArgs
+  int64_t gate_row_stride;
   const int *pos_dev;         // tokens already in the cache (device memory); null: pos_host
   int pos_host;
   // The new token's key and value rows as tensors of their own ([B][Hkv*D], element strides between sequences

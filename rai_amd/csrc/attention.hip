@@ -28,6 +28,10 @@ template <typename T> __device__ __forceinline__ float round_to(float x) {
 template <> __device__ __forceinline__ float round_to<float>(float x) { return x; }
 
 __device__ __forceinline__ float gate_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float cap_score(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
+template <typename T> __device__ __forceinline__ float sink_of(const void *sink, int h) {
+  return sink ? (float)Scalar<T>::load((const T *)sink + h) : -INFINITY;
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
@@ -77,7 +81,7 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
       acc += __shfl_xor(acc, 1, 64);
       if (gl == 0) {
         float sc;
-        if (a.f32_scores) sc = acc * a.scale;
+        if (a.f32_scores) sc = cap_score(acc * a.scale, a.softcap);
         else sc = round_to<T>(round_to<T>(acc) * round_to<T>(a.scale));
         scores[t - t_begin] = sc;
       }
@@ -87,12 +91,13 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
 
   // ---- softmax over the scores of keys [t_begin, t_end)
   const int n_seen = t_end - t_begin;
+  const float sink = sink_of<T>(a.sink, h);
   float m = -INFINITY;
   for (int t = tid; t < n_seen; t += 256) m = fmaxf(m, scores[t]);
   m = wave_max(m);
   if (lane == 0) sh[wave] = m;
   __syncthreads();
-  m = fmaxf(fmaxf(sh[0], sh[1]), fmaxf(sh[2], sh[3]));
+  m = fmaxf(fmaxf(fmaxf(sh[0], sh[1]), fmaxf(sh[2], sh[3])), sink);
   float sum = 0.f;
   for (int t = tid; t < n_seen; t += 256) {
     float e = expf(scores[t] - m);
@@ -104,6 +109,7 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
   if (lane == 0) sh[4 + wave] = sum;
   __syncthreads();
   sum = sh[4] + sh[5] + sh[6] + sh[7];
+  if (a.sink) sum += expf(sink - m);
   if (!a.f32_scores) sum = round_to<T>(sum);
   const float inv = 1.0f / sum;
 
@@ -141,11 +147,15 @@ __global__ void __launch_bounds__(256) k_attn_row(AttnArgs a) {
 // reference's three roundings (x*cos, rotate_half(x)*sin, their sum:
 // rai-models/src/llm/phi2.rs:75).
 template <typename T>
-__device__ __forceinline__ float rope_feature(const T *head, int d, int rot, const T *cos_t, const T *sin_t, int pos) {
+__device__ __forceinline__ float rope_feature(const T *head, int d, int rot, const T *cos_t, const T *sin_t, int pos, int tab_f32) {
   float v = (float)Scalar<T>::load(head + d);
   if (d >= rot) return v;
   const int half = rot >> 1;
   float other = d < half ? -(float)Scalar<T>::load(head + d + half) : (float)Scalar<T>::load(head + d - half);
+  if (tab_f32) {   // f32 tables: products and sum in f32, one rounding
+    const int64_t e = (int64_t)pos * rot + d;
+    return round_to<T>(fmaf(v, ((const float *)cos_t)[e], other * ((const float *)sin_t)[e]));
+  }
   float c = (float)Scalar<T>::load(cos_t + (int64_t)pos * rot + d);
   float s = (float)Scalar<T>::load(sin_t + (int64_t)pos * rot + d);
   return round_to<T>(round_to<T>(v * c) + round_to<T>(other * s));
@@ -207,9 +217,10 @@ __device__ __forceinline__ void decode_merge_last(const AttnDecodeArgs &a, int b
   __syncthreads();
   for (int r = wave; r < R; r += NT / 64) {      // NS <= 64: one split per lane
     const float m = lane < NS ? wm[r * NS + lane] : -INFINITY;
-    const float M = wave_max(m);                 // split 0 always holds a key, so M is finite
+    const float sink = sink_of<T>(a.sink, hq0 + r);
+    const float M = fmaxf(wave_max(m), sink);    // split 0 always holds a key, so M is finite
     const float e = lane < NS ? expf(m - M) : 0.f;  // an empty split has m = -inf: weight 0
-    const float L = wave_sum(lane < NS ? e * wl[r * NS + lane] : 0.f);
+    const float L = wave_sum(lane < NS ? e * wl[r * NS + lane] : 0.f) + (a.sink ? expf(sink - M) : 0.f);
     if (lane < NS) wm[r * NS + lane] = e / L;
   }
   __syncthreads();
@@ -240,9 +251,12 @@ __device__ __forceinline__ void decode_merge_last(const AttnDecodeArgs &a, int b
     }
 #pragma unroll
     for (int i = 0; i < EU; ++i)
-      if (e0 + i * NT < R * D)
+      if (e0 + i * NT < R * D) {
+        if (a.gate)
+          O[i] *= gate_sigmoid((float)Scalar<T>::load((const T *)a.gate + (int64_t)b * a.gate_row_stride + (int64_t)(hq0 + hr[i]) * D + hd[i]));
         Scalar<T>::store((T *)a.out + (int64_t)b * a.out_row_stride + (int64_t)(hq0 + hr[i]) * D + hd[i],
                          (typename Scalar<T>::compute)O[i]);
+      }
   }
   if (tid == 0) *counter = 0;  // ready for the next launch (stream order)
 }
@@ -309,11 +323,11 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_split(AttnDecode
   // ---- rotary embedding of the R query rows (and of the new key where it is needed)
   for (int e = tid; e < R * D; e += NT) {
     const int r = e / D, d = e - r * D;
-    qf[e] = rope_feature<T>(qrow + (hq0 + r) * D, d, a.rot, cos_t, sin_t, pos);
+    qf[e] = rope_feature<T>(qrow + (hq0 + r) * D, d, a.rot, cos_t, sin_t, pos, a.tab_f32);
   }
   if (has_new) {
     for (int d = tid; d < D; d += NT) {
-      const float kr = rope_feature<T>(krow + hk * D, d, a.rot, cos_t, sin_t, pos);
+      const float kr = rope_feature<T>(krow + hk * D, d, a.rot, cos_t, sin_t, pos, a.tab_f32);
       const float vr = (float)Scalar<T>::load(vrow + hk * D + d);
       knew[d] = kr;
       vnew[d] = vr;
@@ -326,7 +340,7 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_split(AttnDecode
   __syncthreads();
 
   auto finish_score = [&](float acc) -> float {
-    if (a.f32_scores) return acc * a.scale;
+    if (a.f32_scores) return cap_score(acc * a.scale, a.softcap);
     return round_to<T>(round_to<T>(acc) * round_to<T>(a.scale));
   };
   // ---- scores against the cached keys: 16 lanes per key row, round 0 from the prefetched registers
@@ -567,8 +581,8 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_mfma(AttnDecodeA
       if (item < 16 * CPR && r < R) {
         const T *head = qrow + (hq0 + r) * D;
         qx[i] = *reinterpret_cast<const ad_u32x4 *>(head + d);
-        if (d < a.rot) {
-          qo[i] = *reinterpret_cast<const ad_u32x4 *>(head + (d < half ? d + half : d - half));
+        if (d < a.rot) qo[i] = *reinterpret_cast<const ad_u32x4 *>(head + (d < half ? d + half : d - half));
+        if (d < a.rot && !a.tab_f32) {
           qc[i] = *reinterpret_cast<const ad_u32x4 *>(cos_t + (int64_t)pos * a.rot + d);
           qn[i] = *reinterpret_cast<const ad_u32x4 *>(sin_t + (int64_t)pos * a.rot + d);
         }
@@ -579,7 +593,21 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_mfma(AttnDecodeA
       const int item = tid + i * kDecodeThreads, r = item / CPR, d = (item - r * CPR) * 8;
       if (item >= 16 * CPR) continue;
       ad_u32x4 out = qx[i];
-      if (r < R && d < a.rot) {
+      if (r < R && d < a.rot && a.tab_f32) {   // f32 tables: products and sum in f32, one rounding
+        const float sign = d < half ? -1.f : 1.f;
+        const float *cp = (const float *)cos_t + (int64_t)pos * a.rot + d, *sp = (const float *)sin_t + (int64_t)pos * a.rot + d;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+          float res[2];
+#pragma unroll
+          for (int hbit = 0; hbit < 2; ++hbit) {
+            const int sh = 16 * hbit;
+            const float x = bf16_bits_to_f32((uint16_t)(qx[i][w] >> sh)), o = sign * bf16_bits_to_f32((uint16_t)(qo[i][w] >> sh));
+            res[hbit] = fmaf(x, cp[2 * w + hbit], o * sp[2 * w + hbit]);
+          }
+          out[w] = pack_bf16x2(res[0], res[1]);
+        }
+      } else if (r < R && d < a.rot) {
         const float sign = d < half ? -1.f : 1.f;
 #pragma unroll
         for (int w = 0; w < 4; ++w) {
@@ -601,14 +629,14 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_mfma(AttnDecodeA
   } else {
     for (int e = tid; e < 16 * D; e += kDecodeThreads) {
       const int r = e / D, d = e - r * D;
-      const float q = r < R ? rope_feature<T>(qrow + (hq0 + r) * D, d, a.rot, cos_t, sin_t, pos) : 0.f;
+      const float q = r < R ? rope_feature<T>(qrow + (hq0 + r) * D, d, a.rot, cos_t, sin_t, pos, a.tab_f32) : 0.f;
       Vs[r * VP + d] = f32_to_bf16_bits(q);
     }
   }
   for (int e = tid; e < 16 * PP; e += kDecodeThreads) ps[e] = 0;
   if (has_new) {
     for (int d = tid; d < D; d += kDecodeThreads) {
-      const uint16_t kr = f32_to_bf16_bits(rope_feature<T>(krow + hk * D, d, a.rot, cos_t, sin_t, pos));
+      const uint16_t kr = f32_to_bf16_bits(rope_feature<T>(krow + hk * D, d, a.rot, cos_t, sin_t, pos, a.tab_f32));
       const uint16_t vr = (vrow + hk * D + d)->bits;
       knew[d] = kr;
       vnew[d] = vr;
@@ -637,7 +665,7 @@ __global__ void __launch_bounds__(kDecodeThreads) k_attn_decode_mfma(AttnDecodeA
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int tl = tile * 16 + 4 * lq + r;
-        float sc = a.f32_scores ? acc[r] * a.scale : round_to<T>(round_to<T>(acc[r]) * round_to<T>(a.scale));
+        float sc = a.f32_scores ? cap_score(acc[r] * a.scale, a.softcap) : round_to<T>(round_to<T>(acc[r]) * round_to<T>(a.scale));
         if (lrow < R) scores[lrow * CH + tl] = tl < n ? sc : -INFINITY;
       }
     }
@@ -711,9 +739,12 @@ __global__ void __launch_bounds__(256) k_attn_decode_merge_bf16(AttnDecodeArgs a
   const float *pr = a.ws + ((int64_t)b * a.Hq + h) * NS * PW;
   const float m = lane < NS ? pr[lane * PW] : -INFINITY;
   const float l = lane < NS ? pr[lane * PW + 1] : 0.f;
-  const float M = wave_max(m);                    // split 0 always holds a key, so M is finite
+  const float sink = sink_of<bf16_raw>(a.sink, h);
+  float gate = 1.f;
+  if (a.gate) gate = gate_sigmoid((float)Scalar<bf16_raw>::load((const bf16_raw *)a.gate + (int64_t)b * a.gate_row_stride + (int64_t)h * D + d));
+  const float M = fmaxf(wave_max(m), sink);       // split 0 always holds a key, so M is finite
   const float e = lane < NS ? expf(m - M) : 0.f;  // an empty split has m = -inf: weight 0
-  const float L = wave_sum(e * l);
+  const float L = wave_sum(e * l) + (a.sink ? expf(sink - M) : 0.f);
   const float w = e / L;
   float O = 0.f;
   constexpr int SB = 16;
@@ -725,7 +756,7 @@ __global__ void __launch_bounds__(256) k_attn_decode_merge_bf16(AttnDecodeArgs a
     for (int j = 0; j < SB; ++j)
       if (s0 + j < NS) O = fmaf(__shfl(w, s0 + j, 64), ov[j], O);
   }
-  ((bf16_raw *)a.out + (int64_t)b * a.out_row_stride + (int64_t)h * D + d)->bits = f32_to_bf16_bits(O);
+  ((bf16_raw *)a.out + (int64_t)b * a.out_row_stride + (int64_t)h * D + d)->bits = f32_to_bf16_bits(O * gate);
 }
 
 template <int D, int CH> static int launch_decode_mfma_cfg(hipStream_t st, AttnDecodeArgs a) {
@@ -830,7 +861,8 @@ template <typename T> static int launch_decode(hipStream_t st, const AttnDecodeA
 int launch_attention_decode(hipStream_t st, const AttnDecodeArgs &a) {
   RAI_REQUIRE(a.B > 0 && a.Hq > 0 && a.Hkv > 0 && a.D > 0 && a.Tmax > 0 && a.Hq % a.Hkv == 0, RAI_ERR_BAD_SHAPE,
               "attention decode: bad problem");
-  RAI_REQUIRE(a.rot > 0 && a.rot % 2 == 0 && a.rot <= a.D, RAI_ERR_BAD_ARG, "attention decode: rot %d", a.rot);
+  RAI_REQUIRE(a.rot >= (a.tab_f32 ? 0 : 2) && a.rot % 2 == 0 && a.rot <= a.D, RAI_ERR_BAD_ARG, "attention decode: rot %d", a.rot);
+  RAI_REQUIRE(a.f32_scores || (!a.sink && a.softcap <= 0.f), RAI_ERR_BAD_ARG, "attention decode: a cap or a sink needs the f32-score form");
   RAI_REQUIRE(a.ws && a.counters, RAI_ERR_BAD_ARG, "attention decode: partial-result workspace missing");
   if (decode_mfma_eligible(a)) {
     if (a.D == 64) return launch_decode_mfma<64>(st, a);
@@ -881,7 +913,8 @@ typedef __attribute__((ext_vector_type(2))) uint32_t fa_u32x2;
 // its own running maximum, sum and output; the two are merged through LDS at the end.  For short sequences and few
 // heads, where the grid has about one block per CU and a wave's chain of key tiles is what the launch takes.
 // (Four waves per group, KSP = 4, gained another half per cent on the Phi-2 prefill: not instantiated.)
-template <int NW, int D, bool F32S, int KSP = 1>
+// MODE: 0 scores rounded to bf16, 1 scores in f32, 2 scores in f32 with the cap and the sink of AttnArgs.
+template <int NW, int D, int MODE, int KSP = 1>
 __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a) {
   constexpr int KS = D / 16;            // K steps of the score product
   constexpr int DT = (D + 31) / 32;     // 32-row tiles of O^T
@@ -1041,11 +1074,19 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
     // needs no masking
     const bool masked = k0 + 63 >= a.T || (a.causal && k0 + 63 > off + q0 + wave * 32) ||
                         (a.window > 0 && k0 <= off + q0 + wave * 32 + 31 - a.window);
-    if constexpr (F32S) {
+    if constexpr (MODE >= 1) {
 #pragma unroll
       for (int u = 0; u < 2; ++u)
 #pragma unroll
         for (int r = 0; r < 16; ++r) sc[u][r] *= a.scale;
+      if (MODE == 2 && a.softcap > 0.f) {   // cap * tanh(s / cap) = cap - 2 cap / (exp(2 s / cap) + 1)
+        const float to_exp = 2.0f * 1.4426950408889634f / a.softcap;
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int r = 0; r < 16; ++r)
+            sc[u][r] = fmaf(-2.0f * a.softcap, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sc[u][r] * to_exp)), a.softcap);
+      }
     } else {   // the product and its scaling are each rounded to bf16, two scores per conversion
 #pragma unroll
       for (int u = 0; u < 2; ++u)
@@ -1168,7 +1209,18 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
         for (int r = 0; r < 16; ++r) o[dt][r] += mb[j * MS + 2 + dt * 16 + r] * wj;
     }
   }
-  const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
+  float l_tot = l_run + __shfl_xor(l_run, 32, 64);
+  if constexpr (MODE == 2) {
+    if (a.sink) {   // relative to the running exponent, moved up to the sink's where that is larger by much
+      const float sink = sink_of<bf16_raw>(a.sink, h), m = fmaxf(m_run, sink);
+      const float w = expf(m_run - m);
+      l_tot = l_tot * w + expf(sink - m);
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[dt][r] *= w;
+    }
+  }
   if (qrow < a.S) {
     const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
     uint16_t *op = (uint16_t *)a.out + ((int64_t)b * a.S + qrow) * a.out_row_stride + (int64_t)h * D;
@@ -1196,26 +1248,27 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
   }
 }
 
-template <int D> static int launch_flash(hipStream_t st, const AttnArgs &a) {
+template <int D, int MODE> static int launch_flash_mode(hipStream_t st, const AttnArgs &a) {
   const int tiles4 = (a.S + 127) / 128;
   if ((int64_t)tiles4 * a.Hq * a.B >= kNumCU) {
-    if (a.f32_scores) hipLaunchKernelGGL((k_flash_prefill_bf16<4, D, true>), dim3(tiles4, a.Hq, a.B), dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((k_flash_prefill_bf16<4, D, false>), dim3(tiles4, a.Hq, a.B), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((k_flash_prefill_bf16<4, D, MODE>), dim3(tiles4, a.Hq, a.B), dim3(256), 0, st, a);
   } else {
     const dim3 grid((a.S + 63) / 64, a.Hq, a.B);
     // about one block per CU or fewer, several key tiles per block: two waves per query group, each half of the keys
     const char *no_split = getenv("RAI_HIP_FLASH_NO_KEY_SPLIT");   // read per call: tests compare both forms
     if constexpr (D <= 80) {
       if ((int64_t)grid.x * grid.y * grid.z < 2 * kNumCU && a.T > 128 && !(no_split && *no_split && *no_split != '0')) {
-        if (a.f32_scores) hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, true, 2>), grid, dim3(256), 0, st, a);
-        else hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, false, 2>), grid, dim3(256), 0, st, a);
+        hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, MODE, 2>), grid, dim3(256), 0, st, a);
         return launch_check("flash_prefill");
       }
     }
-    if (a.f32_scores) hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, true>), grid, dim3(128), 0, st, a);
-    else hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, false>), grid, dim3(128), 0, st, a);
+    hipLaunchKernelGGL((k_flash_prefill_bf16<2, D, MODE>), grid, dim3(128), 0, st, a);
   }
   return launch_check("flash_prefill");
+}
+template <int D> static int launch_flash(hipStream_t st, const AttnArgs &a) {
+  if (!a.f32_scores) return launch_flash_mode<D, 0>(st, a);
+  return a.softcap > 0.f || a.sink ? launch_flash_mode<D, 2>(st, a) : launch_flash_mode<D, 1>(st, a);
 }
 
 static bool flash_eligible(const AttnArgs &a) {
@@ -1234,8 +1287,8 @@ int launch_attention(hipStream_t st, const AttnArgs &a) {
               "attention: empty problem");
   RAI_REQUIRE(a.Hq % a.Hkv == 0, RAI_ERR_BAD_SHAPE, "attention: %d query heads not divisible by %d kv heads", a.Hq,
               a.Hkv);
-  RAI_REQUIRE(a.window >= 0 && (!a.window || a.causal) && (!a.gate || a.f32_scores), RAI_ERR_BAD_ARG,
-              "attention: a window needs the causal form, an output gate the f32-score form");
+  RAI_REQUIRE(a.window >= 0 && (!a.window || a.causal) && (a.f32_scores || (!a.gate && !a.sink && a.softcap <= 0.f)), RAI_ERR_BAD_ARG,
+              "attention: a window needs the causal form, an output gate, a cap or a sink the f32-score form");
   if (flash_eligible(a)) {
     switch (a.D) {
       case 32: return launch_flash<32>(st, a);

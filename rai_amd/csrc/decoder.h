@@ -1,5 +1,6 @@
 // The decoder object behind rai_hip_decoder_*, shared by the drivers of the model families (decoder.hip: Phi-2 and the
-// sequential Qwen2 / Gemma / Phi-3 block; decoder_latent.hip: latent attention with a parallel MLP or mixture).
+// sequential Qwen2 / Gemma / Phi-3 block; decoder_latent.hip: latent attention with a parallel MLP or mixture;
+// decoder_hybrid.hip: attention and gated delta rule layers, some of them looped).
 #pragma once
 #include <map>
 #include <string>
@@ -8,8 +9,10 @@
 #include "attention.h"
 #include "decode_chain.h"
 #include "decode_mega.h"
+#include "delta.h"
 #include "gemm.h"
 #include "latent.h"
+#include "rotary.h"
 
 namespace rai {
 
@@ -75,6 +78,48 @@ struct LatentModel {
   bool derived_ready;          // WukT matches the loaded parameters
 };
 
+// One layer of a hybrid model, padded with zero weights like a latent layer.
+struct HybridLayer {
+  rai_hip_hybrid_layer c;      // the configuration's sizes
+  int Dp, Fp;                  // attention: head width of q, k, v and gate; MLP
+  int ldn;                     // columns of the input projection's output
+  int QD;                      // columns of the mixer's output: heads * Dp, or heads * Vp
+  int a_rank, g_rank;          // padded ranks
+  DeltaShape delta;
+  char *n1_w;
+  char *Wd;                    // [ldn, Hp]  attention: q | k | v | g;  delta rule: q | k | v | b | a1 | g1
+  char *Wgu;                   // [2 Fp, Hp] gate / up rows interleaved
+  char *Wb;                    // [Hp, QD + Fp]: o | down as one contraction
+  char *sink;                  // [heads]
+  char *conv, *A_log, *dt_bias, *norm_w, *a2, *g2;   // [channels, taps], [heads], [heads Dk], [Vp], [heads Dk, a_rank], [heads Vp, g_rank]
+  const float *cos_t, *sin_t;  // [max_context, rot_dims]
+  char *Wd_f, *Wgu_f, *Wb_f, *a2_f, *g2_f;   // in MFMA-fragment order for 9 .. 64 rows (built on first use)
+};
+// One layer run: a looped layer has one per pass, with what that pass carries from step to step.
+struct HybridRun {
+  int layer, pass;             // pass >= 0: the first layer of pass `pass`
+  char *kcache, *vcache;       // attention: [max_batch][kv_heads][max_context][Dp]
+  char *ring;                  // delta rule: the convolutions' last inputs and the state
+  float *carried;
+};
+struct HybridModel {
+  rai_hip_hybrid_config c;
+  int Hp;
+  std::vector<HybridLayer> layers;
+  std::vector<HybridRun> runs;
+  std::vector<std::pair<RotaryParams, std::pair<const float *, const float *>>> tables;
+  char *Wx, *W0, *step;        // loop.in's two halves [Hp, Hp] and [times, Hp]
+  char *Wx_f, *W0_f;
+  float *xs, *xs2, *x0w;       // [max_rows, Hp]: residual stream (two, swapped by the single-row step's loop entry), W0 x0
+  float *stream;               // the one the last forward finished in
+  char *h1, *dn, *cat;
+  float *decay, *q, *k, *v, *beta, *o;
+  char *gate;
+  char *attn_ws;
+  int *attn_counters;
+  bool derived_ready;          // a padded copy of the embedding table serves as the head
+};
+
 }  // namespace rai
 
 using namespace rai;
@@ -131,6 +176,7 @@ struct rai_hip_decoder {
   float graph_penalty;
   int graph_last_n;
   LatentModel *latent;        // the latent-attention family's part; null for the others
+  HybridModel *hybrid;        // the hybrid family's part; null for the others
 };
 
 
@@ -152,5 +198,16 @@ int forward_latent(rai_hip_decoder *d, int B, int S, bool advance_step, bool fro
 // Logits (model dtype, [n, vocab]) of n rows of the residual stream the last forward left; rows_dev: row indices.
 int latent_head_rows(rai_hip_decoder *d, hipStream_t st, const int *rows_dev, int n, char *logits);
 int latent_hidden_to_host(rai_hip_decoder *d, int64_t rows, float *out);
+
+// decoder_hybrid.hip: the same for the hybrid family
+int forward_hybrid(rai_hip_decoder *d, int B, int S, bool advance_step, bool from_tokens);
+int hybrid_head_rows(rai_hip_decoder *d, hipStream_t st, const int *rows_dev, int n, char *logits);
+int hybrid_hidden_to_host(rai_hip_decoder *d, int64_t rows, float *out);
+// device memory that starts as zeros, and a parameter whose rows (columns) come in padded groups (decoder_latent.hip)
+int zalloc(rai_hip_decoder *d, size_t bytes, char **out);
+void add_grouped_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch, int64_t row_group,
+                      int64_t row_stride, int64_t col_group, int64_t col_stride);
+inline int pad64(int n) { return (n + 63) / 64 * 64; }
+inline int pad_head(int n) { return n <= 32 ? 32 : n <= 64 ? 64 : n <= 128 ? 128 : n <= 192 ? 192 : n <= 256 ? 256 : pad64(n); }
 
 }  // namespace rai

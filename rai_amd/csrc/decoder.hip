@@ -1150,6 +1150,7 @@ static int forward_seq(rai_hip_decoder *d, int B, int S, bool advance_step, bool
 
 static int forward_any(rai_hip_decoder *d, int B, int S, bool advance_step, bool from_tokens = false) {
   if (d->latent) return forward_latent(d, B, S, advance_step, from_tokens);
+  if (d->hybrid) return forward_hybrid(d, B, S, advance_step, from_tokens);
   return d->cfg.arch == RAI_ARCH_PHI2 ? forward_phi2(d, B, S, advance_step, from_tokens)
                                        : forward_seq(d, B, S, advance_step, from_tokens);
 }
@@ -1264,6 +1265,7 @@ void decoder_init_fields(rai_hip_decoder *d, int dev, const rai_hip_decoder_conf
   d->mega_prof = nullptr;
   d->mega_xchg = nullptr;
   d->latent = nullptr;
+  d->hybrid = nullptr;
   d->max_rows = (int64_t)cfg->max_batch * cfg->max_context;
   d->history_cap = cfg->max_context;
   hipDeviceProp_t prop;
@@ -1308,6 +1310,7 @@ extern "C" {
 int rai_hip_decoder_create(int dev, const rai_hip_decoder_config *cfg, rai_hip_decoder **out) {
   RAI_REQUIRE(cfg && out, RAI_ERR_BAD_ARG, "decoder_create: null argument");
   RAI_REQUIRE(cfg->arch != RAI_ARCH_LELITAR, RAI_ERR_UNSUPPORTED, "decoder_create: this architecture is built by decoder_create_latent");
+  RAI_REQUIRE(cfg->arch != RAI_ARCH_BEZADRA, RAI_ERR_UNSUPPORTED, "decoder_create: this architecture is built by decoder_create_hybrid");
   RAI_REQUIRE(cfg->arch == RAI_ARCH_PHI2 || cfg->arch == RAI_ARCH_QWEN2 || cfg->arch == RAI_ARCH_GEMMA ||
                   cfg->arch == RAI_ARCH_PHI3,
               RAI_ERR_UNSUPPORTED, "decoder_create: architecture %d not available", cfg->arch);
@@ -1401,6 +1404,7 @@ int rai_hip_decoder_destroy(rai_hip_decoder *d) {
   if (d->step_graph_n) (void)hipGraphExecDestroy(d->step_graph_n);
   for (void *p : d->allocs) (void)hipFree(p);
   delete d->latent;
+  delete d->hybrid;
   delete d;
   return RAI_OK;
 }
@@ -1427,6 +1431,12 @@ int rai_hip_decoder_param_shape(rai_hip_decoder *d, int32_t i, int64_t *rows, in
   return RAI_OK;
 }
 
+static void parameters_changed(rai_hip_decoder *d) {
+  d->frag_ready = false;   // the fragment-order copies are rebuilt on the next batched decode step
+  if (d->latent) d->latent->derived_ready = false;
+  if (d->hybrid) d->hybrid->derived_ready = false;
+}
+
 int rai_hip_decoder_load_param(rai_hip_decoder *d, const char *name, const void *host_data, size_t bytes) {
   RAI_REQUIRE(d && name && host_data, RAI_ERR_BAD_ARG, "null argument");
   auto it = d->slot_by_name.find(name);
@@ -1445,7 +1455,7 @@ int rai_hip_decoder_load_param(rai_hip_decoder *d, const char *name, const void 
                                 (const char *)host_data + ((size_t)r * s.cols + c) * d->es, row_bytes, (size_t)cg * d->es,
                                 (size_t)rg, hipMemcpyHostToDevice));
     s.loaded = true;
-    if (d->latent) d->latent->derived_ready = false;
+    parameters_changed(d);
     return RAI_OK;
   }
   RAI_HIP_TRY(hipMemcpy2D(s.dst, (size_t)s.pitch * d->es, host_data, row_bytes, row_bytes, rows1, hipMemcpyHostToDevice));
@@ -1453,8 +1463,7 @@ int rai_hip_decoder_load_param(rai_hip_decoder *d, const char *name, const void 
     RAI_HIP_TRY(hipMemcpy2D(s.dst2, (size_t)s.pitch * d->es, (const char *)host_data + rows1 * row_bytes, row_bytes, row_bytes,
                             (size_t)s.rows2, hipMemcpyHostToDevice));
   s.loaded = true;
-  d->frag_ready = false;   // the fragment-order copies are rebuilt on the next batched decode step
-  if (d->latent) d->latent->derived_ready = false;
+  parameters_changed(d);
   return RAI_OK;
 }
 
@@ -1497,7 +1506,7 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
   RAI_TRY(check_call(d, batch, seq));
   hipStream_t st = stream_of(d->dev);
   const size_t rows_bytes = (size_t)batch * seq * d->H * d->es;
-  if (hidden_out_host && !d->hidden_copy && !d->latent) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
+  if (hidden_out_host && !d->hidden_copy && !d->latent && !d->hybrid) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
   if (ids_host) {
     RAI_HIP_TRY(hipMemcpyAsync(d->ids, ids_host, (size_t)batch * seq * sizeof(uint32_t), hipMemcpyHostToDevice, st));
   } else {
@@ -1510,6 +1519,7 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
   d->x_holds_next = false;
   RAI_TRY(rc);
   if (hidden_out_host && d->latent) RAI_TRY(latent_hidden_to_host(d, (int64_t)batch * seq, hidden_out_host));
+  else if (hidden_out_host && d->hybrid) RAI_TRY(hybrid_hidden_to_host(d, (int64_t)batch * seq, hidden_out_host));
   else if (hidden_out_host) RAI_TRY(widen_to_host(d, st, d->hidden_copy, (int64_t)batch * seq * d->H, hidden_out_host));
   if (logits_host) RAI_TRY(widen_to_host(d, st, d->logits, (int64_t)batch * d->V, logits_host));
   if (tokens_host) RAI_TRY(rai_hip_d2h(d->dev, tokens_host, d->tokens, (size_t)batch * sizeof(uint32_t)));
@@ -1525,6 +1535,7 @@ int rai_hip_decoder_forward_hidden(rai_hip_decoder *d, const uint32_t *ids_host,
 // Logits of n rows of the residual stream that the last forward left in hidden_copy (rows: device indices).
 static int head_rows(rai_hip_decoder *d, hipStream_t st, const int *rows_dev, int n, char *gathered, char *logits) {
   if (d->latent) return latent_head_rows(d, st, rows_dev, n, logits);
+  if (d->hybrid) return hybrid_head_rows(d, st, rows_dev, n, logits);
   const int dt = d->cfg.dtype, H = d->H;
   if (dt == RAI_BF16)
     hipLaunchKernelGGL((k_pick_rows<bf16_raw>), dim3(grid1d((int64_t)n * H)), dim3(256), 0, st, (bf16_raw *)gathered,
@@ -1558,7 +1569,7 @@ int rai_hip_decoder_forward_rows(rai_hip_decoder *d, const uint32_t *ids_host, i
     RAI_REQUIRE(rows_host[i] >= 0 && rows_host[i] < batch * seq, RAI_ERR_BAD_ARG, "forward_rows: row %d outside this call's %d tokens",
                 rows_host[i], batch * seq);
   hipStream_t st = stream_of(d->dev);
-  if (!d->hidden_copy && !d->latent && n_rows) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
+  if (!d->hidden_copy && !d->latent && !d->hybrid && n_rows) RAI_TRY(dalloc(d, (size_t)d->max_rows * d->H * d->es, &d->hidden_copy));
   RAI_HIP_TRY(hipMemcpyAsync(d->ids, ids_host, (size_t)batch * seq * sizeof(uint32_t), hipMemcpyHostToDevice, st));
   d->want_hidden = n_rows > 0;
   const int rc = forward_any(d, batch, seq, false);

@@ -19,19 +19,16 @@ namespace rai {
 
 constexpr int kAbsorbRows = 16;   // the flash kernel serves 16 query rows and more
 
-static int pad64(int n) { return (n + 63) / 64 * 64; }
-static int pad_head(int n) { return n <= 32 ? 32 : n <= 64 ? 64 : n <= 128 ? 128 : n <= 192 ? 192 : n <= 256 ? 256 : pad64(n); }
-
 // Device memory that starts as zeros: padding rows and columns are never written by a loader.
-static int zalloc(rai_hip_decoder *d, size_t bytes, char **out) {
+int zalloc(rai_hip_decoder *d, size_t bytes, char **out) {
   RAI_TRY(dalloc(d, bytes, out));
   RAI_HIP_TRY(hipMemset(*out, 0, bytes ? bytes : 16));
   return RAI_OK;
 }
 
 // Rows (columns) in groups of `group`, each padded to `stride` elements.
-static void add_grouped_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch,
-                             int64_t row_group, int64_t row_stride, int64_t col_group, int64_t col_stride) {
+void add_grouped_slot(rai_hip_decoder *d, const std::string &name, int64_t rows, int64_t cols, char *dst, int64_t pitch,
+                      int64_t row_group, int64_t row_stride, int64_t col_group, int64_t col_stride) {
   add_slot(d, name, rows, cols, dst, pitch);
   ParamSlot &s = d->slots.back();
   s.row_group = row_group; s.row_stride = row_stride;

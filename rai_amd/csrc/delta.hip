@@ -1,0 +1,401 @@
+// Gated delta rule with a decay per key channel (see delta.h).
+//   k_delta_prep  convolution + silu, unit vectors, decays and step sizes of every token
+//   k_delta_scan  the recurrence, token after token: a block owns 16 columns of one head's state, 16 lanes to a column
+//   k_delta_out   norm over the head's values, weight and output gate
+//   k_delta_step  all of it for one token per sequence: a block owns a head, its state goes through registers once
+#include <cstdlib>
+
+#include "delta.h"
+
+namespace rai {
+
+__device__ __forceinline__ float dl_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float dl_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+template <typename T> __device__ __forceinline__ float ld(const void *p, int64_t i) { return (float)Scalar<T>::load((const T *)p + i); }
+
+// Sum over the 16 lanes of a row, in every lane.
+__device__ __forceinline__ float row16_sum(float v) {
+#define RAI_ROW_ADD(ctrl) v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), ctrl, 0xf, 0xf, true))
+  RAI_ROW_ADD(0xB1);    // quad_perm [1, 0, 3, 2]
+  RAI_ROW_ADD(0x4E);    // quad_perm [2, 3, 0, 1]
+  RAI_ROW_ADD(0x141);   // mirror within 8 lanes
+  RAI_ROW_ADD(0x140);   // mirror within 16 lanes
+#undef RAI_ROW_ADD
+  return v;
+}
+
+// Channel c of token s after convolution and silu.
+template <typename T>
+__device__ __forceinline__ float conv_silu(const DeltaArgs &a, int b, int s, int pos0, int c) {
+  const DeltaShape &z = a.s;
+  float y = 0.f;
+  for (int j = 0; j < z.taps; ++j) {
+    const int t = s - (z.taps - 1) + j;   // token of this call, or an earlier one in the ring
+    float x = 0.f;
+    if (t >= 0) x = ld<T>(a.dn, ((int64_t)b * a.S + t) * z.ldn + c);
+    else if (pos0 + t >= 0) x = ld<T>(a.ring, ((int64_t)b * z.taps + (pos0 + t) % z.taps) * z.channels + c);
+    y = fmaf(x, ld<T>(a.conv, (int64_t)c * z.taps + j), y);
+  }
+  return y * dl_sigmoid(y);
+}
+
+constexpr int kPrepTokens = 8;
+// A wave takes one unit (a q or k head, a v head, or a head's decays) over kPrepTokens tokens.
+template <typename T, int NI>
+__global__ void __launch_bounds__(256) k_delta_prep(DeltaArgs a) {
+  const DeltaShape &z = a.s;
+  const int lane = threadIdx.x & 63, units = 2 * z.kv_heads + 2 * z.heads;
+  const int64_t job = blockIdx.x * 4ll + (threadIdx.x >> 6);
+  const int groups = (a.S + kPrepTokens - 1) / kPrepTokens;
+  const int unit = (int)(job % units);
+  const int64_t grp = job / units;
+  if (grp >= (int64_t)a.B * groups) return;
+  const int b = (int)(grp / groups), s0 = (int)(grp % groups) * kPrepTokens, s1 = s0 + kPrepTokens < a.S ? s0 + kPrepTokens : a.S;
+  const int pos0 = a.state->pos;
+  if (unit < 2 * z.kv_heads) {
+    const bool query = unit < z.kv_heads;
+    float *dst = (query ? a.q : a.k) + (query ? unit : unit - z.kv_heads) * z.Dk;
+    const float mul = query ? 1.0f / sqrtf((float)z.dim) : 1.0f;
+    for (int s = s0; s < s1; ++s) {
+      float y[NI], sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int c = lane + 64 * i;
+        y[i] = c < z.Dk ? conv_silu<T>(a, b, s, pos0, unit * z.Dk + c) : 0.f;
+        sum = fmaf(y[i], y[i], sum);
+      }
+      const float r = mul / sqrtf(wave_sum(sum) + 1e-6f);
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+        if (lane + 64 * i < z.Dk) dst[((int64_t)b * a.S + s) * z.kv_heads * z.Dk + lane + 64 * i] = y[i] * r;
+    }
+  } else if (unit < 2 * z.kv_heads + z.heads) {
+    const int h = unit - 2 * z.kv_heads;
+    for (int s = s0; s < s1; ++s)
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int c = lane + 64 * i;
+        if (c < z.Vp) a.v[(((int64_t)b * a.S + s) * z.heads + h) * z.Vp + c] = conv_silu<T>(a, b, s, pos0, 2 * z.kv_heads * z.Dk + h * z.Vp + c);
+      }
+  } else {
+    const int h = unit - 2 * z.kv_heads - z.heads;
+    const float rate = -expf(ld<T>(a.A_log, h));
+    for (int s = s0; s < s1; ++s) {
+      const int64_t row = (int64_t)b * a.S + s;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int c = lane + 64 * i;
+        if (c < z.Dk) {
+          float *p = a.decay + (row * z.heads + h) * z.Dk + c;
+          *p = rate * dl_softplus(*p + ld<T>(a.dt_bias, h * z.Dk + c));
+        }
+      }
+      if (lane == 0) a.beta[row * z.heads + h] = dl_sigmoid(ld<T>(a.dn, row * z.ldn + z.off_b + h));
+    }
+  }
+}
+
+// The inputs of the last `taps` tokens of this call go to their places in the ring: the v channels of head h, and with
+// the first head of a group the group's q and k channels.
+template <typename T>
+__device__ __forceinline__ void update_ring(const DeltaArgs &a, int b, int h, int pos0, int tid, int nt) {
+  const DeltaShape &z = a.s;
+  const int rep = z.heads / z.kv_heads, kd = z.kv_heads * z.Dk;
+  const int nqk = h % rep == 0 ? 2 * z.Dk : 0, n = nqk + z.Vp;
+  for (int i = tid; i < n; i += nt) {
+    const int c = i < nqk ? (i < z.Dk ? (h / rep) * z.Dk + i : kd + (h / rep) * z.Dk + i - z.Dk) : 2 * kd + h * z.Vp + i - nqk;
+    for (int s = a.S > z.taps ? a.S - z.taps : 0; s < a.S; ++s)
+      ((T *)a.ring)[((int64_t)b * z.taps + (pos0 + s) % z.taps) * z.channels + c] = ((const T *)a.dn)[((int64_t)b * a.S + s) * z.ldn + c];
+  }
+}
+
+// RPL state rows per lane (16 RPL >= Dk); rows past Dk stay zero.
+constexpr int kScanTokens = 16;
+template <typename T, int RPL>
+__global__ void __launch_bounds__(256) k_delta_scan(DeltaArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float ds_lds[];
+  constexpr int R = 16 * RPL;
+  const DeltaShape &z = a.s;
+  const int tid = threadIdx.x, sub = tid & 15, cl = tid >> 4;
+  const int h = blockIdx.y, b = blockIdx.z, kv = h / (z.heads / z.kv_heads);
+  const int c = blockIdx.x * 16 + cl;          // Vp is a multiple of 32
+  float *qs = ds_lds, *ks = qs + kScanTokens * R, *gs = ks + kScanTokens * R, *vs = gs + kScanTokens * R, *bs = vs + kScanTokens * 16;
+  const int pos0 = a.state->pos;
+  float *st = a.carried + ((int64_t)b * z.heads + h) * z.Dk * z.Vp;
+  float S[RPL];
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) {
+    const int r = sub * RPL + i;
+    S[i] = pos0 > 0 && r < z.Dk ? st[(int64_t)r * z.Vp + c] : 0.f;
+  }
+  for (int s0 = 0; s0 < a.S; s0 += kScanTokens) {
+    const int n = a.S - s0 < kScanTokens ? a.S - s0 : kScanTokens;
+    const int64_t row0 = (int64_t)b * a.S + s0;
+    __syncthreads();
+    for (int e = tid; e < n * R; e += 256) {
+      const int t = e / R, r = e - t * R;
+      const bool in = r < z.Dk;
+      qs[e] = in ? a.q[((row0 + t) * z.kv_heads + kv) * z.Dk + r] : 0.f;
+      ks[e] = in ? a.k[((row0 + t) * z.kv_heads + kv) * z.Dk + r] : 0.f;
+      gs[e] = in ? expf(a.decay[((row0 + t) * z.heads + h) * z.Dk + r]) : 0.f;
+    }
+    if (tid < n * 16) vs[tid] = a.v[((row0 + (tid >> 4)) * z.heads + h) * z.Vp + blockIdx.x * 16 + (tid & 15)];
+    if (tid < n) bs[tid] = a.beta[(row0 + tid) * z.heads + h];
+    __syncthreads();
+    for (int t = 0; t < n; ++t) {
+      const float *q = qs + t * R + sub * RPL, *k = ks + t * R + sub * RPL, *g = gs + t * R + sub * RPL;
+      float kr[RPL], sk = 0.f, sq = 0.f, kq = 0.f;
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        kr[i] = k[i];
+        const float qi = q[i];
+        S[i] *= g[i];
+        sk = fmaf(S[i], kr[i], sk);
+        sq = fmaf(S[i], qi, sq);
+        kq = fmaf(kr[i], qi, kq);
+      }
+      sk = row16_sum(sk);
+      sq = row16_sum(sq);
+      kq = row16_sum(kq);
+      const float u = bs[t] * (vs[t * 16 + cl] - sk);
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) S[i] = fmaf(kr[i], u, S[i]);
+      if (sub == 0) a.o[((row0 + t) * z.heads + h) * z.Vp + c] = fmaf(kq, u, sq);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) {
+    const int r = sub * RPL + i;
+    if (r < z.Dk) st[(int64_t)r * z.Vp + c] = S[i];
+  }
+  if (blockIdx.x == 0) update_ring<T>(a, b, h, pos0, tid, 256);
+}
+
+// One wave per (row, head).
+template <typename T, int NI>
+__global__ void __launch_bounds__(256) k_delta_out(DeltaArgs a) {
+  const DeltaShape &z = a.s;
+  const int lane = threadIdx.x & 63;
+  const int64_t job = blockIdx.x * 4ll + (threadIdx.x >> 6);
+  if (job >= (int64_t)a.B * a.S * z.heads) return;
+  const int h = (int)(job % z.heads);
+  const int64_t row = job / z.heads;
+  float o[NI], sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = lane + 64 * i;
+    o[i] = c < z.vdim ? a.o[job * z.Vp + c] : 0.f;
+    sum = fmaf(o[i], o[i], sum);
+  }
+  const float r = 1.0f / sqrtf(wave_sum(sum) / (float)z.vdim + a.eps);
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = lane + 64 * i;
+    if (c < z.Vp) Scalar<T>::store((T *)a.out + row * a.ldo + h * z.Vp + c, o[i] * r * ld<T>(a.norm_w, c) * dl_sigmoid(ld<T>(a.gate, job * z.Vp + c)));
+  }
+}
+
+// ---------------------------------------------------------------- one token per sequence
+// Thread (column quad cq, row group rg) holds rows rg, rg + RG, ... of four columns: NI of them, requested before
+// anything is computed.  Both sums over the state's rows are formed from the decayed state before the write,
+//   S^T q after the write = (g S)^T q + (k . q) u,
+// so one exchange through LDS serves v's correction and the read-out.
+constexpr int kStepThreads = 512;
+template <typename T> __device__ __forceinline__ float factor_row(const T *w, const T *x, int rank, int part) {
+  constexpr int V = 16 / sizeof(T);
+  struct alignas(16) Pack { T v[V]; };
+  float acc = 0.f;
+  for (int k = part * V; k < rank; k += 4 * V) {
+    const Pack p = *reinterpret_cast<const Pack *>(w + k), y = *reinterpret_cast<const Pack *>(x + k);
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc = fmaf((float)Scalar<T>::load(&p.v[e]), (float)Scalar<T>::load(&y.v[e]), acc);
+  }
+  acc += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(acc), 0xB1, 0xf, 0xf, true));
+  acc += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(acc), 0x4E, 0xf, 0xf, true));
+  return acc;
+}
+
+template <typename T, int NI, bool FACTORS>
+__global__ void __launch_bounds__(kStepThreads) k_delta_step(DeltaArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float st_lds[];
+  const DeltaShape &z = a.s;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int h = blockIdx.x, b = blockIdx.y, rep = z.heads / z.kv_heads, kv = h / rep, kd = z.kv_heads * z.Dk;
+  const int CQ = z.Vp / 4, RG = kStepThreads / CQ, cq = tid % CQ, rg = tid / CQ;
+  float *qs = st_lds, *ks = qs + z.Dk, *gs = ks + z.Dk, *vs = gs + z.Dk, *zs = vs + z.Vp, *us = zs + z.Vp, *red = us + z.Vp;   // red[2][RG][Vp]
+  __shared__ float sums[4], part[kStepThreads / 64];
+  const int pos0 = a.state->pos;
+  float *st = a.carried + ((int64_t)b * z.heads + h) * z.Dk * z.Vp;
+  float4 S[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int r = rg + i * RG;
+    S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (rg < RG && r < z.Dk && pos0 > 0) S[i] = *reinterpret_cast<const float4 *>(st + (int64_t)r * z.Vp + cq * 4);
+  }
+  // ---- convolutions; the ring's free place takes this token's inputs
+  for (int i = tid; i < 2 * z.Dk + z.Vp; i += kStepThreads) {
+    const int c = i < z.Dk ? kv * z.Dk + i : i < 2 * z.Dk ? kd + kv * z.Dk + i - z.Dk : 2 * kd + h * z.Vp + i - 2 * z.Dk;
+    (i < 2 * z.Dk ? qs : vs - 2 * z.Dk)[i] = conv_silu<T>(a, b, 0, pos0, c);   // ks follows qs
+    if (i >= 2 * z.Dk || h % rep == 0) ((T *)a.ring)[((int64_t)b * z.taps + pos0 % z.taps) * z.channels + c] = ((const T *)a.dn)[b * z.ldn + c];
+  }
+  // ---- decays and gate
+  const float rate = -expf(ld<T>(a.A_log, h));
+  if constexpr (FACTORS) {
+    const T *a1 = (const T *)a.dn + b * z.ldn + z.off_a1, *g1 = (const T *)a.dn + b * z.ldn + z.off_g1;
+    for (int r = tid >> 2; r < z.Dk + z.Vp; r += kStepThreads / 4) {
+      const bool dec = r < z.Dk;
+      const int n = dec ? h * z.Dk + r : h * z.Vp + r - z.Dk;
+      const float y = dec ? factor_row<T>((const T *)a.a2 + (int64_t)n * a.a_rank, a1, a.a_rank, tid & 3)
+                          : factor_row<T>((const T *)a.g2 + (int64_t)n * a.g_rank, g1, a.g_rank, tid & 3);
+      if ((tid & 3) == 0) {
+        if (dec) gs[r] = expf(rate * dl_softplus(y + ld<T>(a.dt_bias, n)));
+        else zs[r - z.Dk] = dl_sigmoid(y);
+      }
+    }
+  } else {
+    for (int r = tid; r < z.Dk; r += kStepThreads)
+      gs[r] = expf(rate * dl_softplus(a.decay[((int64_t)b * z.heads + h) * z.Dk + r] + ld<T>(a.dt_bias, h * z.Dk + r)));
+    for (int c = tid; c < z.Vp; c += kStepThreads) zs[c] = dl_sigmoid(ld<T>(a.gate, ((int64_t)b * z.heads + h) * z.Vp + c));
+  }
+  const float beta = dl_sigmoid(ld<T>(a.dn, b * z.ldn + z.off_b + h));
+  __syncthreads();
+  if (wave < 3) {   // |q|^2, |k|^2, k . q
+    const float *x = wave == 0 ? qs : ks, *y = wave == 1 ? ks : qs;
+    float s = 0.f;
+    for (int r = lane; r < z.Dk; r += 64) s = fmaf(x[r], y[r], s);
+    s = wave_sum(s);
+    if (lane == 0) sums[wave] = s;
+  }
+  float sk[4] = {0.f, 0.f, 0.f, 0.f}, sq[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int r = rg + i * RG;
+    if (rg < RG && r < z.Dk) {
+      const float g = gs[r], k = ks[r], q = qs[r];
+      S[i].x *= g; S[i].y *= g; S[i].z *= g; S[i].w *= g;
+      sk[0] = fmaf(S[i].x, k, sk[0]); sk[1] = fmaf(S[i].y, k, sk[1]); sk[2] = fmaf(S[i].z, k, sk[2]); sk[3] = fmaf(S[i].w, k, sk[3]);
+      sq[0] = fmaf(S[i].x, q, sq[0]); sq[1] = fmaf(S[i].y, q, sq[1]); sq[2] = fmaf(S[i].z, q, sq[2]); sq[3] = fmaf(S[i].w, q, sq[3]);
+    }
+  }
+  if (rg < RG) {
+    *reinterpret_cast<float4 *>(red + rg * z.Vp + cq * 4) = make_float4(sk[0], sk[1], sk[2], sk[3]);
+    *reinterpret_cast<float4 *>(red + (RG + rg) * z.Vp + cq * 4) = make_float4(sq[0], sq[1], sq[2], sq[3]);
+  }
+  __syncthreads();
+  const float rk = 1.0f / sqrtf(sums[1] + 1e-6f), rq = 1.0f / sqrtf(sums[0] + 1e-6f) / sqrtf((float)z.dim);
+  float o = 0.f;
+  if (tid < z.Vp) {
+    float x = 0.f, y = 0.f;
+    for (int g = 0; g < RG; ++g) {
+      x += red[g * z.Vp + tid];
+      y += red[(RG + g) * z.Vp + tid];
+    }
+    const float u = beta * (vs[tid] - rk * x);
+    us[tid] = u * rk;                                // what a row of the raw k is multiplied with
+    o = fmaf(sums[2] * rk * rq, u, rq * y);
+  }
+  const float s2 = wave_sum(tid < z.vdim ? o * o : 0.f);
+  if (lane == 0) part[wave] = s2;
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int r = rg + i * RG;
+    if (rg < RG && r < z.Dk) {
+      const float k = ks[r];
+      const float4 u = *reinterpret_cast<const float4 *>(us + cq * 4);
+      S[i].x = fmaf(k, u.x, S[i].x); S[i].y = fmaf(k, u.y, S[i].y); S[i].z = fmaf(k, u.z, S[i].z); S[i].w = fmaf(k, u.w, S[i].w);
+      *reinterpret_cast<float4 *>(st + (int64_t)r * z.Vp + cq * 4) = S[i];
+    }
+  }
+  if (tid < z.Vp) {
+    float t = 0.f;
+    for (int w = 0; w < kStepThreads / 64; ++w) t += part[w];
+    const float r = 1.0f / sqrtf(t / (float)z.vdim + a.eps);
+    Scalar<T>::store((T *)a.out + b * a.ldo + h * z.Vp + tid, o * r * ld<T>(a.norm_w, tid) * zs[tid]);
+  }
+}
+
+// ---------------------------------------------------------------- launchers
+static int check_delta(const DeltaArgs &a) {
+  const DeltaShape &z = a.s;
+  RAI_REQUIRE(z.heads > 0 && z.kv_heads > 0 && z.heads % z.kv_heads == 0 && z.taps > 0 && z.Dk % 32 == 0 && z.Vp % 32 == 0 && z.dim <= z.Dk && z.vdim <= z.Vp &&
+                  z.Dk <= kDeltaMaxHead && z.Vp <= kDeltaMaxHead && z.channels == 2 * z.kv_heads * z.Dk + z.heads * z.Vp,
+              RAI_ERR_BAD_SHAPE, "delta rule: %d / %d heads of %d x %d", z.heads, z.kv_heads, z.dim, z.vdim);
+  RAI_REQUIRE(a.B > 0 && a.S > 0 && a.B <= 65535 && z.heads <= 65535, RAI_ERR_UNSUPPORTED, "delta rule: %d sequences of %d heads", a.B, z.heads);
+  return RAI_OK;
+}
+
+template <typename T, int RPL> static int launch_scan(hipStream_t st, const DeltaArgs &a) {
+  const size_t lds = (size_t)kScanTokens * (3 * 16 * RPL + 16 + 1) * sizeof(float);
+  static bool attr_set = false;
+  if (lds > 64 * 1024 && !attr_set) {
+    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_delta_scan<T, RPL>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    attr_set = true;
+  }
+  hipLaunchKernelGGL((k_delta_scan<T, RPL>), dim3(a.s.Vp / 16, a.s.heads, a.B), dim3(256), lds, st, a);
+  return launch_check("delta_scan");
+}
+
+template <typename T> static int launch_tokens_t(hipStream_t st, const DeltaArgs &a) {
+  const DeltaShape &z = a.s;
+  const int wide = z.Dk > z.Vp ? z.Dk : z.Vp;
+  const int64_t jobs = (int64_t)a.B * ((a.S + kPrepTokens - 1) / kPrepTokens) * (2 * z.kv_heads + 2 * z.heads);
+  const int64_t outs = (int64_t)a.B * a.S * z.heads;
+  RAI_REQUIRE((jobs + 3) / 4 < (1ll << 31) && (outs + 3) / 4 < (1ll << 31), RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
+  const dim3 gp((unsigned)((jobs + 3) / 4)), go((unsigned)((outs + 3) / 4)), block(256);
+  if (wide <= 64) hipLaunchKernelGGL((k_delta_prep<T, 1>), gp, block, 0, st, a);
+  else if (wide <= 128) hipLaunchKernelGGL((k_delta_prep<T, 2>), gp, block, 0, st, a);
+  else if (wide <= 256) hipLaunchKernelGGL((k_delta_prep<T, 4>), gp, block, 0, st, a);
+  else hipLaunchKernelGGL((k_delta_prep<T, 8>), gp, block, 0, st, a);
+  RAI_TRY(launch_check("delta_prep"));
+  if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
+  else if (z.Dk <= 64) RAI_TRY((launch_scan<T, 4>(st, a)));
+  else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));
+  else if (z.Dk <= 256) RAI_TRY((launch_scan<T, 16>(st, a)));
+  else RAI_TRY((launch_scan<T, 32>(st, a)));
+  if (z.Vp <= 64) hipLaunchKernelGGL((k_delta_out<T, 1>), go, block, 0, st, a);
+  else if (z.Vp <= 128) hipLaunchKernelGGL((k_delta_out<T, 2>), go, block, 0, st, a);
+  else if (z.Vp <= 256) hipLaunchKernelGGL((k_delta_out<T, 4>), go, block, 0, st, a);
+  else hipLaunchKernelGGL((k_delta_out<T, 8>), go, block, 0, st, a);
+  return launch_check("delta_out");
+}
+
+int launch_delta_tokens(hipStream_t st, int dtype, const DeltaArgs &a) {
+  RAI_TRY(check_delta(a));
+  return dtype == RAI_BF16 ? launch_tokens_t<bf16_raw>(st, a) : launch_tokens_t<float>(st, a);
+}
+
+static int step_rows(const DeltaShape &z) {   // state rows per thread
+  const int RG = kStepThreads / (z.Vp / 4);
+  return (z.Dk + RG - 1) / RG;
+}
+bool delta_step_serves(const DeltaShape &z) {
+  return z.Dk % 32 == 0 && z.Vp % 32 == 0 && z.Dk <= kDeltaMaxHead && z.Vp <= kDeltaMaxHead && step_rows(z) <= 32;
+}
+
+template <typename T, int NI> static int launch_step_n(hipStream_t st, const DeltaArgs &a) {
+  const DeltaShape &z = a.s;
+  const int RG = kStepThreads / (z.Vp / 4);
+  const size_t lds = (size_t)(3 * z.Dk + 3 * z.Vp + 2 * RG * z.Vp) * sizeof(float);   // at most 28 KB
+  const dim3 grid(z.heads, a.B), block(kStepThreads);
+  if (a.a2) hipLaunchKernelGGL((k_delta_step<T, NI, true>), grid, block, lds, st, a);
+  else hipLaunchKernelGGL((k_delta_step<T, NI, false>), grid, block, lds, st, a);
+  return launch_check("delta_step");
+}
+template <typename T> static int launch_step_t(hipStream_t st, const DeltaArgs &a) {
+  const int n = step_rows(a.s);
+  if (n <= 2) return launch_step_n<T, 2>(st, a);
+  if (n <= 4) return launch_step_n<T, 4>(st, a);
+  if (n <= 8) return launch_step_n<T, 8>(st, a);
+  if (n <= 16) return launch_step_n<T, 16>(st, a);
+  return launch_step_n<T, 32>(st, a);
+}
+int launch_delta_step(hipStream_t st, int dtype, const DeltaArgs &a) {
+  RAI_TRY(check_delta(a));
+  RAI_REQUIRE(a.S == 1 && delta_step_serves(a.s) && (a.a2 == nullptr) == (a.g2 == nullptr) && (!a.a2 || (a.a_rank % 8 == 0 && a.g_rank % 8 == 0)),
+              RAI_ERR_BAD_ARG, "delta step: not served");
+  return dtype == RAI_BF16 ? launch_step_t<bf16_raw>(st, a) : launch_step_t<float>(st, a);
+}
+
+}  // namespace rai

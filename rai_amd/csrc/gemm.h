@@ -28,6 +28,7 @@ struct LinearArgs {
   int n_split;   // first column written to out2
   int act;       // rai_hip_unary_op activation or -1
   int act_from;  // activation applies to columns >= act_from
+  float act_limit, act_alpha;  // kActClampedGlu only
   // != 0: residual (when given) and out1 are f32 whatever the operands' dtype, and out = residual + out_scale *
   // act(acc + bias): a residual stream kept in f32 under bf16 products, or plain f32 results (router logits) without a
   // residual.  One output, no gated pairs.
@@ -127,12 +128,29 @@ int launch_gemv_group(hipStream_t st, GemvGroupArgs g);
 int launch_linear_f32(hipStream_t st, const LinearArgs &a);
 bool linear_mfma_fuses_norm(int M, int K, int ln_kind);
 
+// Gated pairs only (glu != 0): with a = min(gate, limit) and b = up cut off at +-limit,  a sigmoid(alpha a) (b + 1).
+constexpr int kActClampedGlu = RAI_UN_COUNT_;
+__device__ __forceinline__ float glu_clamped(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+// The same through the hardware exponential and reciprocal, for results that are rounded to bf16.
+__device__ __forceinline__ float glu_clamped_bf16_out(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * g)) * (u + 1.0f);
+}
 __device__ __forceinline__ float act_eval(int act, float x);
 // act(gate) * up with the reference's roundings of gate, act(gate) and up to bf16.
 __device__ __forceinline__ float glu_bf16(int act, float g, float u) {
   const float gr = bf16_bits_to_f32(f32_to_bf16_bits(g));
   const float ar = bf16_bits_to_f32(f32_to_bf16_bits(act_eval(act, gr)));
   return ar * bf16_bits_to_f32(f32_to_bf16_bits(u));
+}
+
+__device__ __forceinline__ float glu_bf16(const LinearArgs &a, float g, float u) {
+  return a.act == kActClampedGlu ? glu_clamped_bf16_out(g, u, a.act_limit, a.act_alpha) : glu_bf16(a.act, g, u);
 }
 
 __device__ __forceinline__ float act_eval(int act, float x) {

@@ -202,7 +202,7 @@ __global__ void __launch_bounds__(NWV * 64) k_linear_bf16_skinny(LinearArgs a, i
             for (int m = 0; m < MROWS; ++m) {
               if (m >= a.M) break;
               ((uint16_t *)a.out1)[(int64_t)m * a.ld1 + (n >> 1)] =
-                  f32_to_bf16_bits(glu_bf16(a.act, acc[r][m] + bg, acc[r + 1][m] + bu));
+                  f32_to_bf16_bits(glu_bf16(a, acc[r][m] + bg, acc[r + 1][m] + bu));
             }
           }
         }
@@ -359,7 +359,7 @@ __device__ __forceinline__ void gemv_reg_rows(const LinearArgs &a, int n_begin, 
           const int n = n_base + r;
           if (n + 1 >= a.N || n >= n_end) break;
           const float bg = bias ? bf16_bits_to_f32(bias[n]) : 0.f, bu = bias ? bf16_bits_to_f32(bias[n + 1]) : 0.f;
-          ((uint16_t *)a.out1)[n >> 1] = f32_to_bf16_bits(glu_bf16(a.act, acc[r] + bg, acc[r + 1] + bu));
+          ((uint16_t *)a.out1)[n >> 1] = f32_to_bf16_bits(glu_bf16(a, acc[r] + bg, acc[r + 1] + bu));
         }
       }
     } else if (lane == 0) {
@@ -469,7 +469,7 @@ __device__ __forceinline__ void linear_f32_tile(const LinearArgs &a, int tile_m,
         int n = n0 + tx * 4 + j;
         if (n + 1 >= a.N) continue;
         float g = acc[i][j] + (bias ? bias[n] : 0.f), u = acc[i][j + 1] + (bias ? bias[n + 1] : 0.f);
-        ((float *)a.out1)[(int64_t)m * a.ld1 + (n >> 1)] = act_eval(a.act, g) * u;
+        ((float *)a.out1)[(int64_t)m * a.ld1 + (n >> 1)] = a.act == kActClampedGlu ? glu_clamped(g, u, a.act_limit, a.act_alpha) : act_eval(a.act, g) * u;
       }
     }
     return;

@@ -182,15 +182,19 @@ __device__ __forceinline__ void gemm_tile_epilogue(const LinearArgs &a, f32x16 (
       }
       if (a.glu) {  // columns n..n+7 are four (gate, up) pairs -> four outputs at column n/2
         uint16_t *dst = (uint16_t *)a.out1 + (int64_t)m * a.ld1 + (n >> 1);
-        float gr[8], ga[4];
+        float gr[8], ga[4], gl[4];
+        if (a.act == kActClampedGlu) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) gr[e] = bf16_bits_to_f32(f32_to_bf16_bits(v[e] + bv[e]));  // gate / up rounded to bf16 as the reference does
+          for (int e = 0; e < 4; ++e) gl[e] = glu_clamped_bf16_out(v[2 * e] + bv[2 * e], v[2 * e + 1] + bv[2 * e + 1], a.act_limit, a.act_alpha);
+        } else {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) ga[e] = gr[2 * e];
-        act_n<4>(a.act, ga, 0, 0);   // the four gates
-        float gl[4];
+          for (int e = 0; e < 8; ++e) gr[e] = bf16_bits_to_f32(f32_to_bf16_bits(v[e] + bv[e]));  // gate / up rounded to bf16 as the reference does
 #pragma unroll
-        for (int e = 0; e < 4; ++e) gl[e] = bf16_bits_to_f32(f32_to_bf16_bits(ga[e])) * gr[2 * e + 1];
+          for (int e = 0; e < 4; ++e) ga[e] = gr[2 * e];
+          act_n<4>(a.act, ga, 0, 0);   // the four gates
+#pragma unroll
+          for (int e = 0; e < 4; ++e) gl[e] = bf16_bits_to_f32(f32_to_bf16_bits(ga[e])) * gr[2 * e + 1];
+        }
         if (whole && a.ld1 % 4 == 0 && (uintptr_t)a.out1 % 8 == 0) {
           typedef __attribute__((ext_vector_type(2))) uint32_t u32x2;
           u32x2 o = {pack_bf16x2(gl[0], gl[1]), pack_bf16x2(gl[2], gl[3])};
@@ -890,7 +894,7 @@ __global__ void __launch_bounds__(256) k_splitk_epilogue(LinearArgs a, int split
       for (int s = 0; s < splits; ++s) { g += partial[(int64_t)s * total + e]; u += partial[(int64_t)s * total + e + 1]; }
       g += bias ? bf16_bits_to_f32(bias[n]) : 0.f;
       u += bias ? bf16_bits_to_f32(bias[n + 1]) : 0.f;
-      ((uint16_t *)a.out1)[(int64_t)m * a.ld1 + (n >> 1)] = f32_to_bf16_bits(glu_bf16(a.act, g, u));
+      ((uint16_t *)a.out1)[(int64_t)m * a.ld1 + (n >> 1)] = f32_to_bf16_bits(glu_bf16(a, g, u));
       continue;
     }
     float x = 0.f;
@@ -1352,7 +1356,7 @@ __global__ void __launch_bounds__(256) k_linear_bf16_mfma_skinny(LinearArgs a, i
       for (int e = 0; e < 4 && n + e + 1 < a.N; e += 2) {
         const float g = v[e] + (bias ? bf16_bits_to_f32(bias[n + e]) : 0.f);
         const float u = v[e + 1] + (bias ? bf16_bits_to_f32(bias[n + e + 1]) : 0.f);
-        dst[e >> 1] = f32_to_bf16_bits(glu_bf16(a.act, g, u));
+        dst[e >> 1] = f32_to_bf16_bits(glu_bf16(a, g, u));
       }
       continue;
     }
@@ -1585,7 +1589,7 @@ __global__ void __launch_bounds__(512) k_linear_bf16_mfma_stream(LinearArgs a, i
       for (int e = 0; e < 2; ++e) {
         const float gt = x[2 * e] + (bias ? bf16_bits_to_f32(bias[n + 2 * e]) : 0.f);
         const float up = x[2 * e + 1] + (bias ? bf16_bits_to_f32(bias[n + 2 * e + 1]) : 0.f);
-        o[e] = f32_to_bf16_bits(glu_bf16(a.act, gt, up));
+        o[e] = f32_to_bf16_bits(glu_bf16(a, gt, up));
       }
       uint16_t *dst = (uint16_t *)a.out1 + (int64_t)m * a.ld1 + (n >> 1);
       if (((uintptr_t)dst & 3) == 0) *reinterpret_cast<uint32_t *>(dst) = (uint32_t)o[0] | ((uint32_t)o[1] << 16);

@@ -1,4 +1,4 @@
-// Launchers of the latent-attention family's kernels: grouped RMS norms of an f32 residual stream (norm.hip), attention
+// Launchers of the latent-attention family's kernels: norms of an f32 residual stream (norm.hip), attention
 // over cached latents (latent_attention.hip) and the mixture of experts (moe.hip).  `dtype` is RAI_BF16 or RAI_F32
 // throughout; "T" below stands for its storage type.
 #pragma once
@@ -10,8 +10,11 @@ namespace rai {
 
 // Row r of the output is row first + r * step of the stream.  The row is src (f32 stream or T rows) plus
 //   add_scale * sum_j add[add_rows[row * top + j], :]
-// (the pending outputs of a mixture), is written back to `x` when given, and is normalised in `groups` equal runs, each
-// by its own 1 / sqrt(mean square + eps); h1 = normalised * w1 and, when given, h2 = normalised * w2.
+// (the pending outputs of a mixture), times src_scale, is written back to `x` when given, and is normalised in `groups`
+// equal runs, each by its own 1 / sqrt(mean square + eps); h1 = normalised * w1 * h_scale and, when given,
+// h2 = normalised * w2 * h_scale.  kStreamLayerNorm: one run, and its mean is taken off first.  kStreamCopy: not
+// normalised at all, no weights.
+enum StreamNormKind { kStreamRms = 0, kStreamLayerNorm = 1, kStreamCopy = 2 };
 struct StreamNormArgs {
   const void *src;
   int src_f32;
@@ -30,6 +33,8 @@ struct StreamNormArgs {
   float eps;
   int64_t rows, first, step;
   const int *row_map;  // explicit stream row of each output row instead of first + r * step
+  int kind;            // StreamNormKind
+  float src_scale, h_scale;   // 0 stands for 1
 };
 int launch_stream_norm(hipStream_t st, int dtype, const StreamNormArgs &a);
 
@@ -79,11 +84,16 @@ struct LatentInArgs {
   int H, groups, K;             // width, norm groups, padded width
   float eps;
   int64_t ldw;
+  int kind;                     // StreamNormKind; kStreamCopy: no norm, n1 and n2 are not read
+  float src_scale, h_scale;     // 0 stands for 1: what the source and the norm's output are multiplied with
   const void *W1, *n1;          // rows on the first norm's output -> bf16
   int N1;
   void *out1;
   const void *W2, *n2;          // rows on the second norm's: gated pairs -> bf16 out2[n / 2], or plain -> f32 out2[n]
   int N2, gated2, act;
+  float act_limit, act_alpha;   // kActClampedGlu
+  const float *add2;            // plain form: out2[n] = product + add2[n] + bias2[n], either may be null
+  const void *bias2;
   void *out2;
   void *h2;                     // the second norm's output, for the experts; null: not kept
   int waves1, rows_per_wave;    // filled in by the launcher
@@ -135,6 +145,7 @@ struct LatentDownArgs {
   const int *choice;
   const void *res;
   int res_f32, H, N, rows;
+  float res_scale;   // 0 stands for 1
   float mult;
   float *out;
 };

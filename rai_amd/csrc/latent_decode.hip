@@ -34,6 +34,9 @@ __device__ __forceinline__ float ld_dot8(ld_u32x4 a, ld_u32x4 b, float c) {
 __device__ __forceinline__ float lo_f32(uint32_t w) { return __uint_as_float(w << 16); }
 __device__ __forceinline__ float hi_f32(uint32_t w) { return __uint_as_float(w & 0xffff0000u); }
 __device__ __forceinline__ float gated(int act, float g, float u) { return act_eval(act, g) * u; }
+__device__ __forceinline__ float gated(const LatentInArgs &a, float g, float u) {
+  return a.act == kActClampedGlu ? glu_clamped_bf16_out(g, u, a.act_limit, a.act_alpha) : gated(a.act, g, u);
+}
 
 // R rows of W in flight, rows n .. n + R - 1 clamped to n_last.
 template <int KC, int R> struct RowSet {
@@ -88,7 +91,7 @@ __global__ void __launch_bounds__(256) k_latent_in(LatentInArgs a) {
 #pragma unroll
     for (int e = 0; e < 8; ++e) x[u][e] = 0.f;
     if (k < a.H) {
-      wn[u] = *reinterpret_cast<const ld_u32x4 *>(nw + u * 512);
+      if (a.kind != kStreamCopy) wn[u] = *reinterpret_cast<const ld_u32x4 *>(nw + u * 512);
       if (a.src_f32) {
         const ld_f32x4 v0 = *reinterpret_cast<const ld_f32x4 *>((const float *)a.src + k), v1 = *reinterpret_cast<const ld_f32x4 *>((const float *)a.src + k + 4);
 #pragma unroll
@@ -102,7 +105,26 @@ __global__ void __launch_bounds__(256) k_latent_in(LatentInArgs a) {
   }
   RowSet<KC, 2> rs;
   rs.load(W, a.ldw, n0, n1 - 1, a.K, lane);
+  if (a.src_scale != 0.f) {
+#pragma unroll
+    for (int u = 0; u < KC; ++u)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[u][e] *= a.src_scale;
+  }
+  if (a.kind == kStreamLayerNorm) {
+    float s = 0.f;
+#pragma unroll
+    for (int u = 0; u < KC; ++u)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s += x[u][e];
+    const float mean = wave_sum(s) / (float)a.H;
+#pragma unroll
+    for (int u = 0; u < KC; ++u)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[u][e] = lane * 8 + u * 512 < a.H ? x[u][e] - mean : 0.f;
+  }
   const int gsize = a.H / a.groups;
+  const float h_scale = a.h_scale != 0.f ? a.h_scale : 1.0f;
   float q[KC], sc[KC];
   int grp[KC];
 #pragma unroll
@@ -116,11 +138,18 @@ __global__ void __launch_bounds__(256) k_latent_in(LatentInArgs a) {
     float s = 0.f;
 #pragma unroll
     for (int u = 0; u < KC; ++u) s += grp[u] == g ? q[u] : 0.f;
-    s = 1.0f / sqrtf(wave_sum(s) / (float)gsize + a.eps);
+    s = h_scale / sqrtf(wave_sum(s) / (float)gsize + a.eps);
 #pragma unroll
     for (int u = 0; u < KC; ++u) sc[u] = grp[u] == g ? s : sc[u];
   }
   ld_u32x4 xv[KC];
+  if (a.kind == kStreamCopy) {
+#pragma unroll
+    for (int u = 0; u < KC; ++u) {
+      sc[u] = h_scale;
+      wn[u] = ld_u32x4{0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u};   // ones
+    }
+  }
 #pragma unroll
   for (int u = 0; u < KC; ++u)
 #pragma unroll
@@ -136,9 +165,11 @@ __global__ void __launch_bounds__(256) k_latent_in(LatentInArgs a) {
       o[0] = f32_to_bf16_bits(v0);
       if (n + 1 < n1) o[1] = f32_to_bf16_bits(v1);
     } else if (a.gated2) {
-      ((uint16_t *)a.out2)[n >> 1] = f32_to_bf16_bits(gated(a.act, v0, v1));
+      ((uint16_t *)a.out2)[n >> 1] = f32_to_bf16_bits(gated(a, v0, v1));
     } else {
       float *o = (float *)a.out2 + n;
+      if (a.add2) { v0 += a.add2[n]; if (n + 1 < n1) v1 += a.add2[n + 1]; }
+      if (a.bias2) { v0 += bf16_bits_to_f32(((const uint16_t *)a.bias2)[n]); if (n + 1 < n1) v1 += bf16_bits_to_f32(((const uint16_t *)a.bias2)[n + 1]); }
       o[0] = v0;
       if (n + 1 < n1) o[1] = v1;
     }
@@ -291,6 +322,7 @@ __global__ void __launch_bounds__(kDownThreads) k_latent_down(LatentDownArgs a) 
   const int n = blockIdx.x * kDownWaves + (tid >> 6);
   float res = 0.f;
   if (n < a.H) res = a.res_f32 ? ((const float *)a.res)[n] : bf16_bits_to_f32(((const uint16_t *)a.res)[n]);
+  if (a.res_scale != 0.f) res *= a.res_scale;
   for (int c = tid; c < chunks; c += kDownThreads) {
     DownChunk d;
     if (c < c0) {

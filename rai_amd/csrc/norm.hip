@@ -226,11 +226,11 @@ k_rope_tables(TT *cos_t, TT *sin_t, int64_t max_pos, int rot, double theta, int 
   }
 }
 
-// ---------------------------------------------------------------- grouped RMS norm of an f32 residual stream
+// ---------------------------------------------------------------- norms of an f32 residual stream
 // One block per output row (see StreamNormArgs).  A thread owns packs of V elements, tid, tid + 256, ...; the first
 // ITEMS of them stay in registers between the two passes, any others are formed again (ITEMS == 0: all of them).  The
 // sum of squares of a pack goes to LDS and one wave sums each group's packs in a fixed order, so the statistics do not
-// depend on how a group's packs fall on the waves.
+// depend on how a group's packs fall on the waves.  A layer norm sums the packs themselves first, in the same way.
 template <typename T, int V, int ITEMS>
 __global__ void __launch_bounds__(256) k_stream_norm(StreamNormArgs a) {
   extern __shared__ float sn_lds[];   // [packs] sums of squares | [groups] scales
@@ -263,20 +263,45 @@ __global__ void __launch_bounds__(256) k_stream_norm(StreamNormArgs a) {
 #pragma unroll
       for (int e = 0; e < V; ++e) v[e] = fmaf(a.add_scale, sum[e], v[e]);
     }
+    if (a.src_scale != 0.f) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] *= a.src_scale;
+    }
   };
   float keep[ITEMS > 0 ? ITEMS : 1][V];
+  float mean = 0.f;
   auto square = [&](int p, const float (&v)[V]) {
     float q = 0.f;
 #pragma unroll
-    for (int e = 0; e < V; ++e) q = fmaf(v[e], v[e], q);
+    for (int e = 0; e < V; ++e) q = fmaf(v[e] - mean, v[e] - mean, q);
     sn_lds[p] = q;
   };
 #pragma unroll
   for (int i = 0; i < ITEMS; ++i)
-    if (tid + i * 256 < packs) {
-      form(tid + i * 256, keep[i]);
-      square(tid + i * 256, keep[i]);
+    if (tid + i * 256 < packs) form(tid + i * 256, keep[i]);
+  if (a.kind == kStreamLayerNorm) {
+    auto total = [&](int p, const float (&v)[V]) {
+      float q = 0.f;
+#pragma unroll
+      for (int e = 0; e < V; ++e) q += v[e];
+      sn_lds[p] = q;
+    };
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i)
+      if (tid + i * 256 < packs) total(tid + i * 256, keep[i]);
+    for (int p = tid + ITEMS * 256; p < packs; p += 256) {
+      float v[V];
+      form(p, v);
+      total(p, v);
     }
+    __syncthreads();
+    for (int p = lane; p < packs; p += 64) mean += sn_lds[p];   // every wave for itself
+    mean = wave_sum(mean) / (float)a.width;
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < ITEMS; ++i)
+    if (tid + i * 256 < packs) square(tid + i * 256, keep[i]);
   for (int p = tid + ITEMS * 256; p < packs; p += 256) {
     float v[V];
     form(p, v);
@@ -287,7 +312,7 @@ __global__ void __launch_bounds__(256) k_stream_norm(StreamNormArgs a) {
     float q = 0.f;
     for (int p = lane; p < gpacks; p += 64) q += sn_lds[g * gpacks + p];
     q = wave_sum(q);
-    if (lane == 0) scale[g] = 1.0f / sqrtf(q / (float)(gpacks * V) + a.eps);
+    if (lane == 0) scale[g] = (a.kind == kStreamCopy ? 1.0f : 1.0f / sqrtf(q / (float)(gpacks * V) + a.eps)) * (a.h_scale != 0.f ? a.h_scale : 1.0f);
   }
   __syncthreads();
   auto finish = [&](int p, const float (&v)[V]) {
@@ -299,10 +324,15 @@ __global__ void __launch_bounds__(256) k_stream_norm(StreamNormArgs a) {
       *reinterpret_cast<NPack<float, V> *>(a.x + row * a.x_ld + p * V) = o;
     }
     auto put = [&](const void *w, void *h) {
-      const NPack<T, V> wp = *reinterpret_cast<const NPack<T, V> *>((const T *)w + p * V);
       NPack<T, V> o;
+      if (a.kind == kStreamCopy) {
 #pragma unroll
-      for (int e = 0; e < V; ++e) Scalar<T>::store(&o.v[e], v[e] * sc * (float)Scalar<T>::load(&wp.v[e]));
+        for (int e = 0; e < V; ++e) Scalar<T>::store(&o.v[e], v[e] * sc);
+      } else {
+        const NPack<T, V> wp = *reinterpret_cast<const NPack<T, V> *>((const T *)w + p * V);
+#pragma unroll
+        for (int e = 0; e < V; ++e) Scalar<T>::store(&o.v[e], (v[e] - mean) * sc * (float)Scalar<T>::load(&wp.v[e]));
+      }
       *reinterpret_cast<NPack<T, V> *>((T *)h + r * a.h_ld + p * V) = o;
     };
     if (a.h1) put(a.w1, a.h1);
@@ -337,7 +367,7 @@ template <typename T> static int launch_stream_norm_t(hipStream_t st, const Stre
 }
 
 int launch_stream_norm(hipStream_t st, int dtype, const StreamNormArgs &a) {
-  RAI_REQUIRE(a.rows > 0 && a.width > 0 && a.groups > 0 && a.width % a.groups == 0 && a.h_ld >= a.width, RAI_ERR_BAD_SHAPE,
+  RAI_REQUIRE(a.rows > 0 && a.width > 0 && a.groups > 0 && a.width % a.groups == 0 && a.h_ld >= a.width && (a.kind != kStreamLayerNorm || a.groups == 1), RAI_ERR_BAD_SHAPE,
               "stream norm: width %d in %d groups", a.width, a.groups);
   return dtype == RAI_BF16 ? launch_stream_norm_t<bf16_raw>(st, a) : launch_stream_norm_t<float>(st, a);
 }

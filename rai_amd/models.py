@@ -11,7 +11,8 @@ import ctypes as C
 import numpy as np
 
 from . import _lib
-from ._lib import ARCH, DTYPE_BY_NAME, MLP_KIND, UNARY, DecoderConfig, LatentConfig, LatentLayer, call
+from ._lib import (ARCH, DTYPE_BY_NAME, MIXER, MLP_KIND, UNARY, DecoderConfig, HybridConfig, HybridLayer, LatentConfig, LatentLayer,
+                   call)
 
 _ACT = {"gelu_new": "new_gelu", "new_gelu": "new_gelu", "gelu": "gelu", "silu": "silu", "relu": "relu"}
 
@@ -71,6 +72,33 @@ class Decoder:
         self.dtype, self.dev = dtype, dev
         call("rai_hip_init", dev)
         call("rai_hip_decoder_create_latent", dev, C.byref(c), arr, C.byref(self._h))
+        return self
+
+    @classmethod
+    def hybrid(cls, dtype, *, vocab_size, width, layers, norm_eps, embed_scale=1.0, logit_scale=1.0, loop=None, max_batch=1,
+               max_context=2048, dev=0):
+        """A decoder of attention and gated delta rule layers described one by one (rai_hip_decoder_create_hybrid): every
+        entry of `layers` is a dict with the fields of _lib.HybridLayer; mixer and mlp_kind by name.  `loop`: (start, stop,
+        times) of the layers that run several times, or None."""
+        start, stop, times = loop or (0, 0, 0)
+        c = HybridConfig(dtype=DTYPE_BY_NAME[dtype], vocab_size=vocab_size, width=width, num_layers=len(layers), loop_start=start,
+                         loop_stop=stop, loop_times=times, max_batch=max_batch, max_context=max_context, norm_eps=norm_eps,
+                         embed_scale=embed_scale, logit_scale=logit_scale)
+        arr = (HybridLayer * len(layers))()
+        for i, spec in enumerate(layers):
+            spec = dict(spec)
+            spec["mixer"] = MIXER[spec["mixer"]]
+            spec["mlp_kind"] = MLP_KIND[spec.get("mlp_kind", "none")]
+            for k, v in spec.items():
+                setattr(arr[i], k, v)
+        self = cls.__new__(cls)
+        self._h = C.c_void_p()
+        # the fields the other methods read
+        self.cfg = DecoderConfig(arch=ARCH["bezadra"], dtype=c.dtype, vocab_size=vocab_size, hidden_size=width,
+                                 num_hidden_layers=len(layers), max_batch=max_batch, max_context=max_context)
+        self.dtype, self.dev = dtype, dev
+        call("rai_hip_init", dev)
+        call("rai_hip_decoder_create_hybrid", dev, C.byref(c), arr, C.byref(self._h))
         return self
 
     def close(self):
