@@ -1208,6 +1208,7 @@ __global__ void __launch_bounds__(NW * KSP * 64) k_flash_prefill_bf16(AttnArgs a
 #pragma unroll
         for (int r = 0; r < 16; ++r) o[dt][r] += mb[j * MS + 2 + dt * 16 + r] * wj;
     }
+    m_run = ms;
   }
   float l_tot = l_run + __shfl_xor(l_run, 32, 64);
   if constexpr (MODE == 2) {
