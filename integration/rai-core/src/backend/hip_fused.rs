@@ -108,6 +108,15 @@ impl Decoder {
         Self { h, vocab: cfg.vocab_size as usize }
     }
 
+    /// A model of attention and gated delta rule layers (Bezadra), described one by one.
+    pub fn create_hybrid(dev: c_int, cfg: &RaiHipHybridConfig, layers: &[RaiHipHybridLayer]) -> Self {
+        assert_eq!(layers.len(), cfg.num_layers as usize);
+        let mut h = std::ptr::null_mut();
+        check(unsafe { rai_hip_init(dev) });
+        check(unsafe { rai_hip_decoder_create_hybrid(dev, cfg, layers.as_ptr(), &mut h) });
+        Self { h, vocab: cfg.vocab_size as usize }
+    }
+
     /// `(name, element count)` of every parameter the driver expects.
     pub fn param_names(&self) -> Vec<(String, i64)> {
         let mut n = 0i32;
