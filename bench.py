@@ -261,17 +261,49 @@ def lelitar_case(size, kind, max_batch, max_context):
                      key_bytes=2 * z["kv_rank"], layers=n)
 
 
-def run_lelitar(args):
-    """Prefill and decode of the Lelitar design beside the closest family of equal size; one line per case."""
+# Bezadra beside the same Qwen2 layers: attention layers (as many key heads as heads, like Qwen2 here),
+# delta rule layers of as many heads of 128 x 128, and both in the ratio of one to three with the delta run looped twice.
+BEZADRA_RANK = 128
+
+
+def bezadra_case(size, kind, max_batch, max_context):
+    """A decoder of one size: kind 'attention', 'delta', 'mixed' or 'qwen2'."""
+    from rai_amd.models import Decoder
+    if kind == "qwen2":
+        return lelitar_case(size, kind, max_batch, max_context)
+    z, hd = LELITAR_SIZES[size], 128
+    w, heads, n = z["width"], z["heads"], z["layers"]
+    qd = heads * hd
+    mlp = dict(mlp_kind="dense", intermediate=z["ff"], mlp_limit=7.0, mlp_alpha=1.702)
+    attn = dict(mixer="attention", heads=heads, kv_heads=heads, qk_dim=hd, v_dim=hd, rot_dims=hd, rot_base=5e5, rot_factor=8.0, rot_low=1.0,
+                rot_high=4.0, rot_original=8192, attn_scale=hd ** -0.5, softcap=30.0, **mlp)
+    delta = dict(mixer="channel_delta", heads=heads, kv_heads=heads, qk_dim=hd, v_dim=hd, conv_taps=4, decay_rank=BEZADRA_RANK,
+                 gate_rank=BEZADRA_RANK, **mlp)
+    lin_a, lin_d = 5 * w * qd + 3 * w * z["ff"], 4 * w * qd + 2 * BEZADRA_RANK * (w + qd) + w * heads + 3 * w * z["ff"]
+    state = 2 * 4 * heads * hd * hd        # read and written once per token and layer
+    layers, loop, runs = {"attention": ([attn] * n, None, (n, 0)), "delta": ([delta] * n, None, (0, n)),
+                          "mixed": ([attn] + [delta] * 3, (1, 4, 2), (1, 6))}[kind]
+    dec = Decoder.hybrid("bf16", vocab_size=LELITAR_VOCAB, width=w, layers=layers, norm_eps=1e-6, embed_scale=1.0, logit_scale=1.0, loop=loop,
+                         max_batch=max_batch, max_context=max_context)
+    entry = 3 * w * w if loop else 0       # W0 once, Wx per pass
+    total = runs[0] + runs[1]
+    share = runs[0] / total                # the share of runs that read keys
+    lin = (runs[0] * lin_a + runs[1] * lin_d + entry) / total
+    return dec, dict(lin=lin, weights=lin, keys=lambda t: t, key_flops=4 * qd * share, key_bytes=4 * qd * share, layers=total,
+                     state_flops=7 * heads * hd * hd * (1 - share), state_bytes=state * (1 - share))
+
+
+def run_layer_cases(args, kinds, case, what):
+    """Prefill and decode of one family's layers beside the closest family of equal size; one line per case."""
     from rai_amd import synthetic
     B, CTX, NEWT = 32, 1024, 33
-    sizes = args.lelitar_sizes.split(",") if args.lelitar_sizes else list(LELITAR_SIZES)
+    sizes = args.layer_sizes.split(",") if args.layer_sizes else list(LELITAR_SIZES)
     table = {}
     for size in sizes:
-        for kind in ("qwen2", "dense", "moe"):
-            if args.lelitar_kinds and kind not in args.lelitar_kinds.split(","):
+        for kind in kinds:
+            if args.layer_kinds and kind not in args.layer_kinds.split(","):
                 continue
-            dec, c = lelitar_case(size, kind, B, CTX + NEWT)
+            dec, c = case(size, kind, B, CTX + NEWT)
             synthetic.load_tiled_params(dec)
             w = LELITAR_SIZES[size]["width"]
             head = LELITAR_VOCAB * w
@@ -286,18 +318,26 @@ def run_lelitar(args):
                         dcd.append(d / (NEWT - 1))
                 p, d = float(np.mean(pre)) / 1e3, float(np.mean(dcd)) / 1e3
                 seen = sum(c["keys"](t) for t in range(1, CTX + 1)) / CTX
-                flops = 2.0 * batch * CTX * c["layers"] * c["lin"] + batch * CTX * c["layers"] * seen * c["key_flops"] + 2.0 * batch * head
+                flops = 2.0 * batch * CTX * c["layers"] * c["lin"] + batch * CTX * c["layers"] * (seen * c["key_flops"] + c.get("state_flops", 0)) + 2.0 * batch * head
                 wb = c["weights"](batch) if callable(c["weights"]) else c["weights"]
-                byts = 2.0 * (c["layers"] * wb + head) + c["layers"] * batch * c["keys"](CTX + NEWT / 2) * c["key_bytes"]
+                byts = 2.0 * (c["layers"] * wb + head) + c["layers"] * batch * (c["keys"](CTX + NEWT / 2) * c["key_bytes"] + c.get("state_bytes", 0))
                 row[f"prefill_b{batch}"] = dict(tokens_per_s=round(batch * CTX / p), ms=round(p * 1e3, 3), tflops=round(flops / p / 1e12, 1))
                 row[f"decode_b{batch}"] = dict(tokens_per_s=round(batch / d, 1), us=round(d * 1e6, 1), gb_per_s=round(byts / d / 1e9))
             table[f"{size} {kind}"] = row
             print(json.dumps({"case": f"{size} {kind}", **row}), file=sys.stderr, flush=True)
             dec.close()
     first = next(iter(table.values()))
-    _line("Lelitar layers beside Qwen2 layers of equal size, prefill tok/s of the first case", first[f"prefill_b{B}"]["tokens_per_s"], "tokens/s",
+    _line(f"{what[0]} layers beside Qwen2 layers of equal size, prefill tok/s of the first case", first[f"prefill_b{B}"]["tokens_per_s"], "tokens/s",
           args.steps, args.warmup, first[f"prefill_b{B}"]["ms"],
-          f"latent-attention decoders of {sizes} wide layers, bf16, prompts of {CTX}, batch 1 and {B}, random weights", {"cases": table})
+          f"{what[1]} decoders of {sizes} wide layers, bf16, prompts of {CTX}, batch 1 and {B}, random weights", {"cases": table})
+
+
+def run_lelitar(args):
+    run_layer_cases(args, ("qwen2", "dense", "moe"), lelitar_case, ("Lelitar", "latent-attention"))
+
+
+def run_bezadra(args):
+    run_layer_cases(args, ("qwen2", "attention", "delta", "mixed"), bezadra_case, ("Bezadra", "attention and delta rule"))
 
 
 def run_ops(args):
@@ -581,10 +621,11 @@ def main():
                     help="tokens decoded through the lazy-graph path for the graph_decode_* fields (0: skip)")
     ap.add_argument("--cold", action="store_true",
                     help="gemm-tiles: rotate over weight copies so every launch reads its weight from HBM, as in a model")
-    ap.add_argument("--workload", default="phi2-decode", choices=["phi2-decode", "qwen2-prefill", "gemma-decode", "lelitar", "ops", "gemm-tiles", "peaks"],
+    ap.add_argument("--workload", default="phi2-decode", choices=["phi2-decode", "qwen2-prefill", "gemma-decode", "lelitar", "bezadra", "ops", "gemm-tiles", "peaks"],
                     help="phi2-decode is the headline line; the others are the remaining configurations of the path")
-    ap.add_argument("--lelitar-sizes", default="", help="lelitar: comma-separated widths (default: all)")
-    ap.add_argument("--lelitar-kinds", default="", help="lelitar: comma-separated subset of qwen2,dense,moe (default: all)")
+    ap.add_argument("--layer-sizes", "--lelitar-sizes", default="", help="lelitar, bezadra: comma-separated widths (default: all)")
+    ap.add_argument("--layer-kinds", "--lelitar-kinds", default="",
+                    help="lelitar: comma-separated subset of qwen2,dense,moe; bezadra: of qwen2,attention,delta,mixed (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build measures one GPU; --gpus must be 1 (multi-GPU sharding is a design note only)")
@@ -594,6 +635,8 @@ def main():
         return run_gemma_decode(args)
     if args.workload == "lelitar":
         return run_lelitar(args)
+    if args.workload == "bezadra":
+        return run_bezadra(args)
     if args.workload == "ops":
         return run_ops(args)
     if args.workload == "gemm-tiles":
