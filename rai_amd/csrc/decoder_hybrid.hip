@@ -18,6 +18,7 @@
 namespace rai {
 
 static int pad32(int n) { return (n + 31) / 32 * 32; }
+static int pad_key(int n) { return n > 32 && n <= 64 ? 64 : n > 64 && n <= 128 ? 128 : n > 128 && n <= 256 ? 256 : pad32(n); }   // what the chunked form serves
 
 // Tables are shared by the layers that turn alike.
 static int rotary_for(rai_hip_decoder *d, const RotaryParams &r, const float **cos_t, const float **sin_t) {
@@ -106,7 +107,7 @@ static int create_layer(rai_hip_decoder *d, int l, const rai_hip_hybrid_layer &c
   } else {
     DeltaShape &z = y.delta;
     z.heads = c.heads; z.kv_heads = c.kv_heads; z.dim = c.qk_dim; z.vdim = c.v_dim; z.taps = c.conv_taps;
-    z.Dk = pad32(c.qk_dim); z.Vp = pad32(c.v_dim);
+    z.Dk = pad_key(c.qk_dim); z.Vp = pad32(c.v_dim);
     y.a_rank = pad64(c.decay_rank); y.g_rank = pad64(c.gate_rank);
     z.channels = 2 * z.kv_heads * z.Dk + z.heads * z.Vp;
     z.off_b = pad64(z.channels);
@@ -186,7 +187,7 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
   // activations, sized for the widest layer
   const int64_t rows = d->max_rows;
   int ldn = 0, KB = 0;
-  size_t decay = 0, qk = 0, val = 0, beta = 0, ws = 0, counters = 0;
+  size_t decay = 0, qk = 0, val = 0, beta = 0, ws = 0, counters = 0, chunk = 0;
   for (const HybridLayer &y : hm.layers) {
     ldn = std::max(ldn, y.ldn);
     KB = std::max(KB, y.QD + y.Fp);
@@ -198,6 +199,7 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
       decay = std::max(decay, (size_t)z.heads * z.Dk);
       qk = std::max(qk, (size_t)z.kv_heads * z.Dk);
       val = std::max(val, (size_t)z.heads * z.Vp);
+      if (delta_chunk_serves(cfg.dtype, z)) chunk = std::max(chunk, delta_chunk_ws_bytes(z, cfg.max_batch, rows));
       beta = std::max(beta, (size_t)z.heads);
     }
   }
@@ -221,7 +223,8 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
     RAI_TRY(floats(decay, &hm.decay));
     RAI_TRY(floats(qk, &hm.q));
     RAI_TRY(floats(qk, &hm.k));
-    RAI_TRY(floats(val, &hm.v));
+    RAI_TRY(zalloc(d, rows * val * es, &hm.v));
+    if (chunk) RAI_TRY(zalloc(d, chunk, &hm.chunk_ws));
     RAI_TRY(floats(beta, &hm.beta));
     RAI_TRY(floats(val, &hm.o));
     RAI_TRY(zalloc(d, rows * val * es, &hm.gate));
@@ -357,6 +360,7 @@ static DeltaArgs delta_args(rai_hip_decoder *d, const HybridLayer &y, const Hybr
   a.decay = hm.decay; a.q = hm.q; a.k = hm.k; a.v = hm.v; a.beta = hm.beta; a.o = hm.o;
   a.norm_w = y.norm_w; a.eps = (float)hm.c.norm_eps;
   a.gate = hm.gate;
+  a.chunk_ws = hm.chunk_ws;
   a.out = hm.cat; a.ldo = y.QD + y.Fp;
   return a;
 }

@@ -28,8 +28,10 @@ struct DeltaArgs {
   void *ring;                  // [B][taps][channels]: the inputs of the last `taps` positions, position p at p mod taps
   float *carried;              // [B][heads][Dk][Vp]
   const void *A_log, *dt_bias; // [heads], [heads Dk]
-  float *decay;                // [rows, heads Dk]: in: the low-rank factor's output; after the preparation log g
-  float *q, *k, *v, *beta;     // [rows, kv_heads Dk] twice, [rows, heads Vp], [rows, heads]
+  float *decay;                // [rows, heads Dk]: in: the low-rank factor's output; after the preparation log g, or its
+                               // running sum from the start of each chunk of kDeltaChunk tokens of this call
+  float *q, *k, *beta;         // [rows, kv_heads Dk] twice, [rows, heads]
+  void *v;                     // [rows, heads Vp] of the model dtype
   float *o;                    // [rows, heads Vp]
   const void *norm_w;          // [Vp]
   float eps;
@@ -40,7 +42,14 @@ struct DeltaArgs {
   // gate were computed before
   const void *a2, *g2;         // [heads Dk, a_rank], [heads Vp, g_rank]
   int a_rank, g_rank;
+  char *chunk_ws;              // delta_chunk_ws_bytes(); null: the chunked form is not used
+  int chunked;                 // filled in by the launcher
 };
+// The chunked form (bf16 models): see delta_chunk.hip.
+constexpr int kDeltaChunk = 64;
+bool delta_chunk_serves(int dtype, const DeltaShape &s);
+size_t delta_chunk_ws_bytes(const DeltaShape &s, int64_t max_batch, int64_t max_rows);
+int launch_delta_chunks(hipStream_t st, const DeltaArgs &a);   // the recurrence only, after the preparation
 // Any number of tokens: preparation (convolutions, unit vectors, decays), recurrence, norm and gate.
 int launch_delta_tokens(hipStream_t st, int dtype, const DeltaArgs &a);
 // One token per sequence in one launch, where it serves the head sizes.

@@ -1,17 +1,16 @@
 // Gated delta rule with a decay per key channel (see delta.h).
-//   k_delta_prep  convolution + silu, unit vectors, decays and step sizes of every token
+//   k_delta_prep  convolution + silu, unit vectors of every token
+//   k_delta_decay decays and step sizes
 //   k_delta_scan  the recurrence, token after token: a block owns 16 columns of one head's state, 16 lanes to a column
+//                 (f32 models, few tokens, head sizes the chunked form of delta_chunk.hip does not serve)
 //   k_delta_out   norm over the head's values, weight and output gate
 //   k_delta_step  all of it for one token per sequence: a block owns a head, its state goes through registers once
 #include <cstdlib>
 
 #include "delta.h"
+#include "delta_device.h"
 
 namespace rai {
-
-__device__ __forceinline__ float dl_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float dl_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-template <typename T> __device__ __forceinline__ float ld(const void *p, int64_t i) { return (float)Scalar<T>::load((const T *)p + i); }
 
 // Sum over the 16 lanes of a row, in every lane.
 __device__ __forceinline__ float row16_sum(float v) {
@@ -40,73 +39,131 @@ __device__ __forceinline__ float conv_silu(const DeltaArgs &a, int b, int s, int
 }
 
 constexpr int kPrepTokens = 8;
-// A wave takes one unit (a q or k head, a v head, or a head's decays) over kPrepTokens tokens.
-template <typename T, int NI>
+constexpr int kChunkedFrom = 24;   // tokens of a call from which on the chunked form is the faster one
+template <typename T> struct alignas(2 * sizeof(T)) Pair { T v[2]; };
+template <typename T> __device__ __forceinline__ float2 ld2(const void *p, int64_t i) {
+  const Pair<T> x = *reinterpret_cast<const Pair<T> *>((const T *)p + i);
+  return make_float2((float)Scalar<T>::load(&x.v[0]), (float)Scalar<T>::load(&x.v[1]));
+}
+
+// Channels c, c + 1 (c even) of kPrepTokens tokens from s0 on, after convolution and silu; TAPS == 0: any number of taps.
+template <typename T, int TAPS>
+__device__ __forceinline__ void conv_run(const DeltaArgs &a, int b, int s0, int pos0, int c, float2 (&y)[kPrepTokens]) {
+  const DeltaShape &z = a.s;
+  if constexpr (TAPS > 0) {
+    float2 x[kPrepTokens + TAPS - 1], w[TAPS];
+#pragma unroll
+    for (int i = 0; i < kPrepTokens + TAPS - 1; ++i) {
+      const int t = s0 - (TAPS - 1) + i;   // token of this call, or an earlier one in the ring
+      x[i] = make_float2(0.f, 0.f);
+      if (t >= 0 && t < a.S) x[i] = ld2<T>(a.dn, ((int64_t)b * a.S + t) * z.ldn + c);
+      else if (t < 0 && pos0 + t >= 0) x[i] = ld2<T>(a.ring, ((int64_t)b * TAPS + (pos0 + t) % TAPS) * z.channels + c);
+    }
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = make_float2(ld<T>(a.conv, (int64_t)c * TAPS + j), ld<T>(a.conv, (int64_t)(c + 1) * TAPS + j));
+#pragma unroll
+    for (int i = 0; i < kPrepTokens; ++i) {
+      float2 v = make_float2(0.f, 0.f);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        v.x = fmaf(x[i + j].x, w[j].x, v.x);
+        v.y = fmaf(x[i + j].y, w[j].y, v.y);
+      }
+      y[i] = make_float2(v.x * dl_sigmoid(v.x), v.y * dl_sigmoid(v.y));
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < kPrepTokens; ++i)
+      y[i] = s0 + i < a.S ? make_float2(conv_silu<T>(a, b, s0 + i, pos0, c), conv_silu<T>(a, b, s0 + i, pos0, c + 1)) : make_float2(0.f, 0.f);
+  }
+}
+
+// A wave takes one q, k or v head over kPrepTokens tokens; lane l holds channels 2 l + 128 i and the next.
+template <typename T, int NI, int TAPS>
 __global__ void __launch_bounds__(256) k_delta_prep(DeltaArgs a) {
   const DeltaShape &z = a.s;
-  const int lane = threadIdx.x & 63, units = 2 * z.kv_heads + 2 * z.heads;
+  const int lane = threadIdx.x & 63, units = 2 * z.kv_heads + z.heads;
   const int64_t job = blockIdx.x * 4ll + (threadIdx.x >> 6);
   const int groups = (a.S + kPrepTokens - 1) / kPrepTokens;
   const int unit = (int)(job % units);
   const int64_t grp = job / units;
   if (grp >= (int64_t)a.B * groups) return;
-  const int b = (int)(grp / groups), s0 = (int)(grp % groups) * kPrepTokens, s1 = s0 + kPrepTokens < a.S ? s0 + kPrepTokens : a.S;
+  const int b = (int)(grp / groups), s0 = (int)(grp % groups) * kPrepTokens;
   const int pos0 = a.state->pos;
-  if (unit < 2 * z.kv_heads) {
-    const bool query = unit < z.kv_heads;
-    float *dst = (query ? a.q : a.k) + (query ? unit : unit - z.kv_heads) * z.Dk;
-    const float mul = query ? 1.0f / sqrtf((float)z.dim) : 1.0f;
-    for (int s = s0; s < s1; ++s) {
-      float y[NI], sum = 0.f;
+  const int64_t row0 = (int64_t)b * a.S + s0;
+  const bool qk = unit < 2 * z.kv_heads, query = unit < z.kv_heads;
+  const int width = qk ? z.Dk : z.Vp, h = qk ? (query ? unit : unit - z.kv_heads) : unit - 2 * z.kv_heads;
+  const int first = qk ? unit * z.Dk : 2 * z.kv_heads * z.Dk + h * z.Vp;
+  float2 y[NI][kPrepTokens];
 #pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        const int c = lane + 64 * i;
-        y[i] = c < z.Dk ? conv_silu<T>(a, b, s, pos0, unit * z.Dk + c) : 0.f;
-        sum = fmaf(y[i], y[i], sum);
-      }
-      const float r = mul / sqrtf(wave_sum(sum) + 1e-6f);
+  for (int i = 0; i < NI; ++i) {
+    const int c = 2 * lane + 128 * i;
+    if (c < width) conv_run<T, TAPS>(a, b, s0, pos0, first + c, y[i]);
+    else {
 #pragma unroll
-      for (int i = 0; i < NI; ++i)
-        if (lane + 64 * i < z.Dk) dst[((int64_t)b * a.S + s) * z.kv_heads * z.Dk + lane + 64 * i] = y[i] * r;
+      for (int t = 0; t < kPrepTokens; ++t) y[i][t] = make_float2(0.f, 0.f);
     }
-  } else if (unit < 2 * z.kv_heads + z.heads) {
-    const int h = unit - 2 * z.kv_heads;
-    for (int s = s0; s < s1; ++s)
+  }
+  if (!qk) {
+#pragma unroll
+    for (int t = 0; t < kPrepTokens; ++t)
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
-        const int c = lane + 64 * i;
-        if (c < z.Vp) a.v[(((int64_t)b * a.S + s) * z.heads + h) * z.Vp + c] = conv_silu<T>(a, b, s, pos0, 2 * z.kv_heads * z.Dk + h * z.Vp + c);
-      }
-  } else {
-    const int h = unit - 2 * z.kv_heads - z.heads;
-    const float rate = -expf(ld<T>(a.A_log, h));
-    for (int s = s0; s < s1; ++s) {
-      const int64_t row = (int64_t)b * a.S + s;
-#pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        const int c = lane + 64 * i;
-        if (c < z.Dk) {
-          float *p = a.decay + (row * z.heads + h) * z.Dk + c;
-          *p = rate * dl_softplus(*p + ld<T>(a.dt_bias, h * z.Dk + c));
+        const int c = 2 * lane + 128 * i;
+        if (s0 + t < a.S && c < width) {
+          Pair<T> o;
+          Scalar<T>::store(&o.v[0], y[i][t].x);
+          Scalar<T>::store(&o.v[1], y[i][t].y);
+          *reinterpret_cast<Pair<T> *>((T *)a.v + ((row0 + t) * z.heads + h) * z.Vp + c) = o;
         }
       }
-      if (lane == 0) a.beta[row * z.heads + h] = dl_sigmoid(ld<T>(a.dn, row * z.ldn + z.off_b + h));
+    return;
+  }
+  float sum[kPrepTokens];
+#pragma unroll
+  for (int t = 0; t < kPrepTokens; ++t) {
+    sum[t] = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) sum[t] = fmaf(y[i][t].x, y[i][t].x, fmaf(y[i][t].y, y[i][t].y, sum[t]));
+  }
+#pragma unroll
+  for (int t = 0; t < kPrepTokens; ++t) sum[t] = wave_sum(sum[t]);
+  float *dst = (query ? a.q : a.k) + h * z.Dk;
+  const float mul = query ? 1.0f / sqrtf((float)z.dim) : 1.0f;
+#pragma unroll
+  for (int t = 0; t < kPrepTokens; ++t) {
+    const float r = mul / sqrtf(sum[t] + 1e-6f);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int c = 2 * lane + 128 * i;
+      if (s0 + t < a.S && c < width) *reinterpret_cast<float2 *>(dst + (row0 + t) * z.kv_heads * z.Dk + c) = make_float2(y[i][t].x * r, y[i][t].y * r);
     }
   }
 }
 
-// The inputs of the last `taps` tokens of this call go to their places in the ring: the v channels of head h, and with
-// the first head of a group the group's q and k channels.
+// A thread takes one channel of one head over a chunk of tokens; channel 0's also forms the step sizes.
 template <typename T>
-__device__ __forceinline__ void update_ring(const DeltaArgs &a, int b, int h, int pos0, int tid, int nt) {
+__global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   const DeltaShape &z = a.s;
-  const int rep = z.heads / z.kv_heads, kd = z.kv_heads * z.Dk;
-  const int nqk = h % rep == 0 ? 2 * z.Dk : 0, n = nqk + z.Vp;
-  for (int i = tid; i < n; i += nt) {
-    const int c = i < nqk ? (i < z.Dk ? (h / rep) * z.Dk + i : kd + (h / rep) * z.Dk + i - z.Dk) : 2 * kd + h * z.Vp + i - nqk;
-    for (int s = a.S > z.taps ? a.S - z.taps : 0; s < a.S; ++s)
-      ((T *)a.ring)[((int64_t)b * z.taps + (pos0 + s) % z.taps) * z.channels + c] = ((const T *)a.dn)[((int64_t)b * a.S + s) * z.ldn + c];
+  const int c = blockIdx.x * 256 + threadIdx.x, b = blockIdx.z, s0 = blockIdx.y * kDeltaChunk;
+  if (c >= z.heads * z.Dk) return;
+  const int h = c / z.Dk, s1 = s0 + kDeltaChunk < a.S ? s0 + kDeltaChunk : a.S;
+  const float rate = -expf(ld<T>(a.A_log, h)), bias = ld<T>(a.dt_bias, c);
+  float run = 0.f;
+  for (int s = s0; s < s1; s += 8) {
+    float x[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = s + j < s1 ? a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] : 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (s + j < s1) {
+        const float g = rate * dl_softplus(x[j] + bias);
+        run = a.chunked ? run + g : g;
+        a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] = run;
+      }
   }
+  if (c % z.Dk == 0)
+    for (int s = s0; s < s1; ++s) a.beta[((int64_t)b * a.S + s) * z.heads + h] = dl_sigmoid(ld<T>(a.dn, ((int64_t)b * a.S + s) * z.ldn + z.off_b + h));
 }
 
 // RPL state rows per lane (16 RPL >= Dk); rows past Dk stay zero.
@@ -139,7 +196,7 @@ __global__ void __launch_bounds__(256) k_delta_scan(DeltaArgs a) {
       ks[e] = in ? a.k[((row0 + t) * z.kv_heads + kv) * z.Dk + r] : 0.f;
       gs[e] = in ? expf(a.decay[((row0 + t) * z.heads + h) * z.Dk + r]) : 0.f;
     }
-    if (tid < n * 16) vs[tid] = a.v[((row0 + (tid >> 4)) * z.heads + h) * z.Vp + blockIdx.x * 16 + (tid & 15)];
+    if (tid < n * 16) vs[tid] = ld<T>(a.v, ((row0 + (tid >> 4)) * z.heads + h) * z.Vp + blockIdx.x * 16 + (tid & 15));
     if (tid < n) bs[tid] = a.beta[(row0 + tid) * z.heads + h];
     __syncthreads();
     for (int t = 0; t < n; ++t) {
@@ -337,19 +394,31 @@ template <typename T, int RPL> static int launch_scan(hipStream_t st, const Delt
   return launch_check("delta_scan");
 }
 
-template <typename T> static int launch_tokens_t(hipStream_t st, const DeltaArgs &a) {
+template <typename T, int NI> static int launch_prep(hipStream_t st, const DeltaArgs &a) {
+  const DeltaShape &z = a.s;
+  const int64_t jobs = (int64_t)a.B * ((a.S + kPrepTokens - 1) / kPrepTokens) * (2 * z.kv_heads + z.heads);
+  RAI_REQUIRE((jobs + 3) / 4 < (1ll << 31), RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
+  const dim3 grid((unsigned)((jobs + 3) / 4)), block(256);
+  if (z.taps == 4) hipLaunchKernelGGL((k_delta_prep<T, NI, 4>), grid, block, 0, st, a);
+  else hipLaunchKernelGGL((k_delta_prep<T, NI, 0>), grid, block, 0, st, a);
+  return launch_check("delta_prep");
+}
+
+template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, DeltaArgs a) {
   const DeltaShape &z = a.s;
   const int wide = z.Dk > z.Vp ? z.Dk : z.Vp;
-  const int64_t jobs = (int64_t)a.B * ((a.S + kPrepTokens - 1) / kPrepTokens) * (2 * z.kv_heads + 2 * z.heads);
+  const char *off = getenv("RAI_HIP_NO_DELTA_CHUNK");   // read per call: the tests compare both forms in one process
+  a.chunked = a.chunk_ws && a.S >= kChunkedFrom && delta_chunk_serves(dtype, z) && !(off && *off && *off != '0');
   const int64_t outs = (int64_t)a.B * a.S * z.heads;
-  RAI_REQUIRE((jobs + 3) / 4 < (1ll << 31) && (outs + 3) / 4 < (1ll << 31), RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
-  const dim3 gp((unsigned)((jobs + 3) / 4)), go((unsigned)((outs + 3) / 4)), block(256);
-  if (wide <= 64) hipLaunchKernelGGL((k_delta_prep<T, 1>), gp, block, 0, st, a);
-  else if (wide <= 128) hipLaunchKernelGGL((k_delta_prep<T, 2>), gp, block, 0, st, a);
-  else if (wide <= 256) hipLaunchKernelGGL((k_delta_prep<T, 4>), gp, block, 0, st, a);
-  else hipLaunchKernelGGL((k_delta_prep<T, 8>), gp, block, 0, st, a);
-  RAI_TRY(launch_check("delta_prep"));
-  if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
+  RAI_REQUIRE((outs + 3) / 4 < (1ll << 31) && (a.S + kDeltaChunk - 1) / kDeltaChunk <= 65535, RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
+  const dim3 go((unsigned)((outs + 3) / 4)), block(256);
+  if (wide <= 128) RAI_TRY((launch_prep<T, 1>(st, a)));
+  else if (wide <= 256) RAI_TRY((launch_prep<T, 2>(st, a)));
+  else RAI_TRY((launch_prep<T, 4>(st, a)));
+  hipLaunchKernelGGL(k_delta_decay<T>, dim3((z.heads * z.Dk + 255) / 256, (a.S + kDeltaChunk - 1) / kDeltaChunk, a.B), block, 0, st, a);
+  RAI_TRY(launch_check("delta_decay"));
+  if (a.chunked) RAI_TRY(launch_delta_chunks(st, a));
+  else if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
   else if (z.Dk <= 64) RAI_TRY((launch_scan<T, 4>(st, a)));
   else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));
   else if (z.Dk <= 256) RAI_TRY((launch_scan<T, 16>(st, a)));
@@ -363,7 +432,7 @@ template <typename T> static int launch_tokens_t(hipStream_t st, const DeltaArgs
 
 int launch_delta_tokens(hipStream_t st, int dtype, const DeltaArgs &a) {
   RAI_TRY(check_delta(a));
-  return dtype == RAI_BF16 ? launch_tokens_t<bf16_raw>(st, a) : launch_tokens_t<float>(st, a);
+  return dtype == RAI_BF16 ? launch_tokens_t<bf16_raw>(st, dtype, a) : launch_tokens_t<float>(st, dtype, a);
 }
 
 static int step_rows(const DeltaShape &z) {   // state rows per thread

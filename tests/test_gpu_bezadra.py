@@ -231,10 +231,11 @@ def test_long_memory(hip, dt, far):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("bias,rate", [(-12.0, 0.0), (-3.0, 1.5), (4.0, 0.0), (30.0, 3.0), (-60.0, -4.0)])
-def test_decays_from_none_to_all(hip, dt, bias, rate):
+@pytest.mark.parametrize("dim", [32, 64])
+@pytest.mark.parametrize("bias,rate", [(0.5, 1.0), (-12.0, 0.0), (-3.0, 1.5), (4.0, 0.0), (30.0, 3.0), (-60.0, -4.0)])
+def test_decays_from_none_to_all(hip, dt, bias, rate, dim):
     """Channels that forget nothing, that forget everything at once (the decay underflows), and both next to each other."""
-    cfg = bm.config([bm.delta(heads=4, kv_heads=2, dim=32, vdim=32, conv=4, ff=None)])
+    cfg = bm.config([bm.delta(heads=4, kv_heads=2, dim=dim, vdim=32, conv=4, ff=None)])
     p = bezadra.random_params(cfg, "f32", 16)
     p["l0.mix.dt_bias"][::2] = bias
     p["l0.mix.A_log"][:] = rate
@@ -277,7 +278,7 @@ def test_long_prompt(hip, dt):
     dec.close()
 
 
-@pytest.mark.parametrize("switch", ["RAI_HIP_NO_LATENT_FUSED", "RAI_HIP_NO_MFMA_DECODE", "RAI_HIP_FLASH_NO_KEY_SPLIT"])
+@pytest.mark.parametrize("switch", ["RAI_HIP_NO_LATENT_FUSED", "RAI_HIP_NO_MFMA_DECODE", "RAI_HIP_FLASH_NO_KEY_SPLIT", "RAI_HIP_NO_DELTA_CHUNK"])
 def test_the_plain_forms_of_the_bf16_kernels(hip, monkeypatch, switch):
     cfg = bm.config(bm.mixed_config()["layers"] + [bm.attention(heads=8, kv_heads=2, dim=64, vdim=64, dims=32)], loop=(1, 3, 2))
     p = bezadra.random_params(cfg, "bf16", 23)
