@@ -141,7 +141,73 @@ __global__ void __launch_bounds__(256) k_delta_prep(DeltaArgs a) {
   }
 }
 
-// A thread takes one channel of one head over a chunk of tokens; channel 0's also forms the step sizes.
+// Sum over the `lanes` (a power of two) lanes that share a head.
+__device__ __forceinline__ float group_sum(float v, int lanes) {
+  if (lanes == 16) return row16_sum(v);
+  for (int o = lanes >> 1; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+__device__ __forceinline__ float fast_silu(float y) { return y * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * y)); }
+
+// The bf16 form for four taps and key heads of 32, 64, 128, 256 or 512 channels: a thread takes eight channels over
+// kWideTokens tokens, Dk / 8 neighbouring lanes a head.
+constexpr int kWideTokens = 4;
+__global__ void __launch_bounds__(256) k_delta_prep_wide(DeltaArgs a) {
+  struct alignas(16) P8 { uint16_t v[8]; };
+  const DeltaShape &z = a.s;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8, b = blockIdx.z, s0 = blockIdx.y * kWideTokens;
+  const int kd = z.kv_heads * z.Dk;
+  if (c >= z.channels) return;   // whole heads: channels is a multiple of 32, the q and k channels of 2 Dk
+  const int pos0 = a.state->pos;
+  P8 x[kWideTokens + 3], w[4];
+#pragma unroll
+  for (int i = 0; i < kWideTokens + 3; ++i) {
+    const int t = s0 - 3 + i;   // token of this call, or an earlier one in the ring
+    memset(&x[i], 0, sizeof(P8));
+    if (t >= 0 && t < a.S) x[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.dn + ((int64_t)b * a.S + t) * z.ldn + c);
+    else if (t < 0 && pos0 + t >= 0) x[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.ring + ((int64_t)b * 4 + (pos0 + t) % 4) * z.channels + c);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) w[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.conv + (int64_t)c * 4 + 8 * i);
+  const bool qk = c < 2 * kd;
+  const float mul = c < kd ? 1.0f / sqrtf((float)z.dim) : 1.0f;
+#pragma unroll
+  for (int t = 0; t < kWideTokens; ++t) {
+    float y[8], sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float v = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v = fmaf(bf16_bits_to_f32(x[t + j].v[e]), bf16_bits_to_f32(w[e >> 1].v[4 * (e & 1) + j]), v);
+      y[e] = fast_silu(v);
+      sum = fmaf(y[e], y[e], sum);
+    }
+    const int64_t row = (int64_t)b * a.S + s0 + t;
+    if (qk) {
+      const float r = mul / sqrtf(group_sum(sum, z.Dk / 8) + 1e-6f);
+      if (s0 + t < a.S) {
+        float4 *dst = reinterpret_cast<float4 *>((c < kd ? a.q + c : a.k + c - kd) + row * kd);
+        dst[0] = make_float4(y[0] * r, y[1] * r, y[2] * r, y[3] * r);
+        dst[1] = make_float4(y[4] * r, y[5] * r, y[6] * r, y[7] * r);
+      }
+    } else if (s0 + t < a.S) {
+      *reinterpret_cast<uint4 *>((uint16_t *)a.v + row * z.heads * z.Vp + c - 2 * kd) =
+          make_uint4(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]), pack_bf16x2(y[4], y[5]), pack_bf16x2(y[6], y[7]));
+    }
+  }
+}
+
+// log(1 + exp(z)); for results that meet bf16 operands through the hardware's exp2 and log2 and a short series where the
+// logarithm's argument is close to 1 (relative error below 1e-6).
+template <typename T> __device__ __forceinline__ float softplus_for(float z) {
+  if constexpr (sizeof(T) == 4) return dl_softplus(z);
+  const float x = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z));
+  const float series = x * (1.f - x * (0.5f - x * (0.33333333f - x * (0.25f - x * 0.2f))));
+  return fmaxf(z, 0.f) + (x < 0.06f ? series : 0.69314718056f * __builtin_amdgcn_logf(1.f + x));
+}
+
+// A thread takes one channel of one head over a chunk of tokens; the head's first threads also form the step sizes.
+constexpr int kDecayRun = 16;
 template <typename T>
 __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   const DeltaShape &z = a.s;
@@ -150,20 +216,19 @@ __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   const int h = c / z.Dk, s1 = s0 + kDeltaChunk < a.S ? s0 + kDeltaChunk : a.S;
   const float rate = -expf(ld<T>(a.A_log, h)), bias = ld<T>(a.dt_bias, c);
   float run = 0.f;
-  for (int s = s0; s < s1; s += 8) {
-    float x[8];
+  for (int s = s0; s < s1; s += kDecayRun) {
+    float x[kDecayRun];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) x[j] = s + j < s1 ? a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] : 0.f;
+    for (int j = 0; j < kDecayRun; ++j) x[j] = s + j < s1 ? a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] : 0.f;
 #pragma unroll
-    for (int j = 0; j < 8; ++j)
+    for (int j = 0; j < kDecayRun; ++j)
       if (s + j < s1) {
-        const float g = rate * dl_softplus(x[j] + bias);
+        const float g = rate * softplus_for<T>(x[j] + bias);
         run = a.chunked ? run + g : g;
         a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] = run;
       }
   }
-  if (c % z.Dk == 0)
-    for (int s = s0; s < s1; ++s) a.beta[((int64_t)b * a.S + s) * z.heads + h] = dl_sigmoid(ld<T>(a.dn, ((int64_t)b * a.S + s) * z.ldn + z.off_b + h));
+  for (int s = s0 + c % z.Dk; s < s1; s += z.Dk) a.beta[((int64_t)b * a.S + s) * z.heads + h] = dl_sigmoid(ld<T>(a.dn, ((int64_t)b * a.S + s) * z.ldn + z.off_b + h));
 }
 
 // RPL state rows per lane (16 RPL >= Dk); rows past Dk stay zero.
@@ -250,6 +315,31 @@ __global__ void __launch_bounds__(256) k_delta_out(DeltaArgs a) {
     const int c = lane + 64 * i;
     if (c < z.Vp) Scalar<T>::store((T *)a.out + row * a.ldo + h * z.Vp + c, o[i] * r * ld<T>(a.norm_w, c) * dl_sigmoid(ld<T>(a.gate, job * z.Vp + c)));
   }
+}
+
+// The bf16 form for value heads of a power of two: Vp / 8 neighbouring lanes a (row, head).
+__global__ void __launch_bounds__(256) k_delta_out_wide(DeltaArgs a) {
+  const DeltaShape &z = a.s;
+  const int lanes = z.Vp / 8;
+  const int64_t e = (blockIdx.x * 256ll + threadIdx.x) * 8, job = e / z.Vp;
+  const int c = (int)(e - job * z.Vp);
+  if (job >= (int64_t)a.B * a.S * z.heads) return;
+  const int h = (int)(job % z.heads);
+  const int64_t row = job / z.heads;
+  const float4 o0 = *reinterpret_cast<const float4 *>(a.o + e), o1 = *reinterpret_cast<const float4 *>(a.o + e + 4);
+  const uint4 gv = *reinterpret_cast<const uint4 *>((const uint16_t *)a.gate + e), wv = *reinterpret_cast<const uint4 *>((const uint16_t *)a.norm_w + c);
+  float o[8] = {o0.x, o0.y, o0.z, o0.w, o1.x, o1.y, o1.z, o1.w}, sum = 0.f;
+  const uint32_t g[4] = {gv.x, gv.y, gv.z, gv.w}, w[4] = {wv.x, wv.y, wv.z, wv.w};
+#pragma unroll
+  for (int i = 0; i < 8; ++i) sum = fmaf(o[i], o[i], sum);   // padding columns hold zeros
+  const float r = 1.0f / sqrtf(group_sum(sum, lanes) / (float)z.vdim + a.eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const float gate = __uint_as_float(i & 1 ? g[i >> 1] & 0xffff0000u : g[i >> 1] << 16), wt = __uint_as_float(i & 1 ? w[i >> 1] & 0xffff0000u : w[i >> 1] << 16);
+    o[i] *= r * wt * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate));
+  }
+  *reinterpret_cast<uint4 *>((uint16_t *)a.out + row * a.ldo + h * z.Vp + c) =
+      make_uint4(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]), pack_bf16x2(o[4], o[5]), pack_bf16x2(o[6], o[7]));
 }
 
 // ---------------------------------------------------------------- one token per sequence
@@ -412,7 +502,12 @@ template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, Delt
   const int64_t outs = (int64_t)a.B * a.S * z.heads;
   RAI_REQUIRE((outs + 3) / 4 < (1ll << 31) && (a.S + kDeltaChunk - 1) / kDeltaChunk <= 65535, RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
   const dim3 go((unsigned)((outs + 3) / 4)), block(256);
-  if (wide <= 128) RAI_TRY((launch_prep<T, 1>(st, a)));
+  auto pow2 = [](int n) { return (n & (n - 1)) == 0; };
+  const bool wide_prep = sizeof(T) == 2 && z.taps == 4 && pow2(z.Dk) && (a.S + kWideTokens - 1) / kWideTokens <= 65535;
+  if (wide_prep) {
+    hipLaunchKernelGGL(k_delta_prep_wide, dim3((z.channels / 8 + 255) / 256, (a.S + kWideTokens - 1) / kWideTokens, a.B), block, 0, st, a);
+    RAI_TRY(launch_check("delta_prep_wide"));
+  } else if (wide <= 128) RAI_TRY((launch_prep<T, 1>(st, a)));
   else if (wide <= 256) RAI_TRY((launch_prep<T, 2>(st, a)));
   else RAI_TRY((launch_prep<T, 4>(st, a)));
   hipLaunchKernelGGL(k_delta_decay<T>, dim3((z.heads * z.Dk + 255) / 256, (a.S + kDeltaChunk - 1) / kDeltaChunk, a.B), block, 0, st, a);
@@ -423,6 +518,10 @@ template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, Delt
   else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));
   else if (z.Dk <= 256) RAI_TRY((launch_scan<T, 16>(st, a)));
   else RAI_TRY((launch_scan<T, 32>(st, a)));
+  if (sizeof(T) == 2 && pow2(z.Vp) && a.ldo % 8 == 0) {
+    hipLaunchKernelGGL(k_delta_out_wide, dim3((unsigned)((outs * (z.Vp / 8) + 255) / 256)), block, 0, st, a);
+    return launch_check("delta_out_wide");
+  }
   if (z.Vp <= 64) hipLaunchKernelGGL((k_delta_out<T, 1>), go, block, 0, st, a);
   else if (z.Vp <= 128) hipLaunchKernelGGL((k_delta_out<T, 2>), go, block, 0, st, a);
   else if (z.Vp <= 256) hipLaunchKernelGGL((k_delta_out<T, 4>), go, block, 0, st, a);

@@ -6,12 +6,16 @@
 // With L = beta A (strictly lower), U = U0 - W S0 where (1 + L) [U0 | W] = beta [V | K~].
 //   k_delta_chunk  everything that does not depend on the state, all chunks at once: A and P, then U0 and W by forward
 //                  substitution in blocks of 16 rows; the operands of the second kernel leave in MFMA-fragment order
-//   k_delta_pass   chunk after chunk per head and 32 columns of the state, which stays in accumulation registers
+//   k_delta_pass   chunk after chunk per head and 32 or 64 columns of the state, which stays in accumulation registers
 // exp(G_t - G_s) is never formed over a range that could overflow: block row i refers both factors to R_i, the sum at the
 // end of the block before it, so that each is at most 1 outside the block on the diagonal.  On the diagonal the second
 // factor is at least 1; if it would exceed e^60 there, that block is summed up pair by pair.
 // Products that feed the recurrence take their operands as two bf16 parts each (three MFMAs, 16 bits of mantissa);
 // the read-out's operands are rounded to bf16 once, as its result is.
+//
+// The order of the 32 terms of an MFMA step is free as long as both operands agree.  Here lane l's eight terms are
+// 4 (l / 16) .. + 3 of one block of 16 and the same of the next: exactly the rows that lane holds of two accumulator
+// tiles, so within k_delta_chunk a product's result is the next product's operand as it stands ("paired order" below).
 #include <cmath>
 
 #include "delta.h"
@@ -51,12 +55,6 @@ __device__ __forceinline__ dc_f32x4 mma3(const Halves &a, const Halves &b, dc_f3
 }
 __device__ __forceinline__ float fast_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
 __device__ __forceinline__ dc_bf16x8 zero8() { return __builtin_bit_cast(dc_bf16x8, dc_u32x4{0u, 0u, 0u, 0u}); }
-// Lanes of one wave hand values to each other through LDS.
-__device__ __forceinline__ void wave_lds_sync() {
-  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-}
-
 constexpr int C = kDeltaChunk;
 // One (sequence, chunk, head)'s part of the workspace, in bytes.
 struct ChunkLayout {
@@ -64,361 +62,410 @@ struct ChunkLayout {
 };
 __host__ __device__ inline ChunkLayout chunk_layout(int D, int E) {
   ChunkLayout l;
-  l.w = 0;                      // [4 row blocks][D / 32][hi, lo][64 lanes][8]      A operand, rows t
-  l.q = l.w + C * D * 4;        // [4][D / 32][64][8]                               A operand, rows t
-  l.k = l.q + C * D * 2;        // [D / 16][2 steps of 32 tokens][hi, lo][64][8]    B operand, columns d
-  l.p = l.k + C * D * 4;        // [4][2][64][8]                                    A operand, rows t
+  l.w = 0;                      // [4 row blocks][D / 32][hi, lo][64 lanes][8]      rows t, terms d in paired order
+  l.q = l.w + C * D * 4;        // [4][D / 32][64][8]                               rows t, terms d
+  l.k = l.q + C * D * 2;        // [D / 16][2 steps of 32 tokens][hi, lo][64][8]    rows d, terms t
+  l.p = l.k + C * D * 4;        // [4][2][64][8]                                    rows t, terms s (step 1 of blocks 0, 1 unused)
   l.u = l.p + C * C * 2;        // [4][E / 16][64][4] f32                           accumulator order
   l.total = l.u + C * E * 4;
   return l;
 }
 
-__device__ __forceinline__ void load8(const float *p, bool ok, float (&x)[8]) {
+// Two runs of four values, 16 apart: a lane's share of a step in paired order.
+__device__ __forceinline__ void load_pair(const float *p, float (&x)[8]) {
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
-    const dc_f32x4 v = ok ? *reinterpret_cast<const dc_f32x4 *>(p + 4 * i) : dc_f32x4{0.f, 0.f, 0.f, 0.f};
+    const dc_f32x4 v = *reinterpret_cast<const dc_f32x4 *>(p + 16 * i);
 #pragma unroll
     for (int e = 0; e < 4; ++e) x[4 * i + e] = v[e];
   }
 }
+// Two accumulator tiles as one operand; a missing second one counts as zeros.
+__device__ __forceinline__ Halves split_pair(const dc_f32x4 &a, const dc_f32x4 &b) {
+  const float x[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+  return split8(x);
+}
 
-constexpr int kAP = C + 4, kNP = 20, kXP = C + 8;   // LDS pitches
-template <int D>
-__global__ void __launch_bounds__(256) k_delta_chunk(DeltaArgs a) {
-  constexpr int KS = D / 32;
-  __shared__ __attribute__((aligned(16))) float Ls[C * kAP];              // beta A, strictly lower
-  __shared__ __attribute__((aligned(16))) float Ns[4 * 16 * kNP];         // inverses of the diagonal blocks of 1 + L
-  __shared__ __attribute__((aligned(16))) uint16_t Xs[4][2][16 * kXP];    // per wave: solved rows of a 16-column tile, transposed, hi / lo
+constexpr int kLP = 20;   // pitch of a 16 x 16 block in LDS (floats)
+template <int D> constexpr int chunk_lds_floats() { return 2 * C * (D + 4) + 10 * 16 * kLP + C; }   // D = 128: two blocks to a CU
+
+// WAVES = 8 for few chunks, 4 (two blocks to a CU) for many.
+template <int D, int WAVES>
+__global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
+  constexpr int KS = D / 32, KP = D + 4, kChunkWaves = WAVES, kChunkThreads = WAVES * 64;
+  extern __shared__ __attribute__((aligned(16))) float dc_lds[];
+  float *Kl = dc_lds, *Gl = Kl + C * KP;      // [64][D] keys and running sums; rows past the end: 0 and the last sum
+  float *Ls = Gl + C * KP;                    // blocks (i, j <= i) of beta A, strictly lower, number i (i + 1) / 2 + j; on the
+                                              // diagonal later the inverses of the blocks of 1 + L
+  float *bs = Ls + 10 * 16 * kLP;
   const DeltaShape &z = a.s;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lq = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int n = blockIdx.x, h = blockIdx.y, b = blockIdx.z, kv = h / (z.heads / z.kv_heads);
   const int len = a.S - n * C < C ? a.S - n * C : C;
   const int64_t row0 = (int64_t)b * a.S + n * C;
   const int64_t ldk = (int64_t)z.kv_heads * D, ldg = (int64_t)z.heads * D, ldv = (int64_t)z.heads * z.Vp;
   const float *q = a.q + row0 * ldk + kv * D, *k = a.k + row0 * ldk + kv * D, *G = a.decay + row0 * ldg + h * D;
-  const float *beta = a.beta + row0 * z.heads + h;
   const bf16_raw *v = (const bf16_raw *)a.v + row0 * ldv + h * z.Vp;
   const ChunkLayout lay = chunk_layout(D, z.Vp);
   char *ws = a.chunk_ws + (((int64_t)b * gridDim.x + n) * z.heads + h) * lay.total;
-  for (int i = lane; i < 16 * kXP; i += 64) Xs[wave][0][i] = Xs[wave][1][i] = 0;   // multiplied by zeros before they are solved
+  // queries of row t, a step's terms
+  auto query = [&](int t, int ks, float (&x)[8]) {
+    if (t < len) load_pair(q + (int64_t)t * ldk + 32 * ks + 4 * lq, x);
+    else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = 0.f;
+    }
+  };
+  // block (i, j) of the lower triangle number idx
+  auto block_row = [](int idx) { return idx < 1 ? 0 : idx < 3 ? 1 : idx < 6 ? 2 : 3; };
 
-  // ---- A and P, block row `wave`
-  const int i = wave, t0 = 16 * i;
-  const int prev = t0 - 1 < len - 1 ? t0 - 1 : len - 1;                  // the token that R_i is the sum at
-  const int tl = t0 + l16, last = t0 + 15 < len - 1 ? t0 + 15 : len - 1;
-  dc_f32x4 A[4], P[4];
+  float qt[KS][8];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) A[j] = P[j] = dc_f32x4{0.f, 0.f, 0.f, 0.f};
-  float range = 0.f;
-  for (int ks = 0; ks < KS; ++ks) {
-    const int d = 32 * ks + 8 * lq;
-    const bool in = tl < len;
-    float R[8], kt[8], qt[8], gt[8], e[8], x[8];
-    load8(G + (int64_t)prev * ldg + d, i > 0, R);
-    load8(k + (int64_t)tl * ldk + d, in, kt);
-    load8(q + (int64_t)tl * ldk + d, in, qt);
-    load8(G + (int64_t)tl * ldg + d, in, gt);
-    if (t0 < len) {
-      float ge[8];
-      load8(G + (int64_t)last * ldg + d, true, ge);
-#pragma unroll
-      for (int y = 0; y < 8; ++y) range = fmaxf(range, R[y] - ge[y]);
-    }
-#pragma unroll
-    for (int y = 0; y < 8; ++y) x[y] = in ? qt[y] * fast_exp(gt[y]) : 0.f;
-    *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + ((i * KS + ks) * 64 + lane) * 16) = round8(x);
-#pragma unroll
-    for (int y = 0; y < 8; ++y) {
-      e[y] = in ? fast_exp(gt[y] - R[y]) : 0.f;
-      kt[y] *= e[y];
-      qt[y] *= e[y];
-    }
-    const Halves ka = split8(kt);
-    const dc_bf16x8 qa = round8(qt);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      if (j > i) continue;
-      const int s = 16 * j + l16;
-      float kb[8], gs[8];
-      load8(k + (int64_t)s * ldk + d, s < len, kb);
-      load8(G + (int64_t)s * ldg + d, s < len, gs);
-#pragma unroll
-      for (int y = 0; y < 8; ++y) kb[y] = s < len ? kb[y] * fast_exp(R[y] - gs[y]) : 0.f;
-      const Halves kB = split8(kb);
-      A[j] = mma3(ka, kB, A[j]);
-      P[j] = mma(qa, kB.hi, P[j]);
-    }
+  for (int ks = 0; ks < KS; ++ks) query(16 * block_row(wave) + l16, ks, qt[ks]);
+  for (int e = tid; e < C * D / 4; e += kChunkThreads) {
+    const int t = e / (D / 4), d = (e - t * (D / 4)) * 4;
+    const int tc = t < len ? t : len - 1;
+    dc_f32x4 kx = *reinterpret_cast<const dc_f32x4 *>(k + (int64_t)tc * ldk + d);
+    const dc_f32x4 gx = *reinterpret_cast<const dc_f32x4 *>(G + (int64_t)tc * ldg + d);
+    if (t >= len) kx = dc_f32x4{0.f, 0.f, 0.f, 0.f};
+    *reinterpret_cast<dc_f32x4 *>(Kl + t * KP + d) = kx;
+    *reinterpret_cast<dc_f32x4 *>(Gl + t * KP + d) = gx;
   }
-  if (wave_max(range) > 60.f) {   // the diagonal block pair by pair
+  if (tid < C) bs[tid] = tid < len ? a.beta[(row0 + tid) * z.heads + h] : 0.f;
+  __syncthreads();
+
+  // ---- blocks of A and P
+  for (int idx = wave; idx < 10; idx += kChunkWaves) {
+    const int i = block_row(idx), j = idx - i * (i + 1) / 2, t0 = 16 * i, t = t0 + l16, s = 16 * j + l16;
+    dc_f32x4 A = {0.f, 0.f, 0.f, 0.f}, P = A;   // A: rows t, columns s;  P: rows s, columns t
+    float range = 0.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = t0 + 4 * lq + r, s = t0 + l16;
-      float sa = 0.f, sp = 0.f;
-      if (s <= t && t < len)
+    for (int ks = 0; ks < KS; ++ks) {
+      const int d = 32 * ks + 4 * lq;
+      float R[8], kt[8], gt[8], kb[8], gs[8], qx[8];
+      if (idx >= kChunkWaves) query(t, ks, qt[ks]);
+      load_pair(Kl + t * KP + d, kt);
+      load_pair(Gl + t * KP + d, gt);
+      load_pair(Kl + s * KP + d, kb);
+      load_pair(Gl + s * KP + d, gs);
+      if (i > 0) load_pair(Gl + (t0 - 1) * KP + d, R);
+      else {
+#pragma unroll
+        for (int y = 0; y < 8; ++y) R[y] = 0.f;
+      }
+      if (i == j) {
+        float ge[8];
+        load_pair(Gl + (t0 + 15) * KP + d, ge);
+#pragma unroll
+        for (int y = 0; y < 8; ++y) range = fmaxf(range, R[y] - ge[y]);
+      }
+#pragma unroll
+      for (int y = 0; y < 8; ++y) {
+        const float e = fast_exp(gt[y] - R[y]);
+        kt[y] *= e;
+        qx[y] = qt[ks][y] * e;
+        kb[y] *= fast_exp(R[y] - gs[y]);
+      }
+      const Halves kB = split8(kb);
+      A = mma3(split8(kt), kB, A);
+      P = mma(kB.hi, round8(qx), P);
+    }
+    if (i == j && wave_max(range) > 60.f) {   // pair by pair
+#pragma unroll 1
+      for (int r = 0; r < 4; ++r) {
+        const int m = 4 * lq + r;             // A of (t0 + m, t0 + l16) and P of (t0 + l16, t0 + m)
+        float sa = 0.f, sp = 0.f;
         for (int d = 0; d < D; ++d) {
-          const float w = k[(int64_t)s * ldk + d] * fast_exp(G[(int64_t)t * ldg + d] - G[(int64_t)s * ldg + d]);
-          sa = fmaf(k[(int64_t)t * ldk + d], w, sa);
-          sp = fmaf(q[(int64_t)t * ldk + d], w, sp);
+          const float gm = Gl[(t0 + m) * KP + d], gl = Gl[t * KP + d], km = Kl[(t0 + m) * KP + d], kl = Kl[t * KP + d];
+          if (l16 <= m) sa = fmaf(km * kl, fast_exp(gm - gl), sa);
+          if (m <= l16 && t < len) sp = fmaf(q[(int64_t)t * ldk + d] * km, fast_exp(gl - gm), sp);
         }
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (j == i) { A[j][r] = sa; P[j][r] = sp; }
+        for (int e = 0; e < 4; ++e)
+          if (e == r) { A[e] = sa; P[e] = sp; }
+      }
     }
-  }
-  float bt[4];   // beta of the rows this lane holds of a block's accumulator, per block
-#pragma unroll
-  for (int r = 0; r < 4; ++r) bt[r] = t0 + 4 * lq + r < len ? beta[(int64_t)(t0 + 4 * lq + r) * z.heads] : 0.f;
-#pragma unroll
-  for (int j = 0; j < 4; ++j)
+    dc_u32x2 pw;
+    float px[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int t = t0 + 4 * lq + r, s = 16 * j + l16;
-      if (j <= i) Ls[t * kAP + s] = s < t ? bt[r] * A[j][r] : 0.f;
-      const float p = j <= i && s <= t ? P[j][r] : 0.f;
-      reinterpret_cast<uint16_t *>(ws + lay.p)[((i * 2 + j / 2) * 64 + (t & 15) + 16 * ((s & 31) >> 3)) * 8 + (s & 7)] = f32_to_bf16_bits(p);
+      const int m = 4 * lq + r;
+      Ls[(idx * 16 + m) * kLP + l16] = s < t0 + m ? bs[t0 + m] * A[r] : 0.f;
+      px[r] = 16 * j + m <= t ? P[r] : 0.f;
     }
+    pw.x = pack_bf16x2(px[0], px[1]);
+    pw.y = pack_bf16x2(px[2], px[3]);
+    *reinterpret_cast<dc_u32x2 *>(ws + lay.p + ((i * 2 + j / 2) * 64 + lane) * 16 + (j & 1) * 8) = pw;
+  }
+  if (wave >= kChunkWaves - 2) {   // the blocks above the diagonal that share a step with one on or below it
+    const int i = wave == kChunkWaves - 1 ? 2 : 0;
+    *reinterpret_cast<dc_u32x2 *>(ws + lay.p + ((i * 2 + i / 2) * 64 + lane) * 16 + 8) = dc_u32x2{0u, 0u};
+  }
   __syncthreads();
-  // ---- the diagonal block's inverse, lane = column (four copies)
-  {
+  // ---- operand of the state's update: k_s exp(G_C - G_s), rows d
+  auto update_operand = [&](int f) {
+    const int dt = f >> 1, ks = f & 1, d = 16 * dt + l16;
+    const float gc = Gl[(C - 1) * KP + d];
+    float x[8];
+#pragma unroll
+    for (int y = 0; y < 8; ++y) {
+      const int s = 32 * ks + 16 * (y >> 2) + 4 * lq + (y & 3);
+      x[y] = Kl[s * KP + d] * fast_exp(gc - Gl[s * KP + d]);
+    }
+    const Halves o = split8(x);
+    char *dst = ws + lay.k + (f * 2 * 64 + lane) * 16;
+    *reinterpret_cast<dc_bf16x8 *>(dst) = o.hi;
+    *reinterpret_cast<dc_bf16x8 *>(dst + 64 * 16) = o.lo;
+  };
+  if (wave < 4) {
+    // ---- inverses of the diagonal blocks, lane = column (four copies); a block is read whole before it is overwritten
+    float *blk = Ls + (wave * (wave + 1) / 2 + wave) * 16 * kLP;
     float x[16];
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-      float s = t == l16 ? 1.f : 0.f;
+      float s0 = t == l16 ? 1.f : 0.f, s1 = 0.f;
 #pragma unroll
-      for (int m = 0; m < t; ++m) s = fmaf(-Ls[(t0 + t) * kAP + t0 + m], x[m], s);
-      x[t] = s;
-      if (lq == 0) Ns[(i * 16 + t) * kNP + l16] = s;
+      for (int m = 0; m < t; ++m) (m & 1 ? s1 : s0) = fmaf(-blk[t * kLP + m], x[m], m & 1 ? s1 : s0);
+      x[t] = s0 + s1;
     }
+    __builtin_amdgcn_wave_barrier();
+    if (lq == 0) {
+#pragma unroll
+      for (int t = 0; t < 16; ++t) blk[t * kLP + l16] = x[t];
+    }
+    if constexpr (WAVES == 4)
+      for (int f = wave; f < D / 8; f += 4) update_operand(f);
+  } else {
+    for (int f = wave - 4; f < D / 8; f += 4) update_operand(f);
   }
-  // ---- operand of the state's update: k_s exp(G_C - G_s), channels as columns
-  for (int dt = wave; dt < D / 16; dt += 4) {
-    const int d = 16 * dt + l16;
-    const float gc = G[(int64_t)(len - 1) * ldg + d];
+  // ---- scaled queries
+  for (int f = wave; f < 4 * KS; f += kChunkWaves) {
+    const int t = 16 * (f / KS) + l16, ks = f % KS;
+    float x[8], g[8];
+    query(t, ks, x);
+    load_pair(Gl + t * KP + 32 * ks + 4 * lq, g);
 #pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      float x[8];
-#pragma unroll
-      for (int y = 0; y < 8; ++y) {
-        const int s = 32 * ks + 8 * lq + y;
-        x[y] = s < len ? k[(int64_t)s * ldk + d] * fast_exp(gc - G[(int64_t)s * ldg + d]) : 0.f;
-      }
-      const Halves o = split8(x);
-      char *dst = ws + lay.k + ((dt * 2 + ks) * 2 * 64 + lane) * 16;
-      *reinterpret_cast<dc_bf16x8 *>(dst) = o.hi;
-      *reinterpret_cast<dc_bf16x8 *>(dst + 64 * 16) = o.lo;
-    }
+    for (int y = 0; y < 8; ++y) x[y] *= fast_exp(g[y]);
+    *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + (f * 64 + lane) * 16) = round8(x);
   }
   __syncthreads();
-  // ---- (1 + L) X = beta [V | K~], a tile of 16 columns at a time
-  const int vt = z.Vp / 16;
-  uint16_t *xh = Xs[wave][0], *xl = Xs[wave][1];
-  auto put = [&](int at, const dc_f32x4 &y) {   // rows at + 4 lq .. + 3 of column l16
-    const dc_u32x2 hi = {pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
-    const dc_u32x2 lo = {pack_bf16x2(y[0] - bf_lo(hi.x), y[1] - bf_hi(hi.x)), pack_bf16x2(y[2] - bf_lo(hi.y), y[3] - bf_hi(hi.y))};
-    *reinterpret_cast<dc_u32x2 *>(xh + l16 * kXP + at + 4 * lq) = hi;
-    *reinterpret_cast<dc_u32x2 *>(xl + l16 * kXP + at + 4 * lq) = lo;
-  };
-  auto get = [&](int at) {                      // rows at .. + 7 of column l16
-    Halves r;
-    r.hi = *reinterpret_cast<const dc_bf16x8 *>(xh + l16 * kXP + at);
-    r.lo = *reinterpret_cast<const dc_bf16x8 *>(xl + l16 * kXP + at);
-    return r;
-  };
-  for (int tile = wave; tile < vt + D / 16; tile += 4) {
-    const bool val = tile < vt;
-    const int c = (val ? tile : tile - vt) * 16 + l16;
-    float rhs[4][4];
+  // ---- (1 + L) X = beta [V | K~], two tiles of 16 columns at a time
+  Halves Lf[4], Nf[4], one;   // L of block rows 1, 2, 3 (first two blocks) and 3 (third), the inverses, the unit matrix
 #pragma unroll
-    for (int ib = 0; ib < 4; ++ib)
+  for (int ib = 0; ib < 4; ++ib) {
+    float x[8];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = 16 * ib + 4 * lq + r;
-        rhs[ib][r] = 0.f;
-        if (t < len) {
-          const float be = beta[(int64_t)t * z.heads];
-          rhs[ib][r] = be * (val ? bf16_bits_to_f32(v[(int64_t)t * ldv + c].bits) : k[(int64_t)t * ldk + c] * fast_exp(G[(int64_t)t * ldg + c]));
-        }
-      }
+    for (int y = 0; y < 8; ++y) x[y] = 0.f;
+    const dc_f32x4 nv = *reinterpret_cast<const dc_f32x4 *>(Ls + ((ib * (ib + 1) / 2 + ib) * 16 + l16) * kLP + 4 * lq);
 #pragma unroll
-    for (int ib = 0; ib < 4; ++ib) {
-      dc_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int y = 0; y < 4; ++y) x[y] = nv[y];
+    Nf[ib] = split8(x);
+    const int row = ib < 3 ? ib + 1 : 3, col = ib < 3 ? 0 : 2, blk = row * (row + 1) / 2 + col;
 #pragma unroll
-      for (int ks = 0; ks < (16 * ib + 31) / 32; ++ks) {
-        const int s = 32 * ks + 8 * lq;
-        float x[8];
+    for (int y = 0; y < 2; ++y) {   // the second block of the step may lie on the diagonal
+      const bool below = col + y < row;
+      const dc_f32x4 lv = *reinterpret_cast<const dc_f32x4 *>(Ls + ((below ? blk + y : blk) * 16 + l16) * kLP + 4 * lq);
 #pragma unroll
-        for (int y = 0; y < 8; ++y) x[y] = 0.f;
-        if (s < 16 * ib) load8(Ls + (16 * ib + l16) * kAP + s, true, x);
-        acc = mma3(split8(x), get(s), acc);
-      }
-      dc_f32x4 y;
+      for (int e = 0; e < 4; ++e) x[4 * y + e] = below ? lv[e] : 0.f;
+    }
+    Lf[ib] = split8(x);
+  }
+  {
+    float x[8];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) y[r] = rhs[ib][r] - acc[r];
-      wave_lds_sync();
-      put(16 * ib, y);
-      wave_lds_sync();
-      float x[8];
+    for (int y = 0; y < 8; ++y) x[y] = y < 4 && 4 * lq + y == l16 ? 1.f : 0.f;
+    one.hi = round8(x);
+  }
+  const int vp = z.Vp / 32;
+  const dc_f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  for (int pair = wave; pair < vp + KS; pair += kChunkWaves) {
+    const bool val = pair < vp;
+    const int c0 = (val ? pair : pair - vp) * 32 + l16;
+    dc_f32x4 X[2][4];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] = 0.f;
-      Halves yb;
-      yb.hi = yb.lo = zero8();
-      if (lq < 2) {
-        load8(Ns + (ib * 16 + l16) * kNP + 8 * lq, true, x);
-        yb = get(16 * ib + 8 * lq);
-      }
-      const dc_f32x4 o = mma3(split8(x), yb, dc_f32x4{0.f, 0.f, 0.f, 0.f});
-      wave_lds_sync();
-      put(16 * ib, o);
-      wave_lds_sync();
-      if (val) *reinterpret_cast<dc_f32x4 *>(ws + lay.u + ((ib * vt + tile) * 64 + lane) * 16) = o;
-      else {
-        uint16_t *dst = reinterpret_cast<uint16_t *>(ws + lay.w) + (((ib * KS + (c >> 5)) * 2 * 64) + 16 * ((c & 31) >> 3)) * 8 + (c & 7);
+    for (int e = 0; e < 2; ++e)
+#pragma unroll
+      for (int ib = 0; ib < 4; ++ib)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const uint16_t hi = f32_to_bf16_bits(o[r]);
-          dst[(4 * lq + r) * 8] = hi;
-          dst[(64 + 4 * lq + r) * 8] = f32_to_bf16_bits(o[r] - bf16_bits_to_f32(hi));
+          const int t = 16 * ib + 4 * lq + r, c = c0 + 16 * e;
+          X[e][ib][r] = bs[t] * (val ? bf16_bits_to_f32(v[(int64_t)(t < len ? t : len - 1) * ldv + c].bits) : Kl[t * KP + c] * fast_exp(Gl[t * KP + c]));
         }
+    Halves first[2];   // solved blocks 0 and 1
+#pragma unroll
+    for (int ib = 0; ib < 4; ++ib) {
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        dc_f32x4 y = X[e][ib];
+        if (ib > 0) {
+          dc_f32x4 acc = mma3(Lf[ib - 1], first[e], zero);
+          if (ib == 3) acc = mma3(Lf[3], split_pair(X[e][2], zero), acc);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) y[r] -= acc[r];
+        }
+        X[e][ib] = mma3(Nf[ib], split_pair(y, zero), zero);
+        if (ib == 0) first[e] = split_pair(X[e][0], zero);
+        if (ib == 1) first[e] = split_pair(X[e][0], X[e][1]);
+      }
+    }
+#pragma unroll
+    for (int ib = 0; ib < 4; ++ib) {
+      if (val) {
+#pragma unroll
+        for (int e = 0; e < 2; ++e) *reinterpret_cast<dc_f32x4 *>(ws + lay.u + ((ib * 2 * vp + pair * 2 + e) * 64 + lane) * 16) = X[e][ib];
+      } else {   // rows t, columns d become rows d, columns t: each lane then holds the terms d of its own row t
+        dc_f32x4 Xt[2];
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          const Halves x = split_pair(X[e][ib], zero);
+          Xt[e] = mma(x.hi, one.hi, mma(x.lo, one.hi, zero));
+        }
+        const Halves o = split_pair(Xt[0], Xt[1]);
+        char *dst = ws + lay.w + ((ib * KS + pair - vp) * 2 * 64 + lane) * 16;
+        *reinterpret_cast<dc_bf16x8 *>(dst) = o.hi;
+        *reinterpret_cast<dc_bf16x8 *>(dst + 64 * 16) = o.lo;
       }
     }
   }
 }
 
-// One wave's operands of one chunk.
-template <int D> struct PassOperands {
-  static constexpr int KS = D / 32, DT = D / 64;
-  dc_bf16x8 wh[KS], wl[KS], q[KS], p[2], kh[DT][2], kl[DT][2];
-  dc_f32x4 u[2];
-  float g[DT];
-  __device__ __forceinline__ void load(const char *ws, const ChunkLayout &lay, int wave, int lane, int e16, int vt, const float *G) {
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const char *p = ws + lay.w + ((wave * KS + ks) * 2 * 64 + lane) * 16;
-      wh[ks] = *reinterpret_cast<const dc_bf16x8 *>(p);
-      wl[ks] = *reinterpret_cast<const dc_bf16x8 *>(p + 64 * 16);
-      q[ks] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.q + ((wave * KS + ks) * 64 + lane) * 16);
-    }
-#pragma unroll
-    for (int e = 0; e < 2; ++e) u[e] = *reinterpret_cast<const dc_f32x4 *>(ws + lay.u + ((wave * vt + e16 + e) * 64 + lane) * 16);
-#pragma unroll
-    for (int ks = 0; ks < 2; ++ks) p[ks] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + ks) * 64 + lane) * 16);
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      g[dt] = G[(wave * DT + dt) * 16 + (lane & 15)];
-#pragma unroll
-      for (int ks = 0; ks < 2; ++ks) {
-        const char *p = ws + lay.k + (((wave * DT + dt) * 2 + ks) * 2 * 64 + lane) * 16;
-        kh[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(p);
-        kl[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(p + 64 * 16);
-      }
-    }
-  }
-};
-
-// Block = (32 columns e of the state, head, sequence).  Wave w owns rows 16 w .. + 15 of a chunk in the products over the
-// state, and channels w D / 4 .. of the state itself, transposed: rows e, columns d.
-template <int D>
+// Block = (16 EB columns e of the state, head, sequence).  Wave w owns rows 16 w .. + 15 of a chunk in the products over
+// the state, and channels w D / 4 .. of the state itself, transposed: rows e, columns d.  State and U pass through LDS as
+// operands, their terms stored in paired order.  The operands of either half of a chunk are requested as soon as the
+// ones before them have been used.
+__device__ __forceinline__ int paired(int term) { return (term & ~31) | ((term & 12) << 1) | ((term & 16) >> 2) | (term & 3); }
+template <int D, int EB>
 __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
   constexpr int KS = D / 32, DT = D / 64, SP = D + 8, UP = C + 8;
-  __shared__ __attribute__((aligned(16))) uint16_t St[2][32 * SP];   // hi / lo of the state, [e][d]
-  __shared__ __attribute__((aligned(16))) uint16_t Ut[2][32 * UP];   // of U, [e][t]
+  __shared__ __attribute__((aligned(16))) uint16_t St[2][16 * EB * SP];   // hi / lo of the state, [e][d]
+  __shared__ __attribute__((aligned(16))) uint16_t Ut[2][16 * EB * UP];   // of U, [e][t]
   const DeltaShape &z = a.s;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lq = lane >> 4;
-  const int e0 = blockIdx.x * 32, h = blockIdx.y, b = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int e0 = blockIdx.x * 16 * EB, h = blockIdx.y, b = blockIdx.z;
   const int chunks = (a.S + C - 1) / C, vt = z.Vp / 16;
   const ChunkLayout lay = chunk_layout(D, z.Vp);
   const int pos0 = a.state->pos;
-  const char *ws = a.chunk_ws + ((int64_t)b * chunks * z.heads + h) * lay.total;
+  const char *ws0 = a.chunk_ws + ((int64_t)b * chunks * z.heads + h) * lay.total;
   const int64_t step = (int64_t)z.heads * lay.total, ldg = (int64_t)z.heads * D;
   const float *G = a.decay + (int64_t)b * a.S * ldg + h * D;
   float *carried = a.carried + ((int64_t)b * z.heads + h) * D * z.Vp + e0;
-  dc_f32x4 S[DT][2];
+  dc_f32x4 S[DT][EB];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-    for (int e = 0; e < 2; ++e) {
+    for (int e = 0; e < EB; ++e) {
       const int d = (wave * DT + dt) * 16 + l16;
       S[dt][e] = dc_f32x4{0.f, 0.f, 0.f, 0.f};
       if (pos0 > 0) S[dt][e] = *reinterpret_cast<const dc_f32x4 *>(carried + (int64_t)d * z.Vp + 16 * e + 4 * lq);
     }
-  PassOperands<D> cur;
-  auto request = [&](int n) {
-    const int last = (n + 1) * C < a.S ? (n + 1) * C - 1 : a.S - 1;
-    cur.load(ws + n * step, lay, wave, lane, e0 / 16, vt, G + (int64_t)last * ldg);
+  dc_bf16x8 wh[KS], wl[KS], q[KS], p[2], kh[DT][2], kl[DT][2];
+  dc_f32x4 u[EB];
+  float g[DT];
+  auto request_first = [&](int n) {
+    const char *ws = ws0 + n * step;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const char *src = ws + lay.w + ((wave * KS + ks) * 2 * 64 + lane) * 16;
+      wh[ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
+      wl[ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
+      q[ks] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.q + ((wave * KS + ks) * 64 + lane) * 16);
+    }
+#pragma unroll
+    for (int e = 0; e < EB; ++e) u[e] = *reinterpret_cast<const dc_f32x4 *>(ws + lay.u + ((wave * vt + e0 / 16 + e) * 64 + lane) * 16);
   };
-  request(0);
+  auto request_second = [&](int n) {
+    const char *ws = ws0 + n * step;
+    const int last = (n + 1) * C < a.S ? (n + 1) * C - 1 : a.S - 1;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      g[dt] = G[(int64_t)last * ldg + (wave * DT + dt) * 16 + l16];
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks) {
+        const char *src = ws + lay.k + (((wave * DT + dt) * 2 + ks) * 2 * 64 + lane) * 16;
+        kh[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
+        kl[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
+      }
+    }
+    p[0] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + (wave * 2 * 64 + lane) * 16);
+    if (wave >= 2) p[1] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + 1) * 64 + lane) * 16);
+  };
+  request_first(0);
+  request_second(0);
   for (int n = 0; n < chunks; ++n) {
     // ---- the state as an operand
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt)
+    for (int dt = 0; dt < DT; ++dt) {
+      const int pd = paired((wave * DT + dt) * 16 + l16);
 #pragma unroll
-      for (int e = 0; e < 2; ++e)
+      for (int e = 0; e < EB; ++e)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int at = (16 * e + 4 * lq + r) * SP + (wave * DT + dt) * 16 + l16;
+          const int at = (16 * e + 4 * lq + r) * SP + pd;
           const uint16_t hi = f32_to_bf16_bits(S[dt][e][r]);
           St[0][at] = hi;
           St[1][at] = f32_to_bf16_bits(S[dt][e][r] - bf16_bits_to_f32(hi));
         }
+    }
     __syncthreads();
-    dc_f32x4 U[2], O[2];
+    dc_f32x4 O[EB];
 #pragma unroll
-    for (int e = 0; e < 2; ++e) {
+    for (int e = 0; e < EB; ++e) {
       dc_f32x4 x = {0.f, 0.f, 0.f, 0.f}, x2 = x, x3 = x;
       O[e] = x;
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
         const int at = (16 * e + l16) * SP + 32 * ks + 8 * lq;
         const dc_bf16x8 sh = *reinterpret_cast<const dc_bf16x8 *>(St[0] + at), sl = *reinterpret_cast<const dc_bf16x8 *>(St[1] + at);
-        x = mma(cur.wh[ks], sh, x);
-        x2 = mma(cur.wh[ks], sl, x2);
-        x3 = mma(cur.wl[ks], sh, x3);
-        O[e] = mma(cur.q[ks], sh, O[e]);
+        x = mma(wh[ks], sh, x);
+        x2 = mma(wh[ks], sl, x2);
+        x3 = mma(wl[ks], sh, x3);
+        O[e] = mma(q[ks], sh, O[e]);
       }
+      float U[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) U[e][r] = cur.u[e][r] - (x[r] + (x2[r] + x3[r]));
-      const dc_u32x2 hi = {pack_bf16x2(U[e][0], U[e][1]), pack_bf16x2(U[e][2], U[e][3])};
-      const dc_u32x2 lo = {pack_bf16x2(U[e][0] - bf_lo(hi.x), U[e][1] - bf_hi(hi.x)), pack_bf16x2(U[e][2] - bf_lo(hi.y), U[e][3] - bf_hi(hi.y))};
-      const int at = (16 * e + l16) * UP + 16 * wave + 4 * lq;
+      for (int r = 0; r < 4; ++r) U[r] = u[e][r] - (x[r] + (x2[r] + x3[r]));
+      const dc_u32x2 hi = {pack_bf16x2(U[0], U[1]), pack_bf16x2(U[2], U[3])};
+      const dc_u32x2 lo = {pack_bf16x2(U[0] - bf_lo(hi.x), U[1] - bf_hi(hi.x)), pack_bf16x2(U[2] - bf_lo(hi.y), U[3] - bf_hi(hi.y))};
+      const int at = (16 * e + l16) * UP + paired(16 * wave + 4 * lq);
       *reinterpret_cast<dc_u32x2 *>(Ut[0] + at) = hi;
       *reinterpret_cast<dc_u32x2 *>(Ut[1] + at) = lo;
     }
+    if (n + 1 < chunks) request_first(n + 1);
     __syncthreads();
-    // ---- read-out and update
-    Halves ua[2][2];
+    // ---- update and read-out
+    float w[DT];
 #pragma unroll
-    for (int e = 0; e < 2; ++e)
+    for (int dt = 0; dt < DT; ++dt) w[dt] = fast_exp(g[dt]);
+#pragma unroll
+    for (int e = 0; e < EB; ++e) {
+      Halves ua[2];
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         const int at = (16 * e + l16) * UP + 32 * ks + 8 * lq;
-        ua[e][ks].hi = *reinterpret_cast<const dc_bf16x8 *>(Ut[0] + at);
-        ua[e][ks].lo = *reinterpret_cast<const dc_bf16x8 *>(Ut[1] + at);
+        ua[ks].hi = *reinterpret_cast<const dc_bf16x8 *>(Ut[0] + at);
+        ua[ks].lo = *reinterpret_cast<const dc_bf16x8 *>(Ut[1] + at);
       }
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      const float w = fast_exp(cur.g[dt]);
+      for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
-      for (int e = 0; e < 2; ++e) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) S[dt][e][r] *= w;
+        for (int r = 0; r < 4; ++r) S[dt][e][r] *= w[dt];
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
           Halves kb;
-          kb.hi = cur.kh[dt][ks];
-          kb.lo = cur.kl[dt][ks];
-          S[dt][e] = mma3(ua[e][ks], kb, S[dt][e]);
+          kb.hi = kh[dt][ks];
+          kb.lo = kl[dt][ks];
+          S[dt][e] = mma3(ua[ks], kb, S[dt][e]);
         }
       }
+      O[e] = mma(p[0], ua[0].hi, O[e]);
+      if (wave >= 2) O[e] = mma(p[1], ua[1].hi, O[e]);
     }
-#pragma unroll
-    for (int e = 0; e < 2; ++e) {
-#pragma unroll
-      for (int ks = 0; ks < 2; ++ks) O[e] = mma(cur.p[ks], ua[e][ks].hi, O[e]);   // U's columns serve as B: lane = column e
-    }
+    if (n + 1 < chunks) request_second(n + 1);
     const int t0 = n * C + 16 * wave + 4 * lq;
-    if (n + 1 < chunks) request(n + 1);
 #pragma unroll
-    for (int e = 0; e < 2; ++e)
+    for (int e = 0; e < EB; ++e)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (t0 + r < a.S) a.o[(((int64_t)b * a.S + t0 + r) * z.heads + h) * z.Vp + e0 + 16 * e + l16] = O[e][r];
@@ -426,7 +473,7 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-    for (int e = 0; e < 2; ++e)
+    for (int e = 0; e < EB; ++e)
       *reinterpret_cast<dc_f32x4 *>(carried + (int64_t)((wave * DT + dt) * 16 + l16) * z.Vp + 16 * e + 4 * lq) = S[dt][e];
   if (blockIdx.x == 0) update_ring<bf16_raw>(a, b, h, pos0, tid, 256);
 }
@@ -438,11 +485,27 @@ size_t delta_chunk_ws_bytes(const DeltaShape &z, int64_t max_batch, int64_t max_
   return (size_t)(max_rows / C + max_batch) * z.heads * chunk_layout(z.Dk, z.Vp).total;
 }
 
+template <int D, int WAVES> static int launch_chunk_w(hipStream_t st, const DeltaArgs &a) {
+  constexpr size_t lds = chunk_lds_floats<D>() * sizeof(float);
+  static_assert(lds <= 160 * 1024 && (D > 128 || lds <= 80 * 1024), "a chunk's keys and sums fit LDS");
+  static bool attr_set = false;
+  if (lds > 64 * 1024 && !attr_set) {
+    RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_delta_chunk<D, WAVES>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    attr_set = true;
+  }
+  hipLaunchKernelGGL((k_delta_chunk<D, WAVES>), dim3((a.S + C - 1) / C, a.s.heads, a.B), dim3(WAVES * 64), lds, st, a);
+  return launch_check("delta_chunk");
+}
 template <int D> static int launch_chunks(hipStream_t st, const DeltaArgs &a) {
   const DeltaShape &z = a.s;
-  hipLaunchKernelGGL(k_delta_chunk<D>, dim3((a.S + C - 1) / C, z.heads, a.B), dim3(256), 0, st, a);
-  RAI_TRY(launch_check("delta_chunk"));
-  hipLaunchKernelGGL(k_delta_pass<D>, dim3(z.Vp / 32, z.heads, a.B), dim3(256), 0, st, a);
+  const int64_t heads = (int64_t)z.heads * a.B;
+  if (D > 128 || heads * ((a.S + C - 1) / C) <= kNumCU) RAI_TRY((launch_chunk_w<D, 8>(st, a)));
+  else RAI_TRY((launch_chunk_w<D, (D > 128 ? 8 : 4)>(st, a)));
+  // 64 columns a block read the operands half as often, 32 make twice as many blocks
+  if (D <= 128 && z.Vp % 64 == 0 && heads * (z.Vp / 32) > 2 * kNumCU)
+    hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4)>), dim3(z.Vp / 64, z.heads, a.B), dim3(256), 0, st, a);
+  else
+    hipLaunchKernelGGL((k_delta_pass<D, 2>), dim3(z.Vp / 32, z.heads, a.B), dim3(256), 0, st, a);
   return launch_check("delta_pass");
 }
 int launch_delta_chunks(hipStream_t st, const DeltaArgs &a) {
