@@ -226,7 +226,8 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
     RAI_TRY(zalloc(d, rows * val * es, &hm.v));
     if (chunk) RAI_TRY(zalloc(d, chunk, &hm.chunk_ws));
     RAI_TRY(floats(beta, &hm.beta));
-    RAI_TRY(floats(val, &hm.o));
+    RAI_TRY(zalloc(d, (rows + 1) * val * sizeof(float), &tmp));
+    hm.o = (float *)tmp;
     RAI_TRY(zalloc(d, rows * val * es, &hm.gate));
   }
   if (ws) {

@@ -32,7 +32,7 @@ struct DeltaArgs {
                                // running sum from the start of each chunk of kDeltaChunk tokens of this call
   float *q, *k, *beta;         // [rows, kv_heads Dk] twice, [rows, heads]
   void *v;                     // [rows, heads Vp] of the model dtype
-  float *o;                    // [rows, heads Vp]
+  float *o;                    // [rows + 1, heads Vp], the last row is scratch
   const void *norm_w;          // [Vp]
   float eps;
   const void *gate;            // [rows, heads Vp], before its sigmoid

@@ -152,7 +152,7 @@ __device__ __forceinline__ float fast_silu(float y) { return y * __builtin_amdgc
 // The bf16 form for four taps and key heads of 32, 64, 128, 256 or 512 channels: a thread takes eight channels over
 // kWideTokens tokens, Dk / 8 neighbouring lanes a head.
 constexpr int kWideTokens = 4;
-__global__ void __launch_bounds__(256) k_delta_prep_wide(DeltaArgs a) {
+__global__ void __launch_bounds__(256, 4) k_delta_prep_wide(DeltaArgs a) {
   struct alignas(16) P8 { uint16_t v[8]; };
   const DeltaShape &z = a.s;
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8, b = blockIdx.z, s0 = blockIdx.y * kWideTokens;
@@ -207,7 +207,7 @@ template <typename T> __device__ __forceinline__ float softplus_for(float z) {
 }
 
 // A thread takes one channel of one head over a chunk of tokens; the head's first threads also form the step sizes.
-constexpr int kDecayRun = 16;
+constexpr int kDecayRun = 32;
 template <typename T>
 __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   const DeltaShape &z = a.s;

@@ -89,7 +89,8 @@ __device__ __forceinline__ Halves split_pair(const dc_f32x4 &a, const dc_f32x4 &
 constexpr int kLP = 20;   // pitch of a 16 x 16 block in LDS (floats)
 template <int D> constexpr int chunk_lds_floats() { return 2 * C * (D + 4) + 10 * 16 * kLP + C; }   // D = 128: two blocks to a CU
 
-// WAVES = 8 for few chunks, 4 (two blocks to a CU) for many.
+// WAVES = 8 for few chunks, 4 (two blocks to a CU) for many.  Both kernels have the heads in the grid's fastest dimension:
+// blocks go round the eight XCDs, so what a head's chunks leave is read through the same L2 if heads are a multiple of 8.
 template <int D, int WAVES>
 __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
   constexpr int KS = D / 32, KP = D + 4, kChunkWaves = WAVES, kChunkThreads = WAVES * 64;
@@ -101,14 +102,14 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
   const DeltaShape &z = a.s;
   const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int n = blockIdx.x, h = blockIdx.y, b = blockIdx.z, kv = h / (z.heads / z.kv_heads);
+  const int h = blockIdx.x, n = blockIdx.y, b = blockIdx.z, kv = h / (z.heads / z.kv_heads);
   const int len = a.S - n * C < C ? a.S - n * C : C;
   const int64_t row0 = (int64_t)b * a.S + n * C;
   const int64_t ldk = (int64_t)z.kv_heads * D, ldg = (int64_t)z.heads * D, ldv = (int64_t)z.heads * z.Vp;
   const float *q = a.q + row0 * ldk + kv * D, *k = a.k + row0 * ldk + kv * D, *G = a.decay + row0 * ldg + h * D;
   const bf16_raw *v = (const bf16_raw *)a.v + row0 * ldv + h * z.Vp;
   const ChunkLayout lay = chunk_layout(D, z.Vp);
-  char *ws = a.chunk_ws + (((int64_t)b * gridDim.x + n) * z.heads + h) * lay.total;
+  char *ws = a.chunk_ws + (((int64_t)b * gridDim.y + n) * z.heads + h) * lay.total;
   // queries of row t, a step's terms
   auto query = [&](int t, int ks, float (&x)[8]) {
     if (t < len) load_pair(q + (int64_t)t * ldk + 32 * ks + 4 * lq, x);
@@ -144,7 +145,6 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
     for (int ks = 0; ks < KS; ++ks) {
       const int d = 32 * ks + 4 * lq;
       float R[8], kt[8], gt[8], kb[8], gs[8], qx[8];
-      if (idx >= kChunkWaves) query(t, ks, qt[ks]);
       load_pair(Kl + t * KP + d, kt);
       load_pair(Gl + t * KP + d, gt);
       load_pair(Kl + s * KP + d, kb);
@@ -167,6 +167,13 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
         qx[y] = qt[ks][y] * e;
         kb[y] *= fast_exp(R[y] - gs[y]);
       }
+      if (i == j) {   // the scaled queries of this row block, on the way
+        float x[8];
+#pragma unroll
+        for (int y = 0; y < 8; ++y) x[y] = qt[ks][y] * fast_exp(gt[y]);
+        *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + ((i * KS + ks) * 64 + lane) * 16) = round8(x);
+      }
+      if (idx + kChunkWaves < 10) query(16 * block_row(idx + kChunkWaves) + l16, ks, qt[ks]);   // for the next block
       const Halves kB = split8(kb);
       A = mma3(split8(kt), kB, A);
       P = mma(kB.hi, round8(qx), P);
@@ -203,6 +210,21 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
     *reinterpret_cast<dc_u32x2 *>(ws + lay.p + ((i * 2 + i / 2) * 64 + lane) * 16 + 8) = dc_u32x2{0u, 0u};
   }
   __syncthreads();
+  // values of the first pair of column tiles, ahead of their use
+  const int vp = z.Vp / 32;
+  uint16_t vr[2][4][4];
+  auto values = [&](int pair) {
+#pragma unroll
+    for (int e = 0; e < 2; ++e)
+#pragma unroll
+      for (int ib = 0; ib < 4; ++ib)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 16 * ib + 4 * lq + r;
+          vr[e][ib][r] = v[(int64_t)(t < len ? t : len - 1) * ldv + pair * 32 + 16 * e + l16].bits;
+        }
+  };
+  if (wave < vp) values(wave);
   // ---- operand of the state's update: k_s exp(G_C - G_s), rows d
   auto update_operand = [&](int f) {
     const int dt = f >> 1, ks = f & 1, d = 16 * dt + l16;
@@ -239,16 +261,6 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
   } else {
     for (int f = wave - 4; f < D / 8; f += 4) update_operand(f);
   }
-  // ---- scaled queries
-  for (int f = wave; f < 4 * KS; f += kChunkWaves) {
-    const int t = 16 * (f / KS) + l16, ks = f % KS;
-    float x[8], g[8];
-    query(t, ks, x);
-    load_pair(Gl + t * KP + 32 * ks + 4 * lq, g);
-#pragma unroll
-    for (int y = 0; y < 8; ++y) x[y] *= fast_exp(g[y]);
-    *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + (f * 64 + lane) * 16) = round8(x);
-  }
   __syncthreads();
   // ---- (1 + L) X = beta [V | K~], two tiles of 16 columns at a time
   Halves Lf[4], Nf[4], one;   // L of block rows 1, 2, 3 (first two blocks) and 3 (third), the inverses, the unit matrix
@@ -277,10 +289,10 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
     for (int y = 0; y < 8; ++y) x[y] = y < 4 && 4 * lq + y == l16 ? 1.f : 0.f;
     one.hi = round8(x);
   }
-  const int vp = z.Vp / 32;
   const dc_f32x4 zero = {0.f, 0.f, 0.f, 0.f};
   for (int pair = wave; pair < vp + KS; pair += kChunkWaves) {
     const bool val = pair < vp;
+    if (val && pair >= kChunkWaves) values(pair);
     const int c0 = (val ? pair : pair - vp) * 32 + l16;
     dc_f32x4 X[2][4];
 #pragma unroll
@@ -290,7 +302,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int t = 16 * ib + 4 * lq + r, c = c0 + 16 * e;
-          X[e][ib][r] = bs[t] * (val ? bf16_bits_to_f32(v[(int64_t)(t < len ? t : len - 1) * ldv + c].bits) : Kl[t * KP + c] * fast_exp(Gl[t * KP + c]));
+          X[e][ib][r] = bs[t] * (val ? bf16_bits_to_f32(vr[e][ib][r]) : Kl[t * KP + c] * fast_exp(Gl[t * KP + c]));
         }
     Halves first[2];   // solved blocks 0 and 1
 #pragma unroll
@@ -331,9 +343,10 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
 }
 
 // Block = (16 EB columns e of the state, head, sequence).  Wave w owns rows 16 w .. + 15 of a chunk in the products over
-// the state, and channels w D / 4 .. of the state itself, transposed: rows e, columns d.  State and U pass through LDS as
+// the state, and channels w D / 4 .. of the state itself: rows d, columns e.  State and U pass through LDS as
 // operands, their terms stored in paired order.  The operands of either half of a chunk are requested as soon as the
-// ones before them have been used.
+// ones before them have been used; every load and store of the loop is unconditional (rows past the end go to a row
+// behind the last), so that the compiler can count them and wait for no more than it needs.
 __device__ __forceinline__ int paired(int term) { return (term & ~31) | ((term & 12) << 1) | ((term & 16) >> 2) | (term & 3); }
 template <int D, int EB>
 __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
@@ -343,26 +356,24 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
   const DeltaShape &z = a.s;
   const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int e0 = blockIdx.x * 16 * EB, h = blockIdx.y, b = blockIdx.z;
+  const int h = blockIdx.x, e0 = blockIdx.y * 16 * EB, b = blockIdx.z;
   const int chunks = (a.S + C - 1) / C, vt = z.Vp / 16;
   const ChunkLayout lay = chunk_layout(D, z.Vp);
   const int pos0 = a.state->pos;
   const char *ws0 = a.chunk_ws + ((int64_t)b * chunks * z.heads + h) * lay.total;
   const int64_t step = (int64_t)z.heads * lay.total, ldg = (int64_t)z.heads * D;
   const float *G = a.decay + (int64_t)b * a.S * ldg + h * D;
-  float *carried = a.carried + ((int64_t)b * z.heads + h) * D * z.Vp + e0;
+  float *const carried = a.carried + ((int64_t)b * z.heads + h) * D * z.Vp + e0;
   dc_f32x4 S[DT][EB];
+  auto state_at = [&](int dt, int e, int r) { return carried + (int64_t)((wave * DT + dt) * 16 + 4 * lq + r) * z.Vp + 16 * e + l16; };
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-    for (int e = 0; e < EB; ++e) {
-      const int d = (wave * DT + dt) * 16 + l16;
-      S[dt][e] = dc_f32x4{0.f, 0.f, 0.f, 0.f};
-      if (pos0 > 0) S[dt][e] = *reinterpret_cast<const dc_f32x4 *>(carried + (int64_t)d * z.Vp + 16 * e + 4 * lq);
-    }
+    for (int e = 0; e < EB; ++e)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[dt][e][r] = pos0 > 0 ? *state_at(dt, e, r) : 0.f;
   dc_bf16x8 wh[KS], wl[KS], q[KS], p[2], kh[DT][2], kl[DT][2];
-  dc_f32x4 u[EB];
-  float g[DT];
+  dc_f32x4 u[EB], g[DT];
   auto request_first = [&](int n) {
     const char *ws = ws0 + n * step;
 #pragma unroll
@@ -380,7 +391,7 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
     const int last = (n + 1) * C < a.S ? (n + 1) * C - 1 : a.S - 1;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      g[dt] = G[(int64_t)last * ldg + (wave * DT + dt) * 16 + l16];
+      g[dt] = *reinterpret_cast<const dc_f32x4 *>(G + (int64_t)last * ldg + (wave * DT + dt) * 16 + 4 * lq);
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         const char *src = ws + lay.k + (((wave * DT + dt) * 2 + ks) * 2 * 64 + lane) * 16;
@@ -389,25 +400,23 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
       }
     }
     p[0] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + (wave * 2 * 64 + lane) * 16);
-    if (wave >= 2) p[1] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + 1) * 64 + lane) * 16);
+    p[1] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + 1) * 64 + lane) * 16);
+  };
+  // four consecutive terms of one column, hi and lo
+  auto put = [&](auto &dst, int at, const dc_f32x4 &y) {
+    const dc_u32x2 hi = {pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+    const dc_u32x2 lo = {pack_bf16x2(y[0] - bf_lo(hi.x), y[1] - bf_hi(hi.x)), pack_bf16x2(y[2] - bf_lo(hi.y), y[3] - bf_hi(hi.y))};
+    *reinterpret_cast<dc_u32x2 *>(dst[0] + at) = hi;
+    *reinterpret_cast<dc_u32x2 *>(dst[1] + at) = lo;
   };
   request_first(0);
   request_second(0);
   for (int n = 0; n < chunks; ++n) {
     // ---- the state as an operand
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      const int pd = paired((wave * DT + dt) * 16 + l16);
+    for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-      for (int e = 0; e < EB; ++e)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int at = (16 * e + 4 * lq + r) * SP + pd;
-          const uint16_t hi = f32_to_bf16_bits(S[dt][e][r]);
-          St[0][at] = hi;
-          St[1][at] = f32_to_bf16_bits(S[dt][e][r] - bf16_bits_to_f32(hi));
-        }
-    }
+      for (int e = 0; e < EB; ++e) put(St, (16 * e + l16) * SP + paired((wave * DT + dt) * 16 + 4 * lq), S[dt][e]);
     __syncthreads();
     dc_f32x4 O[EB];
 #pragma unroll
@@ -423,21 +432,18 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
         x3 = mma(wl[ks], sh, x3);
         O[e] = mma(q[ks], sh, O[e]);
       }
-      float U[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) U[r] = u[e][r] - (x[r] + (x2[r] + x3[r]));
-      const dc_u32x2 hi = {pack_bf16x2(U[0], U[1]), pack_bf16x2(U[2], U[3])};
-      const dc_u32x2 lo = {pack_bf16x2(U[0] - bf_lo(hi.x), U[1] - bf_hi(hi.x)), pack_bf16x2(U[2] - bf_lo(hi.y), U[3] - bf_hi(hi.y))};
-      const int at = (16 * e + l16) * UP + paired(16 * wave + 4 * lq);
-      *reinterpret_cast<dc_u32x2 *>(Ut[0] + at) = hi;
-      *reinterpret_cast<dc_u32x2 *>(Ut[1] + at) = lo;
+      for (int r = 0; r < 4; ++r) x[r] = u[e][r] - (x[r] + (x2[r] + x3[r]));
+      put(Ut, (16 * e + l16) * UP + paired(16 * wave + 4 * lq), x);
     }
-    if (n + 1 < chunks) request_first(n + 1);
+    request_first(n + 1 < chunks ? n + 1 : n);
     __syncthreads();
     // ---- update and read-out
-    float w[DT];
+    dc_f32x4 w[DT];
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) w[dt] = fast_exp(g[dt]);
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) w[dt][r] = fast_exp(g[dt][r]);
 #pragma unroll
     for (int e = 0; e < EB; ++e) {
       Halves ua[2];
@@ -450,32 +456,33 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[dt][e][r] *= w[dt];
+        for (int r = 0; r < 4; ++r) S[dt][e][r] *= w[dt][r];
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
           Halves kb;
           kb.hi = kh[dt][ks];
           kb.lo = kl[dt][ks];
-          S[dt][e] = mma3(ua[ks], kb, S[dt][e]);
+          S[dt][e] = mma3(kb, ua[ks], S[dt][e]);
         }
       }
       O[e] = mma(p[0], ua[0].hi, O[e]);
       if (wave >= 2) O[e] = mma(p[1], ua[1].hi, O[e]);
     }
-    if (n + 1 < chunks) request_second(n + 1);
+    request_second(n + 1 < chunks ? n + 1 : n);
     const int t0 = n * C + 16 * wave + 4 * lq;
 #pragma unroll
     for (int e = 0; e < EB; ++e)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (t0 + r < a.S) a.o[(((int64_t)b * a.S + t0 + r) * z.heads + h) * z.Vp + e0 + 16 * e + l16] = O[e][r];
+        a.o[((t0 + r < a.S ? (int64_t)b * a.S + t0 + r : (int64_t)a.B * a.S) * z.heads + h) * z.Vp + e0 + 16 * e + l16] = O[e][r];
   }
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
     for (int e = 0; e < EB; ++e)
-      *reinterpret_cast<dc_f32x4 *>(carried + (int64_t)((wave * DT + dt) * 16 + l16) * z.Vp + 16 * e + 4 * lq) = S[dt][e];
-  if (blockIdx.x == 0) update_ring<bf16_raw>(a, b, h, pos0, tid, 256);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) *state_at(dt, e, r) = S[dt][e][r];
+  if (blockIdx.y == 0) update_ring<bf16_raw>(a, b, h, pos0, tid, 256);
 }
 
 bool delta_chunk_serves(int dtype, const DeltaShape &z) {
@@ -493,7 +500,7 @@ template <int D, int WAVES> static int launch_chunk_w(hipStream_t st, const Delt
     RAI_HIP_TRY(hipFuncSetAttribute((const void *)k_delta_chunk<D, WAVES>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     attr_set = true;
   }
-  hipLaunchKernelGGL((k_delta_chunk<D, WAVES>), dim3((a.S + C - 1) / C, a.s.heads, a.B), dim3(WAVES * 64), lds, st, a);
+  hipLaunchKernelGGL((k_delta_chunk<D, WAVES>), dim3(a.s.heads, (a.S + C - 1) / C, a.B), dim3(WAVES * 64), lds, st, a);
   return launch_check("delta_chunk");
 }
 template <int D> static int launch_chunks(hipStream_t st, const DeltaArgs &a) {
@@ -503,9 +510,9 @@ template <int D> static int launch_chunks(hipStream_t st, const DeltaArgs &a) {
   else RAI_TRY((launch_chunk_w<D, (D > 128 ? 8 : 4)>(st, a)));
   // 64 columns a block read the operands half as often, 32 make twice as many blocks
   if (D <= 128 && z.Vp % 64 == 0 && heads * (z.Vp / 32) > 2 * kNumCU)
-    hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4)>), dim3(z.Vp / 64, z.heads, a.B), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4)>), dim3(z.heads, z.Vp / 64, a.B), dim3(256), 0, st, a);
   else
-    hipLaunchKernelGGL((k_delta_pass<D, 2>), dim3(z.Vp / 32, z.heads, a.B), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((k_delta_pass<D, 2>), dim3(z.heads, z.Vp / 32, a.B), dim3(256), 0, st, a);
   return launch_check("delta_pass");
 }
 int launch_delta_chunks(hipStream_t st, const DeltaArgs &a) {
