@@ -113,8 +113,8 @@ struct HybridModel {
   float *xs, *xs2, *x0w;       // [max_rows, Hp]: residual stream (two, swapped by the single-row step's loop entry), W0 x0
   float *stream;               // the one the last forward finished in
   char *h1, *dn, *cat;
-  float *decay, *q, *k, *beta, *o;   // delta rule, see DeltaArgs
-  char *v, *gate, *chunk_ws;
+  float *decay, *qn, *kn, *beta, *o;   // delta rule, see DeltaArgs
+  char *dq, *dk, *dv, *gate, *chunk_ws;
   char *attn_ws;
   int *attn_counters;
   bool derived_ready;          // a padded copy of the embedding table serves as the head

@@ -187,7 +187,7 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
   // activations, sized for the widest layer
   const int64_t rows = d->max_rows;
   int ldn = 0, KB = 0;
-  size_t decay = 0, qk = 0, val = 0, beta = 0, ws = 0, counters = 0, chunk = 0;
+  size_t decay = 0, qk = 0, kvh = 0, val = 0, beta = 0, ws = 0, counters = 0, chunk = 0;
   for (const HybridLayer &y : hm.layers) {
     ldn = std::max(ldn, y.ldn);
     KB = std::max(KB, y.QD + y.Fp);
@@ -198,6 +198,7 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
       const DeltaShape &z = y.delta;
       decay = std::max(decay, (size_t)z.heads * z.Dk);
       qk = std::max(qk, (size_t)z.kv_heads * z.Dk);
+      kvh = std::max(kvh, (size_t)z.kv_heads);
       val = std::max(val, (size_t)z.heads * z.Vp);
       if (delta_chunk_serves(cfg.dtype, z)) chunk = std::max(chunk, delta_chunk_ws_bytes(z, cfg.max_batch, rows));
       beta = std::max(beta, (size_t)z.heads);
@@ -221,9 +222,11 @@ static int create_hybrid(rai_hip_decoder *d, const rai_hip_hybrid_config &cfg, c
   RAI_TRY(zalloc(d, (size_t)cfg.max_batch * Hp * es, &d->last));
   if (val) {
     RAI_TRY(floats(decay, &hm.decay));
-    RAI_TRY(floats(qk, &hm.q));
-    RAI_TRY(floats(qk, &hm.k));
-    RAI_TRY(zalloc(d, rows * val * es, &hm.v));
+    RAI_TRY(zalloc(d, rows * qk * es, &hm.dq));
+    RAI_TRY(zalloc(d, rows * qk * es, &hm.dk));
+    RAI_TRY(floats(kvh, &hm.qn));
+    RAI_TRY(floats(kvh, &hm.kn));
+    RAI_TRY(zalloc(d, rows * val * es, &hm.dv));
     if (chunk) RAI_TRY(zalloc(d, chunk, &hm.chunk_ws));
     RAI_TRY(floats(beta, &hm.beta));
     RAI_TRY(zalloc(d, (rows + 1) * val * sizeof(float), &tmp));
@@ -358,7 +361,7 @@ static DeltaArgs delta_args(rai_hip_decoder *d, const HybridLayer &y, const Hybr
   a.s = y.delta; a.B = B; a.S = S; a.state = d->state;
   a.dn = hm.dn; a.conv = y.conv; a.ring = r.ring; a.carried = r.carried;
   a.A_log = y.A_log; a.dt_bias = y.dt_bias;
-  a.decay = hm.decay; a.q = hm.q; a.k = hm.k; a.v = hm.v; a.beta = hm.beta; a.o = hm.o;
+  a.decay = hm.decay; a.q = hm.dq; a.k = hm.dk; a.qn = hm.qn; a.kn = hm.kn; a.v = hm.dv; a.beta = hm.beta; a.o = hm.o;
   a.norm_w = y.norm_w; a.eps = (float)hm.c.norm_eps;
   a.gate = hm.gate;
   a.chunk_ws = hm.chunk_ws;

@@ -28,9 +28,10 @@ struct DeltaArgs {
   void *ring;                  // [B][taps][channels]: the inputs of the last `taps` positions, position p at p mod taps
   float *carried;              // [B][heads][Dk][Vp]
   const void *A_log, *dt_bias; // [heads], [heads Dk]
-  float *decay;                // [rows, heads Dk]: in: the low-rank factor's output; after the preparation log g, or its
-                               // running sum from the start of each chunk of kDeltaChunk tokens of this call
-  float *q, *k, *beta;         // [rows, kv_heads Dk] twice, [rows, heads]
+  float *decay;                // [rows, heads Dk]: the low-rank factor's output (k_delta_decay makes it log g in place)
+  void *q, *k;                 // [rows, kv_heads Dk] of the model dtype, after convolution and silu
+  float *qn, *kn;              // [rows, kv_heads]: what makes each a unit vector (queries: times dim^-1/2)
+  float *beta;                 // [rows, heads]
   void *v;                     // [rows, heads Vp] of the model dtype
   float *o;                    // [rows + 1, heads Vp], the last row is scratch
   const void *norm_w;          // [Vp]
@@ -43,7 +44,6 @@ struct DeltaArgs {
   const void *a2, *g2;         // [heads Dk, a_rank], [heads Vp, g_rank]
   int a_rank, g_rank;
   char *chunk_ws;              // delta_chunk_ws_bytes(); null: the chunked form is not used
-  int chunked;                 // filled in by the launcher
 };
 // The chunked form (bf16 models): see delta_chunk.hip.
 constexpr int kDeltaChunk = 64;

@@ -1,6 +1,6 @@
 // Gated delta rule with a decay per key channel (see delta.h).
-//   k_delta_prep  convolution + silu, unit vectors of every token
-//   k_delta_decay decays and step sizes
+//   k_delta_prep  convolution + silu of every token, and what makes its queries and keys unit vectors
+//   k_delta_decay decays and step sizes, for k_delta_scan (the chunks form their own)
 //   k_delta_scan  the recurrence, token after token: a block owns 16 columns of one head's state, 16 lanes to a column
 //                 (f32 models, few tokens, head sizes the chunked form of delta_chunk.hip does not serve)
 //   k_delta_out   norm over the head's values, weight and output gate
@@ -44,6 +44,12 @@ template <typename T> struct alignas(2 * sizeof(T)) Pair { T v[2]; };
 template <typename T> __device__ __forceinline__ float2 ld2(const void *p, int64_t i) {
   const Pair<T> x = *reinterpret_cast<const Pair<T> *>((const T *)p + i);
   return make_float2((float)Scalar<T>::load(&x.v[0]), (float)Scalar<T>::load(&x.v[1]));
+}
+
+template <typename T> __device__ __forceinline__ float as_stored(float x) {
+  T t;
+  Scalar<T>::store(&t, x);
+  return (float)Scalar<T>::load(&t);
 }
 
 // Channels c, c + 1 (c even) of kPrepTokens tokens from s0 on, after convolution and silu; TAPS == 0: any number of taps.
@@ -124,19 +130,26 @@ __global__ void __launch_bounds__(256) k_delta_prep(DeltaArgs a) {
   for (int t = 0; t < kPrepTokens; ++t) {
     sum[t] = 0.f;
 #pragma unroll
-    for (int i = 0; i < NI; ++i) sum[t] = fmaf(y[i][t].x, y[i][t].x, fmaf(y[i][t].y, y[i][t].y, sum[t]));
+    for (int i = 0; i < NI; ++i) {
+      const float u = as_stored<T>(y[i][t].x), w = as_stored<T>(y[i][t].y);
+      sum[t] = fmaf(u, u, fmaf(w, w, sum[t]));
+    }
   }
 #pragma unroll
   for (int t = 0; t < kPrepTokens; ++t) sum[t] = wave_sum(sum[t]);
-  float *dst = (query ? a.q : a.k) + h * z.Dk;
+  T *dst = (T *)(query ? a.q : a.k) + h * z.Dk;
   const float mul = query ? 1.0f / sqrtf((float)z.dim) : 1.0f;
 #pragma unroll
   for (int t = 0; t < kPrepTokens; ++t) {
-    const float r = mul / sqrtf(sum[t] + 1e-6f);
+    if (s0 + t >= a.S) break;
+    if (lane == 0) (query ? a.qn : a.kn)[(row0 + t) * z.kv_heads + h] = mul / sqrtf(sum[t] + 1e-6f);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = 2 * lane + 128 * i;
-      if (s0 + t < a.S && c < width) *reinterpret_cast<float2 *>(dst + (row0 + t) * z.kv_heads * z.Dk + c) = make_float2(y[i][t].x * r, y[i][t].y * r);
+      Pair<T> o;
+      Scalar<T>::store(&o.v[0], y[i][t].x);
+      Scalar<T>::store(&o.v[1], y[i][t].y);
+      if (c < width) *reinterpret_cast<Pair<T> *>(dst + (row0 + t) * z.kv_heads * z.Dk + c) = o;
     }
   }
 }
@@ -152,7 +165,7 @@ __device__ __forceinline__ float fast_silu(float y) { return y * __builtin_amdgc
 // The bf16 form for four taps and key heads of 32, 64, 128, 256 or 512 channels: a thread takes eight channels over
 // kWideTokens tokens, Dk / 8 neighbouring lanes a head.
 constexpr int kWideTokens = 4;
-__global__ void __launch_bounds__(256, 4) k_delta_prep_wide(DeltaArgs a) {
+__global__ void __launch_bounds__(256) k_delta_prep_wide(DeltaArgs a) {
   struct alignas(16) P8 { uint16_t v[8]; };
   const DeltaShape &z = a.s;
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8, b = blockIdx.z, s0 = blockIdx.y * kWideTokens;
@@ -169,10 +182,14 @@ __global__ void __launch_bounds__(256, 4) k_delta_prep_wide(DeltaArgs a) {
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) w[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.conv + (int64_t)c * 4 + 8 * i);
-  const bool qk = c < 2 * kd;
-  const float mul = c < kd ? 1.0f / sqrtf((float)z.dim) : 1.0f;
+  const bool query = c < kd, key = !query && c < 2 * kd;
+  const int Dk = z.Dk, unit = c / Dk;
+  uint16_t *dst = query ? (uint16_t *)a.q + c : key ? (uint16_t *)a.k + c - kd : (uint16_t *)a.v + c - 2 * kd;
+  const int64_t ldd = query || key ? kd : z.heads * z.Vp;
+  const float mul = query ? 1.0f / sqrtf((float)z.dim) : 1.0f;
 #pragma unroll
   for (int t = 0; t < kWideTokens; ++t) {
+    const int64_t row = (int64_t)b * a.S + s0 + t;
     float y[8], sum = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
@@ -180,34 +197,24 @@ __global__ void __launch_bounds__(256, 4) k_delta_prep_wide(DeltaArgs a) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) v = fmaf(bf16_bits_to_f32(x[t + j].v[e]), bf16_bits_to_f32(w[e >> 1].v[4 * (e & 1) + j]), v);
       y[e] = fast_silu(v);
-      sum = fmaf(y[e], y[e], sum);
     }
-    const int64_t row = (int64_t)b * a.S + s0 + t;
-    if (qk) {
-      const float r = mul / sqrtf(group_sum(sum, z.Dk / 8) + 1e-6f);
-      if (s0 + t < a.S) {
-        float4 *dst = reinterpret_cast<float4 *>((c < kd ? a.q + c : a.k + c - kd) + row * kd);
-        dst[0] = make_float4(y[0] * r, y[1] * r, y[2] * r, y[3] * r);
-        dst[1] = make_float4(y[4] * r, y[5] * r, y[6] * r, y[7] * r);
-      }
-    } else if (s0 + t < a.S) {
-      *reinterpret_cast<uint4 *>((uint16_t *)a.v + row * z.heads * z.Vp + c - 2 * kd) =
-          make_uint4(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]), pack_bf16x2(y[4], y[5]), pack_bf16x2(y[6], y[7]));
+    uint32_t o[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      o[e] = pack_bf16x2(y[2 * e], y[2 * e + 1]);
+      const float u = __uint_as_float(o[e] << 16), p = __uint_as_float(o[e] & 0xffff0000u);
+      sum = fmaf(u, u, fmaf(p, p, sum));
+    }
+    if (s0 + t < a.S) *reinterpret_cast<uint4 *>(dst + row * ldd) = make_uint4(o[0], o[1], o[2], o[3]);
+    if (query || key) {
+      sum = group_sum(sum, Dk / 8);
+      if (c % Dk == 0 && s0 + t < a.S) (query ? a.qn : a.kn)[row * z.kv_heads + (query ? unit : unit - z.kv_heads)] = mul / sqrtf(sum + 1e-6f);
     }
   }
 }
 
-// log(1 + exp(z)); for results that meet bf16 operands through the hardware's exp2 and log2 and a short series where the
-// logarithm's argument is close to 1 (relative error below 1e-6).
-template <typename T> __device__ __forceinline__ float softplus_for(float z) {
-  if constexpr (sizeof(T) == 4) return dl_softplus(z);
-  const float x = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z));
-  const float series = x * (1.f - x * (0.5f - x * (0.33333333f - x * (0.25f - x * 0.2f))));
-  return fmaxf(z, 0.f) + (x < 0.06f ? series : 0.69314718056f * __builtin_amdgcn_logf(1.f + x));
-}
-
 // A thread takes one channel of one head over a chunk of tokens; the head's first threads also form the step sizes.
-constexpr int kDecayRun = 32;
+constexpr int kDecayRun = 8;
 template <typename T>
 __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   const DeltaShape &z = a.s;
@@ -215,7 +222,6 @@ __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
   if (c >= z.heads * z.Dk) return;
   const int h = c / z.Dk, s1 = s0 + kDeltaChunk < a.S ? s0 + kDeltaChunk : a.S;
   const float rate = -expf(ld<T>(a.A_log, h)), bias = ld<T>(a.dt_bias, c);
-  float run = 0.f;
   for (int s = s0; s < s1; s += kDecayRun) {
     float x[kDecayRun];
 #pragma unroll
@@ -224,8 +230,7 @@ __global__ void __launch_bounds__(256) k_delta_decay(DeltaArgs a) {
     for (int j = 0; j < kDecayRun; ++j)
       if (s + j < s1) {
         const float g = rate * softplus_for<T>(x[j] + bias);
-        run = a.chunked ? run + g : g;
-        a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] = run;
+        a.decay[((int64_t)b * a.S + s + j) * z.heads * z.Dk + c] = g;
       }
   }
   for (int s = s0 + c % z.Dk; s < s1; s += z.Dk) a.beta[((int64_t)b * a.S + s) * z.heads + h] = dl_sigmoid(ld<T>(a.dn, ((int64_t)b * a.S + s) * z.ldn + z.off_b + h));
@@ -257,8 +262,9 @@ __global__ void __launch_bounds__(256) k_delta_scan(DeltaArgs a) {
     for (int e = tid; e < n * R; e += 256) {
       const int t = e / R, r = e - t * R;
       const bool in = r < z.Dk;
-      qs[e] = in ? a.q[((row0 + t) * z.kv_heads + kv) * z.Dk + r] : 0.f;
-      ks[e] = in ? a.k[((row0 + t) * z.kv_heads + kv) * z.Dk + r] : 0.f;
+      const int64_t at = (row0 + t) * z.kv_heads + kv;
+      qs[e] = in ? ld<T>(a.q, at * z.Dk + r) * a.qn[at] : 0.f;
+      ks[e] = in ? ld<T>(a.k, at * z.Dk + r) * a.kn[at] : 0.f;
       gs[e] = in ? expf(a.decay[((row0 + t) * z.heads + h) * z.Dk + r]) : 0.f;
     }
     if (tid < n * 16) vs[tid] = ld<T>(a.v, ((row0 + (tid >> 4)) * z.heads + h) * z.Vp + blockIdx.x * 16 + (tid & 15));
@@ -494,11 +500,11 @@ template <typename T, int NI> static int launch_prep(hipStream_t st, const Delta
   return launch_check("delta_prep");
 }
 
-template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, DeltaArgs a) {
+template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, const DeltaArgs &a) {
   const DeltaShape &z = a.s;
   const int wide = z.Dk > z.Vp ? z.Dk : z.Vp;
   const char *off = getenv("RAI_HIP_NO_DELTA_CHUNK");   // read per call: the tests compare both forms in one process
-  a.chunked = a.chunk_ws && a.S >= kChunkedFrom && delta_chunk_serves(dtype, z) && !(off && *off && *off != '0');
+  const bool chunked = a.chunk_ws && a.S >= kChunkedFrom && delta_chunk_serves(dtype, z) && !(off && *off && *off != '0');
   const int64_t outs = (int64_t)a.B * a.S * z.heads;
   RAI_REQUIRE((outs + 3) / 4 < (1ll << 31) && (a.S + kDeltaChunk - 1) / kDeltaChunk <= 65535, RAI_ERR_UNSUPPORTED, "delta rule: too many tokens");
   const dim3 go((unsigned)((outs + 3) / 4)), block(256);
@@ -510,9 +516,11 @@ template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, Delt
   } else if (wide <= 128) RAI_TRY((launch_prep<T, 1>(st, a)));
   else if (wide <= 256) RAI_TRY((launch_prep<T, 2>(st, a)));
   else RAI_TRY((launch_prep<T, 4>(st, a)));
-  hipLaunchKernelGGL(k_delta_decay<T>, dim3((z.heads * z.Dk + 255) / 256, (a.S + kDeltaChunk - 1) / kDeltaChunk, a.B), block, 0, st, a);
-  RAI_TRY(launch_check("delta_decay"));
-  if (a.chunked) RAI_TRY(launch_delta_chunks(st, a));
+  if (!chunked) {
+    hipLaunchKernelGGL(k_delta_decay<T>, dim3((z.heads * z.Dk + 255) / 256, (a.S + kDeltaChunk - 1) / kDeltaChunk, a.B), block, 0, st, a);
+    RAI_TRY(launch_check("delta_decay"));
+  }
+  if (chunked) RAI_TRY(launch_delta_chunks(st, a));
   else if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
   else if (z.Dk <= 64) RAI_TRY((launch_scan<T, 4>(st, a)));
   else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));

@@ -58,7 +58,7 @@ __device__ __forceinline__ dc_bf16x8 zero8() { return __builtin_bit_cast(dc_bf16
 constexpr int C = kDeltaChunk;
 // One (sequence, chunk, head)'s part of the workspace, in bytes.
 struct ChunkLayout {
-  int w, q, k, p, u, total;
+  int w, q, k, p, u, g, total;
 };
 __host__ __device__ inline ChunkLayout chunk_layout(int D, int E) {
   ChunkLayout l;
@@ -67,7 +67,8 @@ __host__ __device__ inline ChunkLayout chunk_layout(int D, int E) {
   l.k = l.q + C * D * 2;        // [D / 16][2 steps of 32 tokens][hi, lo][64][8]    rows d, terms t
   l.p = l.k + C * D * 4;        // [4][2][64][8]                                    rows t, terms s (step 1 of blocks 0, 1 unused)
   l.u = l.p + C * C * 2;        // [4][E / 16][64][4] f32                           accumulator order
-  l.total = l.u + C * E * 4;
+  l.g = l.u + C * E * 4;        // [D] f32: exp(G_C)
+  l.total = l.g + D * 4;
   return l;
 }
 
@@ -87,7 +88,7 @@ __device__ __forceinline__ Halves split_pair(const dc_f32x4 &a, const dc_f32x4 &
 }
 
 constexpr int kLP = 20;   // pitch of a 16 x 16 block in LDS (floats)
-template <int D> constexpr int chunk_lds_floats() { return 2 * C * (D + 4) + 10 * 16 * kLP + C; }   // D = 128: two blocks to a CU
+template <int D> constexpr int chunk_lds_floats() { return 2 * C * (D + 4) + 10 * 16 * kLP + 2 * C; }   // D = 128: two blocks to a CU
 
 // WAVES = 8 for few chunks, 4 (two blocks to a CU) for many.  Both kernels have the heads in the grid's fastest dimension:
 // blocks go round the eight XCDs, so what a head's chunks leave is read through the same L2 if heads are a multiple of 8.
@@ -98,7 +99,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
   float *Kl = dc_lds, *Gl = Kl + C * KP;      // [64][D] keys and running sums; rows past the end: 0 and the last sum
   float *Ls = Gl + C * KP;                    // blocks (i, j <= i) of beta A, strictly lower, number i (i + 1) / 2 + j; on the
                                               // diagonal later the inverses of the blocks of 1 + L
-  float *bs = Ls + 10 * 16 * kLP;
+  float *bs = Ls + 10 * 16 * kLP, *qs = bs + C;   // beta, and what makes a query a unit vector
   const DeltaShape &z = a.s;
   const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -106,34 +107,60 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
   const int len = a.S - n * C < C ? a.S - n * C : C;
   const int64_t row0 = (int64_t)b * a.S + n * C;
   const int64_t ldk = (int64_t)z.kv_heads * D, ldg = (int64_t)z.heads * D, ldv = (int64_t)z.heads * z.Vp;
-  const float *q = a.q + row0 * ldk + kv * D, *k = a.k + row0 * ldk + kv * D, *G = a.decay + row0 * ldg + h * D;
+  const uint16_t *q = (const uint16_t *)a.q + row0 * ldk + kv * D, *k = (const uint16_t *)a.k + row0 * ldk + kv * D;
   const bf16_raw *v = (const bf16_raw *)a.v + row0 * ldv + h * z.Vp;
   const ChunkLayout lay = chunk_layout(D, z.Vp);
   char *ws = a.chunk_ws + (((int64_t)b * gridDim.y + n) * z.heads + h) * lay.total;
-  // queries of row t, a step's terms
-  auto query = [&](int t, int ks, float (&x)[8]) {
-    if (t < len) load_pair(q + (int64_t)t * ldk + 32 * ks + 4 * lq, x);
-    else {
+  // queries of row t, a step's terms; scaled to unit length where they are used
+  auto query = [&](int t, int ks, dc_u32x2 (&x)[2]) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] = 0.f;
-    }
+    for (int e = 0; e < 2; ++e)
+      x[e] = t < len ? *reinterpret_cast<const dc_u32x2 *>(q + (int64_t)t * ldk + 32 * ks + 16 * e + 4 * lq) : dc_u32x2{0u, 0u};
   };
   // block (i, j) of the lower triangle number idx
   auto block_row = [](int idx) { return idx < 1 ? 0 : idx < 3 ? 1 : idx < 6 ? 2 : 3; };
 
-  float qt[KS][8];
+  dc_u32x2 qt[KS][2];
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) query(16 * block_row(wave) + l16, ks, qt[ks]);
-  for (int e = tid; e < C * D / 4; e += kChunkThreads) {
-    const int t = e / (D / 4), d = (e - t * (D / 4)) * 4;
-    const int tc = t < len ? t : len - 1;
-    dc_f32x4 kx = *reinterpret_cast<const dc_f32x4 *>(k + (int64_t)tc * ldk + d);
-    const dc_f32x4 gx = *reinterpret_cast<const dc_f32x4 *>(G + (int64_t)tc * ldg + d);
-    if (t >= len) kx = dc_f32x4{0.f, 0.f, 0.f, 0.f};
-    *reinterpret_cast<dc_f32x4 *>(Kl + t * KP + d) = kx;
-    *reinterpret_cast<dc_f32x4 *>(Gl + t * KP + d) = gx;
+  // ---- sums of the log decays: a thread takes RUN tokens of one channel, the runs' totals are then added up
+  constexpr int RUN = C * D / kChunkThreads, RUNS = C / RUN;
+  const int gd = tid % D, g0 = tid / D * RUN;
+  float gr[RUN];
+  {
+    const float rate = -expf(ld<bf16_raw>(a.A_log, h)), bias = ld<bf16_raw>(a.dt_bias, h * D + gd);
+    const float *src = a.decay + row0 * ldg + h * D + gd;
+#pragma unroll
+    for (int t = 0; t < RUN; ++t) gr[t] = src[(int64_t)(g0 + t < len ? g0 + t : len - 1) * ldg];
+    for (int e = tid; e < C * D / 8; e += kChunkThreads) {   // keys, meanwhile
+      const int t = e / (D / 8), d = (e - t * (D / 8)) * 8;
+      dc_u32x4 x = *reinterpret_cast<const dc_u32x4 *>(k + (int64_t)(t < len ? t : len - 1) * ldk + d);
+      const float r = t < len ? a.kn[(row0 + t) * z.kv_heads + kv] : 0.f;
+      *reinterpret_cast<dc_f32x4 *>(Kl + t * KP + d) = dc_f32x4{bf_lo(x[0]) * r, bf_hi(x[0]) * r, bf_lo(x[1]) * r, bf_hi(x[1]) * r};
+      *reinterpret_cast<dc_f32x4 *>(Kl + t * KP + d + 4) = dc_f32x4{bf_lo(x[2]) * r, bf_hi(x[2]) * r, bf_lo(x[3]) * r, bf_hi(x[3]) * r};
+    }
+    float run = 0.f;
+#pragma unroll
+    for (int t = 0; t < RUN; ++t) {
+      if (g0 + t < len) run += rate * softplus_for<bf16_raw>(gr[t] + bias);
+      gr[t] = run;
+    }
+    Ls[(g0 / RUN) * D + gd] = run;   // not yet used for its blocks
   }
-  if (tid < C) bs[tid] = tid < len ? a.beta[(row0 + tid) * z.heads + h] : 0.f;
+  if (tid < C) {
+    bs[tid] = tid < len ? dl_sigmoid(ld<bf16_raw>(a.dn, (row0 + tid) * z.ldn + z.off_b + h)) : 0.f;
+    qs[tid] = tid < len ? a.qn[(row0 + tid) * z.kv_heads + kv] : 0.f;
+  }
+  __syncthreads();
+  {
+    float before = 0.f;
+#pragma unroll
+    for (int r = 0; r < RUNS - 1; ++r)
+      if (r < g0 / RUN) before += Ls[r * D + gd];
+#pragma unroll
+    for (int t = 0; t < RUN; ++t) Gl[(g0 + t) * KP + gd] = gr[t] + before;
+    if (g0 + RUN == C) reinterpret_cast<float *>(ws + lay.g)[gd] = fast_exp(gr[RUN - 1] + before);
+  }
   __syncthreads();
 
   // ---- blocks of A and P
@@ -145,6 +172,8 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
     for (int ks = 0; ks < KS; ++ks) {
       const int d = 32 * ks + 4 * lq;
       float R[8], kt[8], gt[8], kb[8], gs[8], qx[8];
+#pragma unroll
+      for (int y = 0; y < 8; ++y) qx[y] = qs[t] * (y & 1 ? bf_hi(qt[ks][y >> 2][(y & 3) >> 1]) : bf_lo(qt[ks][y >> 2][(y & 3) >> 1]));
       load_pair(Kl + t * KP + d, kt);
       load_pair(Gl + t * KP + d, gt);
       load_pair(Kl + s * KP + d, kb);
@@ -160,18 +189,18 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
 #pragma unroll
         for (int y = 0; y < 8; ++y) range = fmaxf(range, R[y] - ge[y]);
       }
+      if (i == j) {   // the scaled queries of this row block, on the way
+        float x[8];
+#pragma unroll
+        for (int y = 0; y < 8; ++y) x[y] = qx[y] * fast_exp(gt[y]);
+        *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + ((i * KS + ks) * 64 + lane) * 16) = round8(x);
+      }
 #pragma unroll
       for (int y = 0; y < 8; ++y) {
         const float e = fast_exp(gt[y] - R[y]);
         kt[y] *= e;
-        qx[y] = qt[ks][y] * e;
+        qx[y] *= e;
         kb[y] *= fast_exp(R[y] - gs[y]);
-      }
-      if (i == j) {   // the scaled queries of this row block, on the way
-        float x[8];
-#pragma unroll
-        for (int y = 0; y < 8; ++y) x[y] = qt[ks][y] * fast_exp(gt[y]);
-        *reinterpret_cast<dc_bf16x8 *>(ws + lay.q + ((i * KS + ks) * 64 + lane) * 16) = round8(x);
       }
       if (idx + kChunkWaves < 10) query(16 * block_row(idx + kChunkWaves) + l16, ks, qt[ks]);   // for the next block
       const Halves kB = split8(kb);
@@ -186,7 +215,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
         for (int d = 0; d < D; ++d) {
           const float gm = Gl[(t0 + m) * KP + d], gl = Gl[t * KP + d], km = Kl[(t0 + m) * KP + d], kl = Kl[t * KP + d];
           if (l16 <= m) sa = fmaf(km * kl, fast_exp(gm - gl), sa);
-          if (m <= l16 && t < len) sp = fmaf(q[(int64_t)t * ldk + d] * km, fast_exp(gl - gm), sp);
+          if (m <= l16 && t < len) sp = fmaf(bf16_bits_to_f32(q[(int64_t)t * ldk + d]) * qs[t] * km, fast_exp(gl - gm), sp);
         }
 #pragma unroll
         for (int e = 0; e < 4; ++e)
@@ -344,12 +373,12 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
 
 // Block = (16 EB columns e of the state, head, sequence).  Wave w owns rows 16 w .. + 15 of a chunk in the products over
 // the state, and channels w D / 4 .. of the state itself: rows d, columns e.  State and U pass through LDS as
-// operands, their terms stored in paired order.  The operands of either half of a chunk are requested as soon as the
-// ones before them have been used; every load and store of the loop is unconditional (rows past the end go to a row
+// operands, their terms stored in paired order.  The operands of either half of a chunk are requested SETS chunks ahead, as
+// soon as the registers they go to have been used; every load and store of the loop is unconditional (rows past the end go to a row
 // behind the last), so that the compiler can count them and wait for no more than it needs.
 __device__ __forceinline__ int paired(int term) { return (term & ~31) | ((term & 12) << 1) | ((term & 16) >> 2) | (term & 3); }
-template <int D, int EB>
-__global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
+template <int D, int EB, int SETS>
+__global__ void __launch_bounds__(256, 1) k_delta_pass(DeltaArgs a) {
   constexpr int KS = D / 32, DT = D / 64, SP = D + 8, UP = C + 8;
   __shared__ __attribute__((aligned(16))) uint16_t St[2][16 * EB * SP];   // hi / lo of the state, [e][d]
   __shared__ __attribute__((aligned(16))) uint16_t Ut[2][16 * EB * UP];   // of U, [e][t]
@@ -361,8 +390,7 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
   const ChunkLayout lay = chunk_layout(D, z.Vp);
   const int pos0 = a.state->pos;
   const char *ws0 = a.chunk_ws + ((int64_t)b * chunks * z.heads + h) * lay.total;
-  const int64_t step = (int64_t)z.heads * lay.total, ldg = (int64_t)z.heads * D;
-  const float *G = a.decay + (int64_t)b * a.S * ldg + h * D;
+  const int64_t step = (int64_t)z.heads * lay.total;
   float *const carried = a.carried + ((int64_t)b * z.heads + h) * D * z.Vp + e0;
   dc_f32x4 S[DT][EB];
   auto state_at = [&](int dt, int e, int r) { return carried + (int64_t)((wave * DT + dt) * 16 + 4 * lq + r) * z.Vp + 16 * e + l16; };
@@ -372,35 +400,36 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
     for (int e = 0; e < EB; ++e)
 #pragma unroll
       for (int r = 0; r < 4; ++r) S[dt][e][r] = pos0 > 0 ? *state_at(dt, e, r) : 0.f;
-  dc_bf16x8 wh[KS], wl[KS], q[KS], p[2], kh[DT][2], kl[DT][2];
-  dc_f32x4 u[EB], g[DT];
-  auto request_first = [&](int n) {
-    const char *ws = ws0 + n * step;
+  struct Operands {
+    dc_bf16x8 wh[KS], wl[KS], q[KS], p[2], kh[DT][2], kl[DT][2];
+    dc_f32x4 u[EB], w[DT];
+  };
+  auto request_first = [&](int n, Operands &x) {
+    const char *ws = ws0 + (n < chunks ? n : chunks - 1) * step;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       const char *src = ws + lay.w + ((wave * KS + ks) * 2 * 64 + lane) * 16;
-      wh[ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
-      wl[ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
-      q[ks] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.q + ((wave * KS + ks) * 64 + lane) * 16);
+      x.wh[ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
+      x.wl[ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
+      x.q[ks] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.q + ((wave * KS + ks) * 64 + lane) * 16);
     }
 #pragma unroll
-    for (int e = 0; e < EB; ++e) u[e] = *reinterpret_cast<const dc_f32x4 *>(ws + lay.u + ((wave * vt + e0 / 16 + e) * 64 + lane) * 16);
+    for (int e = 0; e < EB; ++e) x.u[e] = *reinterpret_cast<const dc_f32x4 *>(ws + lay.u + ((wave * vt + e0 / 16 + e) * 64 + lane) * 16);
   };
-  auto request_second = [&](int n) {
-    const char *ws = ws0 + n * step;
-    const int last = (n + 1) * C < a.S ? (n + 1) * C - 1 : a.S - 1;
+  auto request_second = [&](int n, Operands &x) {
+    const char *ws = ws0 + (n < chunks ? n : chunks - 1) * step;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      g[dt] = *reinterpret_cast<const dc_f32x4 *>(G + (int64_t)last * ldg + (wave * DT + dt) * 16 + 4 * lq);
+      x.w[dt] = *reinterpret_cast<const dc_f32x4 *>(ws + lay.g + ((wave * DT + dt) * 16 + 4 * lq) * 4);
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         const char *src = ws + lay.k + (((wave * DT + dt) * 2 + ks) * 2 * 64 + lane) * 16;
-        kh[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
-        kl[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
+        x.kh[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src);
+        x.kl[dt][ks] = *reinterpret_cast<const dc_bf16x8 *>(src + 64 * 16);
       }
     }
-    p[0] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + (wave * 2 * 64 + lane) * 16);
-    p[1] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + 1) * 64 + lane) * 16);
+    x.p[0] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + (wave * 2 * 64 + lane) * 16);
+    x.p[1] = *reinterpret_cast<const dc_bf16x8 *>(ws + lay.p + ((wave * 2 + 1) * 64 + lane) * 16);
   };
   // four consecutive terms of one column, hi and lo
   auto put = [&](auto &dst, int at, const dc_f32x4 &y) {
@@ -409,9 +438,7 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
     *reinterpret_cast<dc_u32x2 *>(dst[0] + at) = hi;
     *reinterpret_cast<dc_u32x2 *>(dst[1] + at) = lo;
   };
-  request_first(0);
-  request_second(0);
-  for (int n = 0; n < chunks; ++n) {
+  auto chunk = [&](int n, Operands &c) __attribute__((always_inline)) {
     // ---- the state as an operand
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
@@ -427,23 +454,18 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
       for (int ks = 0; ks < KS; ++ks) {
         const int at = (16 * e + l16) * SP + 32 * ks + 8 * lq;
         const dc_bf16x8 sh = *reinterpret_cast<const dc_bf16x8 *>(St[0] + at), sl = *reinterpret_cast<const dc_bf16x8 *>(St[1] + at);
-        x = mma(wh[ks], sh, x);
-        x2 = mma(wh[ks], sl, x2);
-        x3 = mma(wl[ks], sh, x3);
-        O[e] = mma(q[ks], sh, O[e]);
+        x = mma(c.wh[ks], sh, x);
+        x2 = mma(c.wh[ks], sl, x2);
+        x3 = mma(c.wl[ks], sh, x3);
+        O[e] = mma(c.q[ks], sh, O[e]);
       }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) x[r] = u[e][r] - (x[r] + (x2[r] + x3[r]));
+      for (int r = 0; r < 4; ++r) x[r] = c.u[e][r] - (x[r] + (x2[r] + x3[r]));
       put(Ut, (16 * e + l16) * UP + paired(16 * wave + 4 * lq), x);
     }
-    request_first(n + 1 < chunks ? n + 1 : n);
+    request_first(n + SETS, c);
     __syncthreads();
     // ---- update and read-out
-    dc_f32x4 w[DT];
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) w[dt][r] = fast_exp(g[dt][r]);
 #pragma unroll
     for (int e = 0; e < EB; ++e) {
       Halves ua[2];
@@ -456,26 +478,38 @@ __global__ void __launch_bounds__(256) k_delta_pass(DeltaArgs a) {
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[dt][e][r] *= w[dt][r];
+        for (int r = 0; r < 4; ++r) S[dt][e][r] *= c.w[dt][r];
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
           Halves kb;
-          kb.hi = kh[dt][ks];
-          kb.lo = kl[dt][ks];
+          kb.hi = c.kh[dt][ks];
+          kb.lo = c.kl[dt][ks];
           S[dt][e] = mma3(kb, ua[ks], S[dt][e]);
         }
       }
-      O[e] = mma(p[0], ua[0].hi, O[e]);
-      if (wave >= 2) O[e] = mma(p[1], ua[1].hi, O[e]);
+      O[e] = mma(c.p[0], ua[0].hi, O[e]);
+      if (wave >= 2) O[e] = mma(c.p[1], ua[1].hi, O[e]);
     }
-    request_second(n + 1 < chunks ? n + 1 : n);
+    request_second(n + SETS, c);
     const int t0 = n * C + 16 * wave + 4 * lq;
 #pragma unroll
     for (int e = 0; e < EB; ++e)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         a.o[((t0 + r < a.S ? (int64_t)b * a.S + t0 + r : (int64_t)a.B * a.S) * z.heads + h) * z.Vp + e0 + 16 * e + l16] = O[e][r];
+  };
+  Operands ops[SETS];
+#pragma unroll
+  for (int i = 0; i < SETS; ++i) {
+    request_first(i, ops[i]);
+    request_second(i, ops[i]);
   }
+  int n = 0;
+  for (; n + SETS <= chunks; n += SETS) {
+#pragma unroll
+    for (int i = 0; i < SETS; ++i) chunk(n + i, ops[i]);
+  }
+  if (SETS > 1 && n < chunks) chunk(n, ops[0]);
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
@@ -510,9 +544,9 @@ template <int D> static int launch_chunks(hipStream_t st, const DeltaArgs &a) {
   else RAI_TRY((launch_chunk_w<D, (D > 128 ? 8 : 4)>(st, a)));
   // 64 columns a block read the operands half as often, 32 make twice as many blocks
   if (D <= 128 && z.Vp % 64 == 0 && heads * (z.Vp / 32) > 2 * kNumCU)
-    hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4)>), dim3(z.heads, z.Vp / 64, a.B), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4), (D > 128 ? 1 : 2)>), dim3(z.heads, z.Vp / 64, a.B), dim3(256), 0, st, a);
   else
-    hipLaunchKernelGGL((k_delta_pass<D, 2>), dim3(z.heads, z.Vp / 32, a.B), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((k_delta_pass<D, 2, (D > 128 ? 1 : 2)>), dim3(z.heads, z.Vp / 32, a.B), dim3(256), 0, st, a);
   return launch_check("delta_pass");
 }
 int launch_delta_chunks(hipStream_t st, const DeltaArgs &a) {

@@ -117,8 +117,8 @@ SIZES = {
     "delta 64 by 128": bm.config([bm.delta(heads=2, kv_heads=2, dim=64, vdim=128, conv=4)], width=256),
     "delta 256": bm.config([bm.delta(heads=2, kv_heads=1, dim=256, vdim=256, conv=4)], width=128),
     "delta 300 by 500": bm.config([bm.delta(heads=2, kv_heads=2, dim=300, vdim=500, conv=2)], width=128),
-    "odd everything": bm.config([bm.attention(heads=3, kv_heads=3, dim=7, vdim=5, dims=6, ff=21), bm.delta(heads=3, kv_heads=1, dim=3, vdim=9, ff=3),
-                                 bm.delta(heads=2, kv_heads=2, dim=5, vdim=6, ff=7)], loop=(0, 2, 2), vocab=77, width=33),
+    "odd everything": bm.config([bm.attention(heads=3, kv_heads=3, dim=7, vdim=5, dims=6, ff=21), bm.delta(heads=3, kv_heads=1, dim=11, vdim=9, ff=3),
+                                 bm.delta(heads=2, kv_heads=2, dim=13, vdim=15, ff=7)], loop=(0, 2, 2), vocab=77, width=33),
     "wide": bm.config([bm.attention(heads=20, kv_heads=4, dim=128, vdim=128, dims=128, scale=0.09, ff=1024),
                        bm.delta(heads=16, kv_heads=8, dim=128, vdim=128, conv=4, ff=1024)], width=2304, loop=(0, 2, 2)),
 }
@@ -126,7 +126,7 @@ SIZES = {
 
 def test_heads_of_one(hip):
     """Unit vectors and norms of a single value are signs: f32 only, a rounding to bf16 could turn one."""
-    cfg = bm.config([bm.delta(heads=4, kv_heads=2, dim=1, vdim=1, ff=7), bm.attention(heads=2, kv_heads=2, dim=2, vdim=1, dims=2)], width=40)
+    cfg = bm.config([bm.delta(heads=4, kv_heads=2, dim=1, vdim=1, ff=7), bm.delta(heads=3, kv_heads=1, dim=3, vdim=2, ff=3), bm.attention(heads=2, kv_heads=2, dim=2, vdim=1, dims=2)], width=40)
     p = bezadra.random_params(cfg, "f32", 22, a_rank=1, g_rank=1)
     dec, ids = bm.build(cfg, p, "f32"), tokens(cfg, 80)
     for portions in ([80], [33, 1], [5]):
