@@ -166,22 +166,53 @@ __device__ __forceinline__ float fast_silu(float y) { return y * __builtin_amdgc
 // kWideTokens tokens, Dk / 8 neighbouring lanes a head.
 constexpr int kWideTokens = 4;
 __global__ void __launch_bounds__(256) k_delta_prep_wide(DeltaArgs a) {
-  struct alignas(16) P8 { uint16_t v[8]; };
+  typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
   const DeltaShape &z = a.s;
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8, b = blockIdx.z, s0 = blockIdx.y * kWideTokens;
   const int kd = z.kv_heads * z.Dk;
   if (c >= z.channels) return;   // whole heads: channels is a multiple of 32, the q and k channels of 2 Dk
   const int pos0 = a.state->pos;
-  P8 x[kWideTokens + 3], w[4];
+  u32x4 x[kWideTokens + 3], wv[4];
 #pragma unroll
   for (int i = 0; i < kWideTokens + 3; ++i) {
     const int t = s0 - 3 + i;   // token of this call, or an earlier one in the ring
-    memset(&x[i], 0, sizeof(P8));
-    if (t >= 0 && t < a.S) x[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.dn + ((int64_t)b * a.S + t) * z.ldn + c);
-    else if (t < 0 && pos0 + t >= 0) x[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.ring + ((int64_t)b * 4 + (pos0 + t) % 4) * z.channels + c);
+    x[i] = u32x4{0u, 0u, 0u, 0u};
+    if (t >= 0 && t < a.S) x[i] = *reinterpret_cast<const u32x4 *>((const uint16_t *)a.dn + ((int64_t)b * a.S + t) * z.ldn + c);
+    else if (t < 0 && pos0 + t >= 0) x[i] = *reinterpret_cast<const u32x4 *>((const uint16_t *)a.ring + ((int64_t)b * 4 + (pos0 + t) % 4) * z.channels + c);
   }
 #pragma unroll
-  for (int i = 0; i < 4; ++i) w[i] = *reinterpret_cast<const P8 *>((const uint16_t *)a.conv + (int64_t)c * 4 + 8 * i);
+  for (int i = 0; i < 4; ++i) wv[i] = *reinterpret_cast<const u32x4 *>((const uint16_t *)a.conv + (int64_t)c * 4 + 8 * i);
+  // one pair of channels after the other: its taps and rows unpacked, its results packed
+  uint32_t o[kWideTokens][4];
+  float sum[kWideTokens];
+#pragma unroll
+  for (int t = 0; t < kWideTokens; ++t) sum[t] = 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    float w[2][4], lo[kWideTokens + 3], hi[kWideTokens + 3];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {   // channel 2 e + m: words 2 m, 2 m + 1 of wv[e]
+      w[0][j] = __uint_as_float(j & 1 ? wv[e][j >> 1] & 0xffff0000u : wv[e][j >> 1] << 16);
+      w[1][j] = __uint_as_float(j & 1 ? wv[e][2 + (j >> 1)] & 0xffff0000u : wv[e][2 + (j >> 1)] << 16);
+    }
+#pragma unroll
+    for (int i = 0; i < kWideTokens + 3; ++i) {
+      lo[i] = __uint_as_float(x[i][e] << 16);
+      hi[i] = __uint_as_float(x[i][e] & 0xffff0000u);
+    }
+#pragma unroll
+    for (int t = 0; t < kWideTokens; ++t) {
+      float v0 = lo[t] * w[0][0], v1 = hi[t] * w[1][0];
+#pragma unroll
+      for (int j = 1; j < 4; ++j) {
+        v0 = fmaf(lo[t + j], w[0][j], v0);
+        v1 = fmaf(hi[t + j], w[1][j], v1);
+      }
+      o[t][e] = pack_bf16x2(fast_silu(v0), fast_silu(v1));
+      const float u = __uint_as_float(o[t][e] << 16), p = __uint_as_float(o[t][e] & 0xffff0000u);
+      sum[t] = fmaf(u, u, fmaf(p, p, sum[t]));
+    }
+  }
   const bool query = c < kd, key = !query && c < 2 * kd;
   const int Dk = z.Dk, unit = c / Dk;
   uint16_t *dst = query ? (uint16_t *)a.q + c : key ? (uint16_t *)a.k + c - kd : (uint16_t *)a.v + c - 2 * kd;
@@ -190,25 +221,10 @@ __global__ void __launch_bounds__(256) k_delta_prep_wide(DeltaArgs a) {
 #pragma unroll
   for (int t = 0; t < kWideTokens; ++t) {
     const int64_t row = (int64_t)b * a.S + s0 + t;
-    float y[8], sum = 0.f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float v = 0.f;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) v = fmaf(bf16_bits_to_f32(x[t + j].v[e]), bf16_bits_to_f32(w[e >> 1].v[4 * (e & 1) + j]), v);
-      y[e] = fast_silu(v);
-    }
-    uint32_t o[4];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      o[e] = pack_bf16x2(y[2 * e], y[2 * e + 1]);
-      const float u = __uint_as_float(o[e] << 16), p = __uint_as_float(o[e] & 0xffff0000u);
-      sum = fmaf(u, u, fmaf(p, p, sum));
-    }
-    if (s0 + t < a.S) *reinterpret_cast<uint4 *>(dst + row * ldd) = make_uint4(o[0], o[1], o[2], o[3]);
+    if (s0 + t < a.S) *reinterpret_cast<uint4 *>(dst + row * ldd) = make_uint4(o[t][0], o[t][1], o[t][2], o[t][3]);
     if (query || key) {
-      sum = group_sum(sum, Dk / 8);
-      if (c % Dk == 0 && s0 + t < a.S) (query ? a.qn : a.kn)[row * z.kv_heads + (query ? unit : unit - z.kv_heads)] = mul / sqrtf(sum + 1e-6f);
+      const float total = group_sum(sum[t], Dk / 8);
+      if (c % Dk == 0 && s0 + t < a.S) (query ? a.qn : a.kn)[row * z.kv_heads + (query ? unit : unit - z.kv_heads)] = mul / sqrtf(total + 1e-6f);
     }
   }
 }

@@ -438,6 +438,11 @@ __global__ void __launch_bounds__(256, 1) k_delta_pass(DeltaArgs a) {
     *reinterpret_cast<dc_u32x2 *>(dst[0] + at) = hi;
     *reinterpret_cast<dc_u32x2 *>(dst[1] + at) = lo;
   };
+  const int64_t ldo = (int64_t)z.heads * z.Vp;
+  float *const o0 = a.o + h * z.Vp + e0 + l16, *const behind = o0 + (int64_t)a.B * a.S * ldo;
+  float *out[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) out[r] = o0 + ((int64_t)b * a.S + 16 * wave + 4 * lq + r) * ldo;
   auto chunk = [&](int n, Operands &c) __attribute__((always_inline)) {
     // ---- the state as an operand
 #pragma unroll
@@ -491,12 +496,14 @@ __global__ void __launch_bounds__(256, 1) k_delta_pass(DeltaArgs a) {
       if (wave >= 2) O[e] = mma(c.p[1], ua[1].hi, O[e]);
     }
     request_second(n + SETS, c);
-    const int t0 = n * C + 16 * wave + 4 * lq;
+    const int left = a.S - n * C - 16 * wave - 4 * lq;
 #pragma unroll
-    for (int e = 0; e < EB; ++e)
+    for (int r = 0; r < 4; ++r) {
+      float *const p = r < left ? out[r] : behind;
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        a.o[((t0 + r < a.S ? (int64_t)b * a.S + t0 + r : (int64_t)a.B * a.S) * z.heads + h) * z.Vp + e0 + 16 * e + l16] = O[e][r];
+      for (int e = 0; e < EB; ++e) p[16 * e] = O[e][r];
+      out[r] += C * ldo;
+    }
   };
   Operands ops[SETS];
 #pragma unroll
