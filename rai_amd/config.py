@@ -93,7 +93,7 @@ def bezadra_layers(c, shapes):
         y = dict(mixer=spec["type"], heads=m["heads"], kv_heads=m["kv_heads"], qk_dim=m["dim"], v_dim=m["vdim"])
         if spec["type"] == "attention":
             rot, scaling = m["rot"], m["rot"].get("scaling")
-            y.update(attn_scale=m["scale"], softcap=m["softcap"], rot_dims=rot["dims"], rot_base=rot["base"])
+            y.update(attn_scale=m["scale"], softcap=m.get("softcap") or 0.0, rot_dims=rot["dims"], rot_base=rot["base"])
             if scaling:
                 y.update(rot_factor=scaling["factor"], rot_low=scaling["low"], rot_high=scaling["high"], rot_original=scaling["original"])
         elif spec["type"] == "channel_delta":
