@@ -6,7 +6,7 @@
 // With L = beta A (strictly lower), U = U0 - W S0 where (1 + L) [U0 | W] = beta [V | K~].
 //   k_delta_chunk  everything that does not depend on the state, all chunks at once: A and P, then U0 and W by forward
 //                  substitution in blocks of 16 rows; the operands of the second kernel leave in MFMA-fragment order
-//   k_delta_pass   chunk after chunk per head and 32 or 64 columns of the state, which stays in accumulation registers
+//   k_delta_pass   chunk after chunk per head and 16 to 64 columns of the state, which stays in accumulation registers
 // exp(G_t - G_s) is never formed over a range that could overflow: block row i refers both factors to R_i, the sum at the
 // end of the block before it, so that each is at most 1 outside the block on the diagonal.  On the diagonal the second
 // factor is at least 1; if it would exceed e^60 there, that block is summed up pair by pair.
@@ -549,8 +549,10 @@ template <int D> static int launch_chunks(hipStream_t st, const DeltaArgs &a) {
   const int64_t heads = (int64_t)z.heads * a.B;
   if (D > 128 || heads * ((a.S + C - 1) / C) <= kNumCU) RAI_TRY((launch_chunk_w<D, 8>(st, a)));
   else RAI_TRY((launch_chunk_w<D, (D > 128 ? 8 : 4)>(st, a)));
-  // 64 columns a block read the operands half as often, 32 make twice as many blocks
-  if (D <= 128 && z.Vp % 64 == 0 && heads * (z.Vp / 32) > 2 * kNumCU)
+  // 64 columns a block read the operands half as often as 32; 16 make the shortest chain while there are CUs to spare
+  if (D <= 128 && heads * (z.Vp / 16) <= kNumCU)
+    hipLaunchKernelGGL((k_delta_pass<D, 1, (D > 128 ? 1 : 2)>), dim3(z.heads, z.Vp / 16, a.B), dim3(256), 0, st, a);
+  else if (D <= 128 && z.Vp % 64 == 0 && heads * (z.Vp / 32) > 2 * kNumCU)
     hipLaunchKernelGGL((k_delta_pass<D, (D > 128 ? 2 : 4), (D > 128 ? 1 : 2)>), dim3(z.heads, z.Vp / 64, a.B), dim3(256), 0, st, a);
   else
     hipLaunchKernelGGL((k_delta_pass<D, 2, (D > 128 ? 1 : 2)>), dim3(z.heads, z.Vp / 32, a.B), dim3(256), 0, st, a);
