@@ -532,16 +532,17 @@ template <typename T> static int launch_tokens_t(hipStream_t st, int dtype, cons
   } else if (wide <= 128) RAI_TRY((launch_prep<T, 1>(st, a)));
   else if (wide <= 256) RAI_TRY((launch_prep<T, 2>(st, a)));
   else RAI_TRY((launch_prep<T, 4>(st, a)));
-  if (!chunked) {
+  if (chunked) {
+    RAI_TRY(launch_delta_chunks(st, a));
+  } else {
     hipLaunchKernelGGL(k_delta_decay<T>, dim3((z.heads * z.Dk + 255) / 256, (a.S + kDeltaChunk - 1) / kDeltaChunk, a.B), block, 0, st, a);
     RAI_TRY(launch_check("delta_decay"));
+    if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
+    else if (z.Dk <= 64) RAI_TRY((launch_scan<T, 4>(st, a)));
+    else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));
+    else if (z.Dk <= 256) RAI_TRY((launch_scan<T, 16>(st, a)));
+    else RAI_TRY((launch_scan<T, 32>(st, a)));
   }
-  if (chunked) RAI_TRY(launch_delta_chunks(st, a));
-  else if (z.Dk <= 32) RAI_TRY((launch_scan<T, 2>(st, a)));
-  else if (z.Dk <= 64) RAI_TRY((launch_scan<T, 4>(st, a)));
-  else if (z.Dk <= 128) RAI_TRY((launch_scan<T, 8>(st, a)));
-  else if (z.Dk <= 256) RAI_TRY((launch_scan<T, 16>(st, a)));
-  else RAI_TRY((launch_scan<T, 32>(st, a)));
   if (sizeof(T) == 2 && pow2(z.Vp) && a.ldo % 8 == 0) {
     hipLaunchKernelGGL(k_delta_out_wide, dim3((unsigned)((outs * (z.Vp / 8) + 255) / 256)), block, 0, st, a);
     return launch_check("delta_out_wide");
