@@ -54,7 +54,6 @@ __device__ __forceinline__ dc_f32x4 mma3(const Halves &a, const Halves &b, dc_f3
   return mma(a.hi, b.hi, c);
 }
 __device__ __forceinline__ float fast_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
-__device__ __forceinline__ dc_bf16x8 zero8() { return __builtin_bit_cast(dc_bf16x8, dc_u32x4{0u, 0u, 0u, 0u}); }
 constexpr int C = kDeltaChunk;
 // One (sequence, chunk, head)'s part of the workspace, in bytes.
 struct ChunkLayout {
@@ -187,7 +186,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
         float ge[8];
         load_pair(Gl + (t0 + 15) * KP + d, ge);
 #pragma unroll
-        for (int y = 0; y < 8; ++y) range = fmaxf(range, R[y] - ge[y]);
+        for (int y = 0; y < 8; ++y) range = d + 16 * (y >> 2) + (y & 3) < z.dim ? fmaxf(range, R[y] - ge[y]) : range;   // padding does not count
       }
       if (i == j) {   // the scaled queries of this row block, on the way
         float x[8];

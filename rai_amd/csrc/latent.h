@@ -77,7 +77,8 @@ int launch_latent_attention(hipStream_t st, int dtype, LatentAttnArgs a);
 // WukT[h][r][d] = Wuk[h * Dp + d][r]
 int launch_latent_transpose_uk(hipStream_t st, int dtype, const void *Wuk, void *WukT, int heads, int Dp, int Rp);
 
-// ---- the single-row bf16 step (latent_decode.hip): launches with norms, routing, append and residual folded in
+// ---- the single-row bf16 step (latent_decode.hip): launches with norms, routing, append and residual folded in.  The
+// hybrid family's step uses the first and the last of them.
 struct LatentInArgs {
   const void *src;              // the stream row, f32 or (first layer) the bf16 embedding row
   int src_f32;
