@@ -141,7 +141,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
     float run = 0.f;
 #pragma unroll
     for (int t = 0; t < RUN; ++t) {
-      if (g0 + t < len) run += rate * softplus_for<bf16_raw>(gr[t] + bias);
+      if (g0 + t < len && gd < z.dim) run += rate * softplus_for<bf16_raw>(gr[t] + bias);   // padding channels do not decay: their factors stay finite
       gr[t] = run;
     }
     Ls[(g0 / RUN) * D + gd] = run;   // not yet used for its blocks
@@ -186,7 +186,7 @@ __global__ void __launch_bounds__(WAVES * 64) k_delta_chunk(DeltaArgs a) {
         float ge[8];
         load_pair(Gl + (t0 + 15) * KP + d, ge);
 #pragma unroll
-        for (int y = 0; y < 8; ++y) range = d + 16 * (y >> 2) + (y & 3) < z.dim ? fmaxf(range, R[y] - ge[y]) : range;   // padding does not count
+        for (int y = 0; y < 8; ++y) range = fmaxf(range, R[y] - ge[y]);
       }
       if (i == j) {   // the scaled queries of this row block, on the way
         float x[8];

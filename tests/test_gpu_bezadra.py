@@ -231,7 +231,7 @@ def test_long_memory(hip, dt, far):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("dim", [32, 64])
+@pytest.mark.parametrize("dim", [32, 48, 64, 100])
 @pytest.mark.parametrize("bias,rate", [(0.5, 1.0), (-12.0, 0.0), (-3.0, 1.5), (4.0, 0.0), (30.0, 3.0), (-60.0, -4.0)])
 def test_decays_from_none_to_all(hip, dt, bias, rate, dim):
     """Channels that forget nothing, that forget everything at once (the decay underflows), and both next to each other."""
